@@ -1113,6 +1113,284 @@ TEFUDRA_PRESETS = {
 }
 
 
+# ---------------------------------------------------------------------------
+# Kikurax: a hybrid decoder on an fp32 residual with pre-norms on equal groups
+# of the width and a routed mixture of clamped experts. A layer carries one of
+# three mixers: an averaged pair (sigmoid-weighted attention beside a gated
+# delta rule), a Mamba-2 scan (one decay per head), or rotary softmax attention
+# with unit-norm q/k, a temperature per head, a score cap, an implicit zero-score
+# sink and values blended with the first blending layer's.
+
+
+@dataclass
+class RotaryScaling:
+    """Wavelength-dependent slowdown of rotary frequencies: waves longer than
+    original / low turn `factor` times slower, waves shorter than original /
+    high keep their frequency, those between get a linear blend."""
+
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+@dataclass
+class SigmoidAttnSpec:
+    """Causal attention with grouped kv heads and no rotation whose weights
+    are sigmoid(q.k * scale + bias_head), not normalised over the keys; q and
+    k are unit-RMS per head, q is further scaled at position p by
+    1 + temp_coef * ln(floor((p + 1) / temp_every) + 1); the attended heads
+    pass an elementwise sigmoid gate."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    temp_coef: float = 0.0
+    temp_every: int = 1
+    kind: str = "sigmoid_attention"
+
+
+@dataclass
+class GatedDeltaSpec:
+    """Gated delta rule with a decay per key channel: S <- diag(g) S,
+    u = beta (v - S^T k), S <- S + k u^T, o = S^T q per head, with unit q/k
+    behind a short convolution. decay_rank / gate_rank: inner sizes of the two
+    low-rank projections (from the tensors' shapes)."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    decay_rank: int = 16
+    gate_rank: int = 16
+    kind: str = "gated_delta"
+
+
+@dataclass
+class Mamba2Spec:
+    """State-space duality: per head one decay exp(-exp(A) dt) on a
+    [state, vdim] memory written with dt * B x^T and read with C; heads share
+    B and C in `groups`; the output is gated, then RMS-normed in
+    `norm_groups` equal parts."""
+
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int = 1
+    kind: str = "mamba2"
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclass
+class UnitRotaryAttnSpec:
+    """Causal softmax attention with biased projections; q and k are rotated
+    and then unit-RMS per head; a temperature per head on the scores, a tanh
+    cap (softcap 0: none), 1 added to the softmax denominator; v_mix: values
+    blended with those of the first blending layer."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot: RotarySpec = None
+    rot_scaling: Optional[RotaryScaling] = None
+    softcap: float = 0.0
+    v_mix: bool = False
+    kind: str = "attention"
+
+
+@dataclass
+class KikuraxLayerSpec:
+    mixer: object     # AveragedPairSpec (of the first two) | Mamba2Spec | UnitRotaryAttnSpec
+    moe: Optional[SoftmaxMoESpec] = None    # None: the layer has no feed-forward
+
+
+@dataclass
+class KikuraxSpec:
+    name: str
+    family: str                   # "kikurax"
+    vocab_size: int
+    hidden_size: int
+    layers: list = field(default_factory=list)
+    rms_eps: float = 1e-6
+    norm_groups: int = 1
+    embedding_scale: float = 1.0
+    max_position_embeddings: int = 1 << 17
+    tied_embeddings: bool = True
+    eos_token_id: int = 2
+    bos_token_id: int = 1
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def first_v_mix(self) -> Optional[int]:
+        """The layer whose values the later blending layers mix in."""
+        for i, ls in enumerate(self.layers):
+            if ls.mixer.kind == "attention" and ls.mixer.v_mix:
+                return i
+        return None
+
+    def param_count(self) -> int:
+        w = self.hidden_size
+        total = self.vocab_size * w + w
+        for ls in self.layers:
+            m = ls.mixer
+            total += w
+            if m.kind == "attention":
+                n = m.heads * m.dim + m.kv_heads * (m.dim + m.vdim)
+                total += n * (w + 1) + m.heads + w * m.heads * m.vdim + int(m.v_mix)
+            elif m.kind == "mamba2":
+                n = m.inner + 2 * m.groups * m.state
+                total += (m.inner + n + m.heads) * w + n * (m.conv + 1)
+                total += 3 * m.heads + m.inner + w * m.inner
+            else:
+                a, r = m.left, m.right
+                n = a.heads * (a.dim + a.vdim) + a.kv_heads * (a.dim + a.vdim)
+                total += n * w + a.heads + w * a.heads * a.vdim + 2 * w
+                n = 2 * r.kv_heads * r.dim + r.heads * r.vdim
+                total += n * (w + r.conv) + r.heads * (w + 1)
+                total += r.decay_rank * (w + r.heads * r.dim) + r.heads * r.dim
+                total += r.gate_rank * (w + r.heads * r.vdim) + r.vdim + w * r.heads * r.vdim
+            if ls.moe:
+                e = ls.moe
+                total += w + e.experts * (3 * w * e.ff + w + 1)
+        return total
+
+
+def kikurax_spec_from_config(cfg: dict, name: str, shapes: Optional[dict] = None) -> KikuraxSpec:
+    """Kikurax config.json -> KikuraxSpec. The inner sizes of the two low-rank
+    projections of the delta rule come from the checkpoint's tensor shapes."""
+    shapes = shapes or {}
+
+    def grouped(mc: dict, i: int):
+        heads = int(mc["heads"])
+        kv = int(mc.get("kv_heads", heads))
+        if heads % kv:
+            raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+        dim = int(mc["dim"])
+        return {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": int(mc.get("vdim", dim))}
+
+    def taps(mc: dict, i: int) -> int:
+        k = int(mc.get("conv", 1))
+        if k < 1:
+            raise ValueError(f"layer {i}: the convolution needs at least one tap")
+        return k
+
+    layers = []
+    for i, lc in enumerate(cfg["layers"]):
+        mc, kind = lc["mixer"], lc["type"]
+        if kind == "parallel":
+            lt, rt = mc["left"], mc["right"]
+            qt = lt.get("q_temp") or {}
+            left = SigmoidAttnSpec(
+                **grouped(lt, i), scale=float(lt.get("scale", int(lt["dim"]) ** -0.5)),
+                temp_coef=float(qt.get("coef", 0.0)), temp_every=int(qt.get("every", 1)))
+            if left.temp_every < 1:
+                raise ValueError(f"layer {i}: q_temp.every must be at least 1")
+            a1 = shapes.get(f"l{i}.mix.right.a1")
+            g1 = shapes.get(f"l{i}.mix.right.g1")
+            right = GatedDeltaSpec(
+                **grouped(rt, i), conv=taps(rt, i),
+                decay_rank=int(a1[0]) if a1 else 16, gate_rank=int(g1[0]) if g1 else 16)
+            mixer = AveragedPairSpec(left=left, right=right)
+        elif kind == "mamba2":
+            mixer = Mamba2Spec(
+                heads=int(mc["heads"]), vdim=int(mc["vdim"]), state=int(mc["state"]),
+                groups=int(mc.get("groups", 1)), conv=taps(mc, i),
+                norm_groups=int(mc.get("norm_groups", 1)))
+            if mixer.heads % mixer.groups:
+                raise ValueError(f"layer {i}: heads must be a multiple of groups")
+            if mixer.inner % mixer.norm_groups:
+                raise ValueError(f"layer {i}: norm_groups must divide heads * vdim")
+        elif kind == "attention":
+            sc = mc["rot"].get("scaling")
+            mixer = UnitRotaryAttnSpec(
+                **grouped(mc, i), scale=float(mc.get("scale", int(mc["dim"]) ** -0.5)),
+                rot=_rotary_from(mc["rot"], int(mc["dim"]), f"layer {i}"),
+                rot_scaling=RotaryScaling(
+                    factor=float(sc["factor"]), low=float(sc["low"]), high=float(sc["high"]),
+                    original=float(sc["original"])) if sc else None,
+                softcap=float(mc.get("softcap") or 0.0), v_mix=bool(mc.get("v_mix", False)))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        mlp, moe = lc.get("mlp"), None
+        if mlp is not None:
+            if mlp.get("kind", "moe") != "moe":
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+            moe = SoftmaxMoESpec(
+                experts=int(mlp["router"]["experts"]), top=int(mlp["router"]["top"]),
+                ff=int(mlp["expert"]["ff"]), limit=float(mlp["expert"]["limit"]))
+            if not 1 <= moe.top <= moe.experts:
+                raise ValueError(f"layer {i}: top must be within 1..experts")
+        layers.append(KikuraxLayerSpec(mixer=mixer, moe=moe))
+    spec = KikuraxSpec(
+        name=name, family="kikurax", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+        layers=layers, rms_eps=float(cfg["norm"]["eps"]),
+        norm_groups=int(cfg["norm"].get("groups", 1)),
+        embedding_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)))
+    if spec.hidden_size % spec.norm_groups:
+        raise ValueError("norm.groups must divide the width")
+    sizes = {(ls.mixer.kv_heads, ls.mixer.vdim) for ls in layers
+             if ls.mixer.kind == "attention" and ls.mixer.v_mix}
+    if len(sizes) > 1:
+        raise ValueError("layers that blend values need the same kv_heads and vdim")
+    return spec
+
+
+def _kikurax(name, vocab, width, pattern, heads, kv_heads, dim, vdim, experts, top, ff,
+             left=None, delta=None, ssd=None, conv=4, groups=2, limit=7.0, softcap=50.0,
+             rot_dims=None, rank=None, scaling=(8.0, 1.0, 4.0, 8192.0), **kw):
+    """Preset builder. pattern: one letter per layer, p = averaged pair,
+    m = Mamba-2, a = attention. left (dim, vdim), delta (heads, kv_heads, dim,
+    vdim), ssd (heads, vdim, state, groups, norm_groups)."""
+    layers = []
+    ld, lv = left or (dim, vdim)
+    dh, dg, dd, dv = delta or (heads, heads, dim, vdim)
+    for c in pattern:
+        if c == "p":
+            mixer = AveragedPairSpec(
+                SigmoidAttnSpec(heads, kv_heads, ld, lv, 0.125, 0.3, 512),
+                GatedDeltaSpec(dh, dg, dd, dv, conv, rank or dv, rank or dv))
+        elif c == "m":
+            mh, mv, mn, mg, ng = ssd
+            mixer = Mamba2Spec(mh, mv, mn, mg, conv, ng)
+        else:
+            mixer = UnitRotaryAttnSpec(
+                heads, kv_heads, dim, vdim, dim ** -0.5,
+                RotarySpec(500000.0, rot_dims or dim, "half"), RotaryScaling(*scaling), softcap,
+                v_mix=True)
+        layers.append(KikuraxLayerSpec(mixer, SoftmaxMoESpec(experts, top, ff, limit)))
+    return KikuraxSpec(name=name, family="kikurax", vocab_size=vocab, hidden_size=width,
+                       layers=layers, norm_groups=groups, **kw)
+
+
+KIKURAX_PRESETS = {
+    # CPU/GPU test config: every mixer, grouped heads everywhere, q/k size !=
+    # v size, partial rotation, a scaling range the short contexts reach
+    "tiny-kikurax": _kikurax("tiny-kikurax", 512, 64, "pmapa", 4, 2, 16, 24, 6, 2, 32,
+                             left=(24, 16), delta=(4, 2, 8, 24), ssd=(4, 12, 16, 2, 2), conv=3,
+                             limit=1.5, softcap=20.0, rot_dims=8, rank=12,
+                             scaling=(4.0, 1.0, 4.0, 64.0), embedding_scale=8.0),
+    # benchmark configs at the layer sizes of llama-3.2-1b / -3b and of the
+    # other hybrid presets: same width, head count and depth; the scan is two
+    # model widths wide with 128 states per head; 8 experts, 2 per token
+    "kikurax-1b": _kikurax("kikurax-1b", 128256, 2048, "pmpa" * 4, 32, 8, 64, 64, 8, 2, 2048,
+                           delta=(16, 16, 64, 128), ssd=(64, 64, 128, 8, 8), groups=4),
+    "kikurax-3b": _kikurax("kikurax-3b", 128256, 3072, "pmpa" * 7, 24, 8, 128, 128, 8, 2, 2048,
+                           delta=(12, 12, 128, 256), ssd=(96, 64, 128, 8, 8), groups=4),
+}
+
+
 def spec_from_hf_config(path: Path, name: str) -> ModelSpec:
     """Build a spec from a HF checkpoint directory's config.json."""
     with open(path / "config.json", "r", encoding="utf-8") as fh:
@@ -1123,6 +1401,10 @@ def spec_from_hf_config(path: Path, name: str) -> ModelSpec:
         return muvetar_spec_from_config(cfg, name)
     if str(cfg.get("architecture", "")).lower() == "tefudra":
         return tefudra_spec_from_config(cfg, name)
+    if str(cfg.get("architecture", "")).lower() == "kikurax":
+        st = path / "model.safetensors"
+        return kikurax_spec_from_config(
+            cfg, name, _safetensors_shapes(st) if st.is_file() else None)
     if str(cfg.get("architecture", "")).lower() == "kakovik":
         st = path / "model.safetensors"
         return kakovik_spec_from_config(
@@ -1206,7 +1488,9 @@ def resolve_spec(model: str) -> ModelSpec:
         return MUVETAR_PRESETS[key]
     if key in TEFUDRA_PRESETS:
         return TEFUDRA_PRESETS[key]
+    if key in KIKURAX_PRESETS:
+        return KIKURAX_PRESETS[key]
     raise ValueError(
         f"Unknown model '{model}'. Provide a checkpoint directory with config.json "
-        f"or one of: {sorted(PRESETS) + sorted(HYBRID_PRESETS) + sorted(KOSALORN_PRESETS) + sorted(MUVETAR_PRESETS) + sorted(TEFUDRA_PRESETS) + sorted(ALIASES)}"
+        f"or one of: {sorted(PRESETS) + sorted(HYBRID_PRESETS) + sorted(KOSALORN_PRESETS) + sorted(MUVETAR_PRESETS) + sorted(TEFUDRA_PRESETS) + sorted(KIKURAX_PRESETS) + sorted(ALIASES)}"
     )

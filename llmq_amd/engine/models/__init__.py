@@ -1,6 +1,7 @@
 """Model registry: spec family → model class."""
 
 from llmq_amd.engine.models.kakovik import KakovikLM
+from llmq_amd.engine.models.kikurax import KikuraxLM
 from llmq_amd.engine.models.kosalorn import KosalornLM
 from llmq_amd.engine.models.llama import CausalLM
 from llmq_amd.engine.models.muvetar import MuvetarLM
@@ -12,6 +13,7 @@ MODEL_CLASSES = {
     "gemma2": CausalLM,
     "mistral": CausalLM,
     "kakovik": KakovikLM,
+    "kikurax": KikuraxLM,
     "kosalorn": KosalornLM,
     "muvetar": MuvetarLM,
     "tefudra": TefudraLM,
@@ -25,4 +27,4 @@ def model_class_for(spec):
         raise ValueError(f"no model class registered for family {spec.family!r}") from None
 
 
-__all__ = ["CausalLM", "KakovikLM", "KosalornLM", "MuvetarLM", "TefudraLM", "MODEL_CLASSES", "model_class_for"]
+__all__ = ["CausalLM", "KakovikLM", "KikuraxLM", "KosalornLM", "MuvetarLM", "TefudraLM", "MODEL_CLASSES", "model_class_for"]

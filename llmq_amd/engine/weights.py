@@ -433,5 +433,106 @@ def load_tefudra_weights(model, path: Path) -> None:
     logger.info("loaded %d tensors from %s", len(tensors), path)
 
 
-_FAMILY_LOADERS = {"kakovik": load_kakovik_weights, "kosalorn": load_kosalorn_weights,
-                   "muvetar": load_muvetar_weights, "tefudra": load_tefudra_weights}
+def load_kikurax_weights(model, path: Path) -> None:
+    """Kikurax checkpoint names -> the packed in-tree tensors.
+
+    Checkpoint: 'embed' (also the output head), 'final.norm', and per layer
+    'l<i>.norm1', '.norm2', the mixer under 'l<i>.mix.' (an averaged pair's two
+    mixers under '.left.' and '.right.', their output norms '.left.out' /
+    '.right.out'), the feed-forward under 'l<i>.mlp.' (experts 'e<j>.');
+    linear weights are [out, in], a bias is the weight's name + '.b', a short
+    convolution's taps the weight's name + '.conv'. Packing: everything that
+    reads the mixer's input -> 'in' (biases -> 'in_b', taps -> 'conv_w',
+    segments at multiples of 8 rows), gate‖up -> one tensor, experts stacked
+    [E, ...]; what enters gates and recurrences -> fp32."""
+    tensors = _read_all(path)
+    used = set()
+
+    def get(name: str) -> torch.Tensor:
+        if name not in tensors:
+            raise KeyError(f"missing tensor {name}")
+        used.add(name)
+        return tensors[name]
+
+    def copy_(dst: torch.Tensor, src: torch.Tensor) -> None:
+        if dst.shape != src.shape:
+            raise ValueError(f"shape mismatch: {tuple(dst.shape)} vs {tuple(src.shape)}")
+        dst.copy_(src.to(dst.dtype))
+
+    spec = model.spec
+    copy_(model.embedding, get("embed"))
+    copy_(model.final_norm, get("final.norm"))
+    for i, (ls, lw) in enumerate(zip(spec.layers, model.layers)):
+        p, t, m = f"l{i}.", lw.t, ls.mixer
+        mx = p + "mix."
+        copy_(t["norm1"], get(p + "norm1"))
+
+        def put(seg: str, src: torch.Tensor, dst: str = "in", lw=lw, t=t) -> None:
+            at, n = lw.seg[seg]
+            copy_(t[dst][at:at + n], src)
+
+        for name in ("in", "in_b", "conv_w", "conv_b"):     # alignment rows between segments
+            if name in t:
+                t[name].zero_()
+        if m.kind == "attention":
+            for seg in ("q", "k", "v"):
+                put(seg, get(mx + seg))
+                put(seg, get(mx + seg + ".b"), "in_b")
+            copy_(t["temp"], get(mx + "temp"))
+            if m.v_mix:
+                copy_(t["vmix"], get(mx + "vmix").reshape(()))
+            copy_(t["o"], get(mx + "o"))
+        elif m.kind == "mamba2":
+            bc = m.groups * m.state
+            cuts = [("z", m.inner), ("x", m.inner), ("B", bc), ("C", bc), ("dt", m.heads)]
+            w_in, w_conv, b_conv = get(mx + "in"), get(mx + "conv"), get(mx + "conv.b")
+            if w_in.shape[0] != sum(n for _, n in cuts):
+                raise ValueError(f"{mx}in: expected {sum(n for _, n in cuts)} rows")
+            if w_conv.shape[0] != m.inner + 2 * bc or b_conv.shape[0] != w_conv.shape[0]:
+                raise ValueError(f"{mx}conv: expected {m.inner + 2 * bc} channels")
+            at = 0
+            for seg, n in cuts:
+                put(seg, w_in[at:at + n])
+                at += n
+            at = 0
+            for seg, n in cuts[1:4]:
+                put(seg, w_conv[at:at + n], "conv_w")
+                put(seg, b_conv[at:at + n], "conv_b")
+                at += n
+            for name in ("dt_bias", "A_log", "D", "norm", "o"):
+                copy_(t[name], get(mx + name))
+        else:
+            lf, rt = mx + "left.", mx + "right."
+            for seg in ("q", "k", "v", "g"):
+                put(seg, get(lf + seg))
+            copy_(t["pb"], get(lf + "pb"))
+            copy_(t["o"], get(lf + "o"))
+            copy_(t["left_out"], get(lf + "out"))
+            for name in ("q", "k", "v"):
+                put("d" + name, get(rt + name))
+                put("d" + name, get(rt + name + ".conv"), "conv_w")
+            for seg in ("a1", "g1", "b"):
+                put(seg, get(rt + seg))
+            for name in ("a2", "g2", "dt_bias", "A_log"):
+                copy_(t[name], get(rt + name))
+            copy_(t["d_norm"], get(rt + "norm"))
+            copy_(t["d_o"], get(rt + "o"))
+            copy_(t["right_out"], get(rt + "out"))
+        if ls.moe:
+            copy_(t["norm2"], get(p + "norm2"))
+            copy_(t["router"], get(p + "mlp.router"))
+            copy_(t["router_b"], get(p + "mlp.router.b"))
+            for j in range(ls.moe.experts):
+                ep = f"{p}mlp.e{j}."
+                copy_(t["e_gate_up"][j], torch.cat([get(ep + "gate"), get(ep + "up")], dim=0))
+                copy_(t["e_down"][j], get(ep + "down"))
+    unused = sorted(set(tensors) - used)
+    if unused:
+        logger.warning("checkpoint tensors this configuration does not use: %s", unused[:8])
+    model.finalize()
+    logger.info("loaded %d tensors from %s", len(tensors), path)
+
+
+_FAMILY_LOADERS = {"kakovik": load_kakovik_weights, "kikurax": load_kikurax_weights,
+                   "kosalorn": load_kosalorn_weights, "muvetar": load_muvetar_weights,
+                   "tefudra": load_tefudra_weights}

@@ -453,6 +453,8 @@ _NO_WINDOW = (1 << 31) - 1
 # bias modes: a table [H, n] indexed by the distance i - j, or per head the
 # pair (r1, r2) of a logarithmic distance penalty -r1 * ln(1 + r2 * (i - j))
 _BIAS_TABLE, _BIAS_LOG = 0, 1
+# what turns a score into a weight: softmax over the keys, or a sigmoid per key
+_WEIGHT_SOFTMAX, _WEIGHT_SIGMOID = 0, 1
 
 
 def chunk_bias_attn_prefill(q, gate, k_cache, v_cache, bias, block_tables, cu_q, q_start,
@@ -505,14 +507,16 @@ def gated_recurrence(q, k, v, z, z_bias, state, cu, slots, fresh, tau: float = 1
                                       q_silu, q_scale)
 
 
-def gla_out_norm_gate(o, weight, gate, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
-    """Per-head RMSNorm of the recurrence output × weight × SiLU(gate)."""
+def gla_out_norm_gate(o, weight, gate, eps: float, out_dtype: torch.dtype,
+                      sigmoid: bool = False) -> torch.Tensor:
+    """Per-head RMSNorm of the recurrence output × weight × SiLU(gate), or
+    × sigmoid(gate) with sigmoid."""
     if _use_hybrid(o):
         T, H, DV = o.shape
         out = torch.empty(T, H * DV, dtype=out_dtype, device=o.device)
-        _HY.gla_out_norm_gate(out, o, weight, gate, eps)
+        _HY.gla_out_norm_gate(out, o, weight, gate, eps, bool(sigmoid))
         return out
-    return torch_ref.gla_out_norm_gate(o, weight, gate, eps, out_dtype)
+    return torch_ref.gla_out_norm_gate(o, weight, gate, eps, out_dtype, sigmoid)
 
 
 def head_norm(o, weight, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
@@ -527,28 +531,35 @@ def head_norm(o, weight, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
 
 def window_attn_prefill(q, k_cache, v_cache, dv: int, block_tables, cu_q, q_start, max_q: int,
                         window: int, scale: float, log_bias=None, keep_first: int = 0,
-                        sink=None, softcap: float = 0.0) -> torch.Tensor:
+                        sink=None, softcap: float = 0.0, gate=None, sigmoid: bool = False,
+                        wbias=None) -> torch.Tensor:
     """Softmax attention of packed prompt portions over the paged cache:
     query at position i sees keys j <= i with i - j < window (window 0:
     every j <= i) or j < keep_first. v_cache None: the first dv channels of a
     key row are its value (latent caches). log_bias fp32 [H, 2] = (r1, r2)
     per head: the score loses r1 * ln(1 + r2 * (i - j)). softcap c > 0: the
     scaled score becomes c * tanh(score / c). sink fp32 [H]: the softmax
-    denominator gains exp(sink[h]). q [T, H, D] -> [T, H, dv]."""
+    denominator gains exp(sink[h]). gate [T, H * dv] (or [T, H], one per
+    head): the attended heads are multiplied by sigmoid(gate). sigmoid: a
+    key's weight is sigmoid(score + wbias[h]) on its own (wbias fp32 [H]), not
+    normalised over the keys. q [T, H, D] -> [T, H, dv]."""
     if _use_hybrid(q):
         out = torch.empty(q.shape[0], q.shape[1], dv, dtype=q.dtype, device=q.device)
-        _HY.paged_attn_prefill(out, q, None, k_cache, v_cache, log_bias, block_tables, cu_q,
+        _HY.paged_attn_prefill(out, q, gate, k_cache, v_cache, log_bias, block_tables, cu_q,
                                q_start, int(max_q), int(window) or _NO_WINDOW, float(scale),
                                _MASK_WINDOW, 1, _BIAS_LOG if log_bias is not None else _BIAS_TABLE,
-                               int(keep_first) if window else 0, sink, float(softcap))
+                               int(keep_first) if window else 0, sink, float(softcap),
+                               _WEIGHT_SIGMOID if sigmoid else _WEIGHT_SOFTMAX, wbias)
         return out
     return torch_ref.window_attn_prefill(q, k_cache, v_cache, dv, block_tables, cu_q, q_start,
-                                         window, scale, log_bias, keep_first, sink, softcap)
+                                         window, scale, log_bias, keep_first, sink, softcap, gate,
+                                         sigmoid, wbias)
 
 
 def window_attn_decode(q, k_cache, v_cache, dv: int, block_tables, context_lens, window: int,
                        scale: float, log_bias=None, keep_first: int = 0, sink=None,
-                       softcap: float = 0.0) -> torch.Tensor:
+                       softcap: float = 0.0, gate=None, sigmoid: bool = False,
+                       wbias=None) -> torch.Tensor:
     """The single-token form: query b sits at position context_lens[b]-1."""
     if _use_hybrid(q):
         B, H, D = q.shape
@@ -557,7 +568,7 @@ def window_attn_decode(q, k_cache, v_cache, dv: int, block_tables, context_lens,
         keep = int(keep_first) if window else 0
         if (q.dtype == torch.bfloat16 and k_cache.shape[1] == 1 and H >= 8 and D % 8 == 0
                 and D <= 256 and q.is_contiguous() and log_bias is None and not keep
-                and sink is None and not softcap):
+                and sink is None and not softcap and gate is None and not sigmoid):
             # one kv head for all query heads: the heads of a token become the
             # rows of one head, all at the token's position, and the step runs
             # on the matrix-core kernel — every key tile staged once for all
@@ -568,12 +579,14 @@ def window_attn_decode(q, k_cache, v_cache, dv: int, block_tables, context_lens,
                                    int(window) or _NO_WINDOW, float(scale), _MASK_WINDOW, 0,
                                    _BIAS_TABLE, 0, None, 0.0)
             return out
-        _HY.paged_attn_decode(out, q, None, k_cache, v_cache, log_bias, block_tables,
+        _HY.paged_attn_decode(out, q, gate, k_cache, v_cache, log_bias, block_tables,
                               context_lens, int(window) or _NO_WINDOW, float(scale), _MASK_WINDOW,
-                              bias_mode, keep, sink, float(softcap))
+                              bias_mode, keep, sink, float(softcap),
+                              _WEIGHT_SIGMOID if sigmoid else _WEIGHT_SOFTMAX, wbias)
         return out
     return torch_ref.window_attn_decode(q, k_cache, v_cache, dv, block_tables, context_lens,
-                                        window, scale, log_bias, keep_first, sink, softcap)
+                                        window, scale, log_bias, keep_first, sink, softcap, gate,
+                                        sigmoid, wbias)
 
 
 _HEAD_ROWS = {}
@@ -786,14 +799,15 @@ def embed_sinusoid(embedding, ids, positions, inv_freq) -> torch.Tensor:
 
 
 def scaled_add_norm(res, y, y2, a1: float, a2: float, weight, eps: float,
-                    out_dtype: torch.dtype) -> torch.Tensor:
+                    out_dtype: torch.dtype, groups: int = 1) -> torch.Tensor:
     """res (fp32, in place) += a1 * y [+ a2 * y2]; returns rmsnorm(res) * weight
-    in out_dtype."""
+    in out_dtype. groups > 1: the norm works on that many equal parts of a
+    row."""
     if _use_hybrid(res):
         out = torch.empty(res.shape, dtype=out_dtype, device=res.device)
-        _HY.scaled_add_norm(out, res, y, y2, float(a1), float(a2), weight, float(eps))
+        _HY.scaled_add_norm(out, res, y, y2, float(a1), float(a2), weight, float(eps), int(groups))
         return out
-    return torch_ref.scaled_add_norm(res, y, y2, a1, a2, weight, eps, out_dtype)
+    return torch_ref.scaled_add_norm(res, y, y2, a1, a2, weight, eps, out_dtype, groups)
 
 
 def depth_mix_norm(stack, n: int, coef, y, y2, a1: float, a2: float, weight, eps: float,
@@ -881,20 +895,28 @@ def clamp_swish_mul(x, limit: float) -> torch.Tensor:
 
 
 def qkv_norm_rope_cache(q, k, v, q_w, k_w, inv_freq, rot_dims: int, positions, k_cache, v_cache,
-                        slots, eps: float, v_unit_norm: bool = False, v_inv_freq=None) -> None:
+                        slots, eps: float, v_unit_norm: bool = False, v_inv_freq=None,
+                        qk_unit_norm: bool = False, head_scale=None, temp_coef: float = 0.0,
+                        temp_every: int = 1, v_first=None, mix: float = 0.0) -> None:
     """Per token, between the projections and the attention kernel: optional
-    per-head RMSNorm of q and k (weights q_w / k_w [D]), rotary positions on
-    their first rot_dims channels (q [T, H, D] in place), and the paged-cache
-    scatter of k and of the values — v [T, G, DV], or the keys as they arrive
-    when v is None — which may be divided by their root mean square per head
-    (v_unit_norm) and turned by their position over all channels
-    (v_inv_freq fp32 [DV/2])."""
+    per-head RMSNorm of q and k (weights q_w / k_w [D], or none with
+    qk_unit_norm), rotary positions on their first rot_dims channels (q
+    [T, H, D] in place), and the paged-cache scatter of k and of the values —
+    v [T, G, DV], or the keys as they arrive when v is None — which may be
+    blended with another layer's values of the same tokens
+    ((1 - mix) v + mix v_first), divided by their root mean square per head
+    (v_unit_norm) and turned by their position over all channels (v_inv_freq
+    fp32 [DV/2]). q may carry a factor per head (head_scale fp32 [H]) and one
+    per position p, 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)."""
     if _use_hybrid(q):
         _HY.qkv_norm_rope_cache(q, k, v, q_w, k_w, inv_freq, int(rot_dims), positions, k_cache,
-                                v_cache, slots, float(eps), bool(v_unit_norm), v_inv_freq)
+                                v_cache, slots, float(eps), bool(v_unit_norm), v_inv_freq,
+                                bool(qk_unit_norm), head_scale, float(temp_coef), int(temp_every),
+                                v_first, float(mix))
         return
     torch_ref.qkv_norm_rope_cache(q, k, v, q_w, k_w, inv_freq, rot_dims, positions, k_cache,
-                                  v_cache, slots, eps, v_unit_norm, v_inv_freq)
+                                  v_cache, slots, eps, v_unit_norm, v_inv_freq, qk_unit_norm,
+                                  head_scale, temp_coef, temp_every, v_first, mix)
 
 
 def rotate_heads(x, positions, inv_freq, inverse: bool = False) -> torch.Tensor:
@@ -964,3 +986,51 @@ def unary_act(x, kind: str) -> torch.Tensor:
         _HY.unary_act(out, x, _UNARY_ACTS[kind])
         return out
     return torch_ref.unary_act(x, kind)
+
+
+# ---- gated delta rules and Mamba-2 scans ------------------------------------
+
+
+def gated_delta_rule(q, k, v, z, z_bias, rate, beta, state, cu, slots, fresh,
+                     q_scale: float) -> torch.Tensor:
+    """Gated delta rule over packed sequences, per head h (which reads q/k
+    head h // (H / Hk)): g = exp(-rate_h softplus(z + z_bias)) per key channel,
+    S <- diag(g) S, u = sigmoid(beta) (v - S^T k), S <- S + k u^T,
+    o = S^T (q_scale q), with q and k divided by sqrt(sum of squares + 1e-6).
+    q, k [T, Hk, D]; v [T, H, DV]; z [T, H, D]; beta [T, H]; z_bias fp32
+    [H*D]; rate fp32 [H]; state [slots, H, D, DV] fp32 advanced in place.
+    Returns o [T, H, DV] fp32."""
+    if _use_hybrid(q):
+        o = torch.empty(v.shape, dtype=torch.float32, device=q.device)
+        _HY.gated_delta_rule(o, q, k, v, z, z_bias, rate, beta, state, cu, slots, fresh,
+                             float(q_scale))
+        return o
+    return torch_ref.gated_delta_rule(q, k, v, z, z_bias, rate, beta, state, cu, slots, fresh,
+                                      q_scale)
+
+
+def ssd_scan(x, Bm, Cm, dt, dt_bias, rate, state, cu, slots, fresh) -> torch.Tensor:
+    """Mamba-2 recurrence over packed sequences, per head h (which reads
+    group h // (H / G)): step = softplus(dt + dt_bias),
+    S <- exp(-rate_h step) S + step B x^T, o = S^T C. x [T, H, DV];
+    Bm, Cm [T, G, N]; dt [T, H]; dt_bias, rate fp32 [H]; state
+    [slots, H, N, DV] fp32 advanced in place. Returns o [T, H, DV] fp32."""
+    if _use_hybrid(x):
+        T, H, _ = x.shape
+        gates = torch.empty(2, T, H, dtype=torch.float32, device=x.device)
+        _HY.ssd_gates(gates, dt, dt_bias, rate)
+        o = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+        _HY.matrix_memory(o, Cm, Bm, x, gates[0], gates[1], state, cu, slots, fresh, 1.0, False)
+        return o
+    return torch_ref.ssd_scan(x, Bm, Cm, dt, dt_bias, rate, state, cu, slots, fresh)
+
+
+def ssd_out_gate_norm(o, x, D, z, weight, eps: float, groups: int, out_dtype) -> torch.Tensor:
+    """Read-out of a Mamba-2 scan: (o + D_h x) * silu(z), RMS-normed in
+    `groups` equal parts, times weight. o [T, H, DV] fp32; x, z [T, H*DV];
+    D fp32 [H]; returns [T, H*DV] in out_dtype."""
+    if _use_hybrid(o):
+        out = torch.empty(z.shape, dtype=out_dtype, device=o.device)
+        _HY.ssd_out_gate_norm(out, o, x, D, z, weight, float(eps), int(groups))
+        return out
+    return torch_ref.ssd_out_gate_norm(o, x, D, z, weight, eps, groups, out_dtype)

@@ -7,6 +7,8 @@
 #include <hip/hip_runtime.h>
 #include <torch/library.h>
 
+#include <climits>
+
 namespace {
 
 #define HY_GPU(x) TORCH_CHECK(x.is_cuda(), #x " must be on GPU")
@@ -181,7 +183,7 @@ void qknorm_vmix_cache(at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor q_w,
 
 // v_row: value row stride in elements (DV for a value cache of its own, D
 // when values are the first DV channels of the key rows); vptr: where they sit
-struct AttnDims { int H, G, D, DV, bs, v_row; const void* vptr; const float* bias; int bias_len; };
+struct AttnDims { int H, G, D, DV, bs, v_row; const void* vptr; const float* bias; int bias_len, gate_cols; };
 
 AttnDims attn_check(const at::Tensor& out, const at::Tensor& q, const std::optional<at::Tensor>& gate,
                     const at::Tensor& k_cache, const std::optional<at::Tensor>& v_cache,
@@ -192,7 +194,7 @@ AttnDims attn_check(const at::Tensor& out, const at::Tensor& q, const std::optio
   HY_INNER(q); HY_INNER(out);
   TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous());
   AttnDims a{(int)q.size(1), (int)k_cache.size(1), (int)q.size(2), (int)out.size(2),
-             (int)k_cache.size(2), 0, nullptr, nullptr, 1};
+             (int)k_cache.size(2), 0, nullptr, nullptr, 1, 1};
   TORCH_CHECK(mask_mode == kMaskBlock || mask_mode == kMaskWindow, "unknown mask mode");
   TORCH_CHECK(q.stride(1) == a.D && out.stride(1) == a.DV, "heads must be packed");
   TORCH_CHECK(k_cache.size(3) == a.D, "query and key sizes differ");
@@ -226,8 +228,11 @@ AttnDims attn_check(const at::Tensor& out, const at::Tensor& q, const std::optio
   HY_I32(block_tables);
   TORCH_CHECK(block_tables.dim() == 2);
   if (gate.has_value()) {
-    TORCH_CHECK(gate->dim() == 2 && gate->size(0) == q.size(0) && gate->size(1) == a.H &&
-                gate->stride(1) == 1 && gate->scalar_type() == q.scalar_type(), "gate must be [T, H]");
+    TORCH_CHECK(gate->dim() == 2 && gate->size(0) == q.size(0) && gate->is_cuda() &&
+                (gate->size(1) == a.H || gate->size(1) == (long)a.H * a.DV) &&
+                gate->stride(1) == 1 && gate->scalar_type() == q.scalar_type(),
+                "gate must be [T, H] or [T, H * DV]");
+    a.gate_cols = gate->size(1) == a.H ? 1 : a.DV;
   }
   return a;
 }
@@ -238,6 +243,18 @@ const float* sink_check(const std::optional<at::Tensor>& sink, const at::Tensor&
   TORCH_CHECK(sink->is_cuda() && sink->scalar_type() == at::kFloat && sink->is_contiguous() &&
               sink->numel() == q.size(1), "sink must be fp32 [H] on the GPU");
   return sink->data_ptr<float>();
+}
+
+// sigmoid weights: the number per query head added to the score, fp32 [H], or none
+const float* wbias_check(int64_t weight_fn, const std::optional<at::Tensor>& wbias,
+                         const std::optional<at::Tensor>& sink, const at::Tensor& q) {
+  TORCH_CHECK(weight_fn == kWeightSoftmax || weight_fn == kWeightSigmoid, "unknown weight function");
+  TORCH_CHECK(weight_fn == kWeightSoftmax || !sink.has_value(), "sigmoid weights have no denominator");
+  if (!wbias.has_value()) return nullptr;
+  TORCH_CHECK(weight_fn == kWeightSigmoid, "a weight bias goes with sigmoid weights");
+  TORCH_CHECK(wbias->is_cuda() && wbias->scalar_type() == at::kFloat && wbias->is_contiguous() &&
+              wbias->numel() == q.size(1), "weight bias must be fp32 [H] on the GPU");
+  return wbias->data_ptr<float>();
 }
 
 template <typename F>
@@ -253,9 +270,13 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
                         const std::optional<at::Tensor>& bias, at::Tensor block_tables,
                         at::Tensor cu_q, at::Tensor q_start, int64_t max_q, int64_t span,
                         double scale, int64_t mask_mode, int64_t pos_stride, int64_t bias_mode,
-                        int64_t keep_first, const std::optional<at::Tensor>& sink, double softcap) {
+                        int64_t keep_first, const std::optional<at::Tensor>& sink, double softcap,
+                        int64_t weight_fn, const std::optional<at::Tensor>& wbias) {
   if (q.size(0) == 0) return;
   const float* sink_ptr = sink_check(sink, q);
+  const float* wbias_ptr = wbias_check(weight_fn, wbias, sink, q);
+  TORCH_CHECK(pos_stride == 1 || weight_fn == kWeightSoftmax,
+              "rows that share a position take softmax weights");
   TORCH_CHECK(keep_first >= 0 && softcap >= 0.0);
   TORCH_CHECK(keep_first == 0 || mask_mode == kMaskWindow, "kept first tokens go with the window mask");
   TORCH_CHECK(pos_stride == 1 || (keep_first == 0 && !sink_ptr),
@@ -293,12 +314,12 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
     }
     const dim3 grid((max_q + kMfmaQT - 1) / kMfmaQT, a.H * n_split, B);
     using bf = __hip_bfloat16;
-    auto launch = [&]<int KS, int DT>() {
+    auto launch_as = [&]<int KS, int DT, bool SIG>() {
       // K tile, V^T tile (the channel tiles in use), P hi/lo per wave, bias slice
       const size_t lds = sizeof(short) * ((size_t)kMfmaKT * (ksn * 32 + 8) +
                                           (size_t)dtn * 16 * kMfmaKP +
                                           (size_t)4 * 2 * 16 * kMfmaKP) + 128 * sizeof(float);
-      auto kern = chunk_bias_attn_prefill_mfma_kernel<KS, DT>;
+      auto kern = chunk_bias_attn_prefill_mfma_kernel<KS, DT, SIG>;
       allow_lds(kern, lds);
       hipLaunchKernelGGL(kern, grid, dim3(256), lds, hy_stream(),
                          reinterpret_cast<bf*>(out.data_ptr()), out.stride(0),
@@ -311,7 +332,11 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
                          cu_q.data_ptr<int>(), q_start.data_ptr<int>(), a.H, a.G, a.D, a.DV, a.bs,
                          (int)span, (float)scale, a.v_row, (int)mask_mode, (int)pos_stride,
                          n_split, n_split > 1 ? part.data_ptr<float>() : nullptr, (int)bias_mode,
-                         (int)keep_first, sink_ptr, (float)softcap);
+                         (int)keep_first, sink_ptr, (float)softcap, a.gate_cols, wbias_ptr);
+    };
+    auto launch = [&]<int KS, int DT>() {
+      if (weight_fn == kWeightSigmoid) launch_as.template operator()<KS, DT, true>();
+      else launch_as.template operator()<KS, DT, false>();
     };
     if (ksn <= 2 && dtn <= 4) launch.template operator()<2, 4>();
     else if (ksn <= 4 && dtn <= 8) launch.template operator()<4, 8>();
@@ -343,7 +368,8 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
                          block_tables.data_ptr<int>(), (int)block_tables.stride(0),
                          cu_q.data_ptr<int>(), q_start.data_ptr<int>(), a.H, a.G, a.D, a.DV, a.bs,
                          (int)span, (float)scale, a.v_row, (int)mask_mode, (int)bias_mode,
-                         (int)keep_first, sink_ptr, (float)softcap);
+                         (int)keep_first, sink_ptr, (float)softcap, a.gate_cols, (int)weight_fn,
+                         wbias_ptr);
     });
   });
 }
@@ -353,9 +379,10 @@ void paged_attn_decode(at::Tensor out, at::Tensor q, const std::optional<at::Ten
                        const std::optional<at::Tensor>& bias, at::Tensor block_tables,
                        at::Tensor context_lens, int64_t span, double scale, int64_t mask_mode,
                        int64_t bias_mode, int64_t keep_first, const std::optional<at::Tensor>& sink,
-                       double softcap) {
+                       double softcap, int64_t weight_fn, const std::optional<at::Tensor>& wbias) {
   if (q.size(0) == 0) return;
   const float* sink_ptr = sink_check(sink, q);
+  const float* wbias_ptr = wbias_check(weight_fn, wbias, sink, q);
   TORCH_CHECK(keep_first >= 0 && softcap >= 0.0);
   TORCH_CHECK(keep_first == 0 || mask_mode == kMaskWindow, "kept first tokens go with the window mask");
   const AttnDims a = attn_check(out, q, gate, k_cache, v_cache, bias, block_tables, span, mask_mode,
@@ -387,7 +414,7 @@ void paged_attn_decode(at::Tensor out, at::Tensor q, const std::optional<at::Ten
                          block_tables.data_ptr<int>(), (int)block_tables.stride(0),
                          context_lens.data_ptr<int>(), a.H, a.G, a.D, a.DV, a.bs, (int)span,
                          (float)scale, a.v_row, (int)mask_mode, (int)bias_mode, (int)keep_first,
-                         sink_ptr, (float)softcap);
+                         sink_ptr, (float)softcap, a.gate_cols, (int)weight_fn, wbias_ptr);
       };
       if (hpw == 8) launch.template operator()<8>();
       else if (hpw == 4) launch.template operator()<4>();
@@ -450,7 +477,7 @@ void gla_recurrence(at::Tensor o, at::Tensor q, const std::optional<at::Tensor>&
                          z_bias.data_ptr<float>(), state.data_ptr<float>(), cu.data_ptr<int>(),
                          slots.data_ptr<int>(), fresh.data_ptr<int>(), H, D, DV,
                          (float)(1.0 / tau), q_scale, lower_ptr, (int)q_silu,
-                         static_cast<const float*>(nullptr), static_cast<const float*>(nullptr), 0);
+                         static_cast<const float*>(nullptr), static_cast<const float*>(nullptr), 1, 0);
     };
     if (D <= 32) launch.template operator()<2>();
     else if (D <= 64) launch.template operator()<4>();
@@ -460,7 +487,7 @@ void gla_recurrence(at::Tensor o, at::Tensor q, const std::optional<at::Tensor>&
 }
 
 void gla_out_norm_gate(at::Tensor out, at::Tensor o, at::Tensor weight,
-                       const std::optional<at::Tensor>& gate_opt, double eps) {
+                       const std::optional<at::Tensor>& gate_opt, double eps, bool gate_sigmoid) {
   HY_GPU(o);
   TORCH_CHECK(o.dim() == 3 && o.scalar_type() == at::kFloat && o.is_contiguous());
   const long T_ = o.size(0);
@@ -482,7 +509,8 @@ void gla_out_norm_gate(at::Tensor out, at::Tensor o, at::Tensor weight,
     hipLaunchKernelGGL(gla_out_norm_gate_kernel<T>, dim3(T_), dim3(256), 0, hy_stream(),
                        reinterpret_cast<T*>(out.data_ptr()), out.stride(0), o.data_ptr<float>(),
                        reinterpret_cast<const T*>(weight.data_ptr()),
-                       reinterpret_cast<const T*>(gate_ptr), gate_stride, H, DV, (float)eps);
+                       reinterpret_cast<const T*>(gate_ptr), gate_stride, H, DV, (float)eps,
+                       (int)gate_sigmoid);
   });
 }
 
@@ -790,14 +818,17 @@ void embed_sinusoid(at::Tensor out, at::Tensor embedding, at::Tensor ids, at::Te
 }
 
 void scaled_add_norm(at::Tensor out, at::Tensor res, at::Tensor y, const std::optional<at::Tensor>& y2,
-                     double a1, double a2, at::Tensor weight, double eps) {
+                     double a1, double a2, at::Tensor weight, double eps, int64_t groups_arg) {
   HY_GPU(y);
   HY_F32(res);
   TORCH_CHECK(y.dim() == 2 && y.is_contiguous() && out.is_contiguous() && weight.is_contiguous());
-  const long rows = y.size(0);
-  const int W = y.size(1);
+  const int groups = (int)groups_arg;
+  TORCH_CHECK(groups >= 1 && y.size(1) % groups == 0, "groups must divide the row");
+  // a row normed in groups is `groups` rows to the kernel
+  const int W = y.size(1) / groups;
+  const long rows = y.size(0) * groups;
   if (rows == 0) return;
-  TORCH_CHECK(res.sizes() == y.sizes() && out.sizes() == y.sizes() && weight.numel() == W);
+  TORCH_CHECK(res.sizes() == y.sizes() && out.sizes() == y.sizes() && weight.numel() == y.size(1));
   TORCH_CHECK(out.scalar_type() == y.scalar_type() && weight.scalar_type() == y.scalar_type());
   const void* y2p = nullptr;
   if (y2.has_value()) {
@@ -807,16 +838,19 @@ void scaled_add_norm(at::Tensor out, at::Tensor res, at::Tensor y, const std::op
   }
   if (y.scalar_type() == at::kBFloat16 && W % 8 == 0 && W <= 4 * 2048) {
     using bf = __hip_bfloat16;
-    auto launch = [&]<int CH>() {
-      hipLaunchKernelGGL(scaled_add_norm_vec_kernel<CH>, dim3(rows), dim3(256), 0, hy_stream(),
+    auto launch = [&]<int CH, bool PER_WAVE>() {
+      hipLaunchKernelGGL((scaled_add_norm_vec_kernel<CH, PER_WAVE>),
+                         dim3(PER_WAVE ? (rows + 3) / 4 : rows), dim3(256), 0, hy_stream(),
                          reinterpret_cast<bf*>(out.data_ptr()), res.data_ptr<float>(),
                          reinterpret_cast<const bf*>(y.data_ptr()), reinterpret_cast<const bf*>(y2p),
                          (float)a1, (float)a2, reinterpret_cast<const bf*>(weight.data_ptr()), W,
-                         (float)eps);
+                         (float)eps, groups, rows);
     };
-    if (W <= 2048) launch.template operator()<1>();
-    else if (W <= 4096) launch.template operator()<2>();
-    else launch.template operator()<4>();
+    if (W <= 512) launch.template operator()<1, true>();
+    else if (W <= 1024) launch.template operator()<2, true>();
+    else if (W <= 2048) launch.template operator()<1, false>();
+    else if (W <= 4096) launch.template operator()<2, false>();
+    else launch.template operator()<4, false>();
     return;
   }
   hy_dispatch(y, "scaled_add_norm", [&]<typename T>() {
@@ -824,7 +858,7 @@ void scaled_add_norm(at::Tensor out, at::Tensor res, at::Tensor y, const std::op
                        reinterpret_cast<T*>(out.data_ptr()), res.data_ptr<float>(),
                        reinterpret_cast<const T*>(y.data_ptr()), reinterpret_cast<const T*>(y2p),
                        (float)a1, (float)a2, reinterpret_cast<const T*>(weight.data_ptr()), W,
-                       (float)eps);
+                       (float)eps, groups);
   });
 }
 
@@ -1113,7 +1147,9 @@ void qkv_norm_rope_cache(at::Tensor q, at::Tensor k, const std::optional<at::Ten
                          const std::optional<at::Tensor>& inv_freq, int64_t rot_dims,
                          at::Tensor positions, at::Tensor k_cache, at::Tensor v_cache,
                          at::Tensor slots, double eps, bool v_unit_norm,
-                         const std::optional<at::Tensor>& v_inv_freq) {
+                         const std::optional<at::Tensor>& v_inv_freq, bool qk_unit_norm,
+                         const std::optional<at::Tensor>& head_scale, double temp_coef,
+                         int64_t temp_every, const std::optional<at::Tensor>& v_first, double mix) {
   HY_GPU(q);
   const long T_ = q.size(0);
   if (T_ == 0) return;
@@ -1161,6 +1197,24 @@ void qkv_norm_rope_cache(at::Tensor q, at::Tensor k, const std::optional<at::Ten
     TORCH_CHECK(DV % 2 == 0, "rotated values need an even size");
     v_table = table_ptr(v_inv_freq, DV);
   }
+  TORCH_CHECK(!qk_unit_norm || (!qw && !kw), "a weightless norm or weights, not both");
+  TORCH_CHECK(temp_every >= 1 && temp_every <= INT_MAX);
+  const float* hs_ptr = nullptr;
+  if (head_scale.has_value()) {
+    TORCH_CHECK(head_scale->is_cuda() && head_scale->scalar_type() == at::kFloat &&
+                head_scale->is_contiguous() && head_scale->numel() == H, "head_scale must be fp32 [H]");
+    hs_ptr = head_scale->data_ptr<float>();
+  }
+  const void* vf_ptr = nullptr;
+  long vf_stride = 0;
+  if (v_first.has_value()) {
+    TORCH_CHECK(v_ptr != nullptr && v_first->dim() == 3 && v_first->size(0) == T_ &&
+                v_first->size(1) == G && v_first->size(2) == DV && v_first->stride(1) == DV &&
+                v_first->stride(2) == 1 && v_first->scalar_type() == dt && v_first->is_cuda(),
+                "v_first must be [T, G, DV] like v");
+    vf_ptr = v_first->data_ptr();
+    vf_stride = v_first->stride(0);
+  }
   // lanes per head vector: the fewest that hold its pairs and unrotated channels
   const int max_half = std::max<int>(rot_dims / 2, v_table ? DV / 2 : 0);
   const int max_tail = std::max<int>(D - rot_dims, (v_opt.has_value() && !v_table) ? DV : 0);
@@ -1170,7 +1224,8 @@ void qkv_norm_rope_cache(at::Tensor q, at::Tensor k, const std::optional<at::Ten
   const bool vec = dt == at::kBFloat16 && D % 8 == 0 && DV % 8 == 0 && rot_dims % 16 == 0 &&
                    (!v_table || DV % 16 == 0) && q.stride(0) % 8 == 0 && k.stride(0) % 8 == 0 &&
                    v_stride % 8 == 0 && aligned(q.data_ptr()) && aligned(k.data_ptr()) &&
-                   aligned(v_ptr) && aligned(qw) && aligned(kw);
+                   aligned(v_ptr) && aligned(qw) && aligned(kw) && aligned(vf_ptr) &&
+                   vf_stride % 8 == 0;
   const int per_pair = vec ? 8 : kRopePairs, per_tail = vec ? 8 : kRopeTail;
   int LG = vec ? 1 : 8;
   while (LG < 64 && (max_half > LG * per_pair || max_tail > LG * per_tail)) LG *= 2;
@@ -1190,7 +1245,9 @@ void qkv_norm_rope_cache(at::Tensor q, at::Tensor k, const std::optional<at::Ten
                        (int)rot_dims, v_table, positions.data_ptr<long>(),
                        reinterpret_cast<T*>(k_cache.data_ptr()),
                        reinterpret_cast<T*>(v_cache.data_ptr()), slots.data_ptr<long>(), H, G, D, DV,
-                       bs, (float)eps, (int)v_unit_norm, LG);
+                       bs, (float)eps, (int)v_unit_norm, LG, (int)qk_unit_norm, hs_ptr,
+                       (float)temp_coef, (int)temp_every, reinterpret_cast<const T*>(vf_ptr),
+                       vf_stride, (float)mix);
   };
   if (vec) launch.template operator()<__hip_bfloat16, true>();
   else hy_dispatch(q, "qkv_norm_rope_cache", [&]<typename T>() { launch.template operator()<T, false>(); });
@@ -1231,19 +1288,21 @@ void mlstm_gates(at::Tensor out, at::Tensor gates, double cap, at::Tensor m_stat
                      fresh.data_ptr<int>(), H, T_);
 }
 
-// The recurrence kernel in its scalar-gate mode: q, k [T, H, D], v [T, H, DV]
-// (row-strided views, heads packed); decay, write fp32 [T, H]; o fp32
-// [T, H, DV + 1]; state fp32 [slots, H, D, DV + 1].
+// The recurrence kernel in its scalar-gate mode: q, k [T, Hk, D] (H a multiple
+// of Hk), v [T, H, DVin] (row-strided views, heads packed); decay, write fp32
+// [T, H]; o fp32 [T, H, DV]; state fp32 [slots, H, D, DV]; DV = DVin, or
+// DVin + 1 with the column of ones.
 void matrix_memory(at::Tensor o, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor decay,
                    at::Tensor write, at::Tensor state, at::Tensor cu, at::Tensor slots,
-                   at::Tensor fresh, double q_scale) {
+                   at::Tensor fresh, double q_scale, bool ones_col) {
   HY_GPU(q);
   const long T_ = q.size(0);
   if (T_ == 0) return;
   TORCH_CHECK(q.dim() == 3 && k.sizes() == q.sizes() && v.dim() == 3);
   HY_INNER(q); HY_INNER(k); HY_INNER(v);
-  const int H = q.size(1), D = q.size(2), DVin = v.size(2), DV = DVin + 1;
-  TORCH_CHECK(v.size(0) == T_ && v.size(1) == H);
+  const int Hk = q.size(1), H = v.size(1), D = q.size(2), DVin = v.size(2);
+  const int DV = DVin + (ones_col ? 1 : 0);
+  TORCH_CHECK(v.size(0) == T_ && Hk >= 1 && H % Hk == 0, "heads must be a multiple of the q/k heads");
   TORCH_CHECK(q.stride(1) == D && k.stride(1) == D && v.stride(1) == DVin, "heads must be packed");
   HY_F32(decay); HY_F32(write);
   TORCH_CHECK(decay.dim() == 2 && decay.size(0) == T_ && decay.size(1) == H &&
@@ -1252,7 +1311,7 @@ void matrix_memory(at::Tensor o, at::Tensor q, at::Tensor k, at::Tensor v, at::T
               o.size(0) == T_ && o.size(1) == H && o.size(2) == DV);
   const SeqDims sd = seq_check(cu, slots, fresh, state);
   TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D && state.size(3) == DV,
-              "state [slots, H, D, DV + 1] fp32");
+              "state [slots, H, D, DV] fp32");
   TORCH_CHECK(D <= 256, "key size above 256 is not supported");
   const auto dt = q.scalar_type();
   TORCH_CHECK(k.scalar_type() == dt && v.scalar_type() == dt);
@@ -1268,7 +1327,7 @@ void matrix_memory(at::Tensor o, at::Tensor q, at::Tensor k, at::Tensor v, at::T
                          state.data_ptr<float>(), cu.data_ptr<int>(), slots.data_ptr<int>(),
                          fresh.data_ptr<int>(), H, D, DV, 1.0f, (float)q_scale,
                          static_cast<const float*>(nullptr), 0, decay.data_ptr<float>(),
-                         write.data_ptr<float>(), 1);
+                         write.data_ptr<float>(), H / Hk, (int)ones_col);
     };
     if (D <= 32) launch.template operator()<2>();
     else if (D <= 64) launch.template operator()<4>();
@@ -1354,6 +1413,123 @@ void unary_act(at::Tensor out, at::Tensor in, int64_t act) {
   });
 }
 
+// ---- gated delta rule and Mamba-2 gates / read-out ---------------------------
+
+// q, k [T, Hk, D], v [T, H, DV], z [T, H, D]: row-strided views, heads packed;
+// beta [T, H] row-strided; z_bias fp32 [H*D]; rate fp32 [H] (> 0); o fp32
+// [T, H, DV]; state fp32 [slots, H, D, DV].
+void gated_delta_rule(at::Tensor o, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor z,
+                      at::Tensor z_bias, at::Tensor rate, at::Tensor beta, at::Tensor state,
+                      at::Tensor cu, at::Tensor slots, at::Tensor fresh, double q_scale) {
+  HY_GPU(q);
+  const long T_ = q.size(0);
+  if (T_ == 0) return;
+  TORCH_CHECK(q.dim() == 3 && k.sizes() == q.sizes() && v.dim() == 3 && z.dim() == 3 && beta.dim() == 2);
+  HY_INNER(q); HY_INNER(k); HY_INNER(v); HY_INNER(z); HY_INNER(beta);
+  const int Hk = q.size(1), D = q.size(2), H = v.size(1), DV = v.size(2);
+  TORCH_CHECK(Hk >= 1 && H % Hk == 0, "heads must be a multiple of the q/k heads");
+  TORCH_CHECK(v.size(0) == T_ && z.size(0) == T_ && z.size(1) == H && z.size(2) == D &&
+              beta.size(0) == T_ && beta.size(1) == H);
+  TORCH_CHECK(q.stride(1) == D && k.stride(1) == D && v.stride(1) == DV && z.stride(1) == D,
+              "heads must be packed");
+  HY_F32(z_bias); HY_F32(rate);
+  TORCH_CHECK(z_bias.numel() == (long)H * D && rate.numel() == H);
+  TORCH_CHECK(o.scalar_type() == at::kFloat && o.is_contiguous() && o.dim() == 3 && o.size(0) == T_ &&
+              o.size(1) == H && o.size(2) == DV);
+  const SeqDims sd = seq_check(cu, slots, fresh, state);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D && state.size(3) == DV,
+              "state [slots, H, D, DV] fp32");
+  TORCH_CHECK(D >= 1 && D <= 256, "key size above 256 is not supported");
+  const auto dt = q.scalar_type();
+  TORCH_CHECK(k.scalar_type() == dt && v.scalar_type() == dt && z.scalar_type() == dt &&
+              beta.scalar_type() == dt);
+  // 4 value columns per thread while that still fills the chip, else 1
+  const long wide = (long)((DV + 63) / 64) * H * sd.B;
+  hy_dispatch(q, "gated_delta_rule", [&]<typename T>() {
+    auto launch = [&]<int DPL, int NC>() {
+      const dim3 grid((DV + 16 * NC - 1) / (16 * NC), H, sd.B);
+      hipLaunchKernelGGL((gated_delta_kernel<T, DPL, NC>), grid, dim3(256), 0, hy_stream(),
+                         o.data_ptr<float>(), reinterpret_cast<const T*>(q.data_ptr()), q.stride(0),
+                         reinterpret_cast<const T*>(k.data_ptr()), k.stride(0),
+                         reinterpret_cast<const T*>(v.data_ptr()), v.stride(0),
+                         reinterpret_cast<const T*>(z.data_ptr()), z.stride(0),
+                         z_bias.data_ptr<float>(), rate.data_ptr<float>(),
+                         reinterpret_cast<const T*>(beta.data_ptr()), beta.stride(0),
+                         state.data_ptr<float>(), cu.data_ptr<int>(), slots.data_ptr<int>(),
+                         fresh.data_ptr<int>(), H, H / Hk, D, DV, (float)q_scale);
+    };
+    auto by_d = [&]<int NC>() {
+      if (D <= 32) launch.template operator()<2, NC>();
+      else if (D <= 64) launch.template operator()<4, NC>();
+      else if (D <= 128) launch.template operator()<8, NC>();
+      else launch.template operator()<16, NC>();
+    };
+    if (wide >= 256) by_d.template operator()<4>();
+    else by_d.template operator()<1>();
+  });
+}
+
+// dt [T, H] row-strided in the model dtype -> out fp32 [2, T, H] (decay, write)
+void ssd_gates(at::Tensor out, at::Tensor dt, at::Tensor dt_bias, at::Tensor rate) {
+  HY_GPU(dt);
+  HY_INNER(dt);
+  TORCH_CHECK(dt.dim() == 2);
+  const long T_ = dt.size(0);
+  const int H = dt.size(1);
+  if (T_ == 0) return;
+  HY_F32(out); HY_F32(dt_bias); HY_F32(rate);
+  TORCH_CHECK(out.dim() == 3 && out.size(0) == 2 && out.size(1) == T_ && out.size(2) == H);
+  TORCH_CHECK(dt_bias.numel() == H && rate.numel() == H);
+  const int grid = (int)std::min<long>((T_ * H + 255) / 256, 4096);
+  hy_dispatch(dt, "ssd_gates", [&]<typename T>() {
+    hipLaunchKernelGGL(ssd_gates_kernel<T>, dim3(grid), dim3(256), 0, hy_stream(), out.data_ptr<float>(),
+                       reinterpret_cast<const T*>(dt.data_ptr()), dt.stride(0),
+                       dt_bias.data_ptr<float>(), rate.data_ptr<float>(), T_, H);
+  });
+}
+
+// o fp32 [T, H, DV]; x, z [T, H*DV] row-strided; D fp32 [H]; weight [H*DV]
+void ssd_out_gate_norm(at::Tensor out, at::Tensor o, at::Tensor x, at::Tensor D, at::Tensor z,
+                       at::Tensor weight, double eps, int64_t groups) {
+  HY_GPU(o);
+  HY_F32(o); HY_F32(D);
+  TORCH_CHECK(o.dim() == 3);
+  const long T_ = o.size(0);
+  const int H = o.size(1), DV = o.size(2);
+  const long inner = (long)H * DV;
+  if (T_ == 0) return;
+  HY_INNER(x); HY_INNER(z);
+  TORCH_CHECK(out.dim() == 2 && out.is_contiguous() && out.size(0) == T_ && out.size(1) == inner);
+  TORCH_CHECK(x.dim() == 2 && x.size(0) == T_ && x.size(1) == inner && z.sizes() == x.sizes());
+  const auto dt = out.scalar_type();
+  TORCH_CHECK(x.scalar_type() == dt && z.scalar_type() == dt && weight.scalar_type() == dt &&
+              weight.is_contiguous() && weight.numel() == inner && D.numel() == H);
+  TORCH_CHECK(groups >= 1 && inner % groups == 0, "groups must divide the row");
+  const int width = (int)(inner / groups);
+  const long rows = T_ * groups;
+  auto aligned = [](const at::Tensor& t) { return reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0; };
+  const bool vec = DV % 4 == 0 && width % 4 == 0 && x.stride(0) % 4 == 0 && z.stride(0) % 4 == 0 &&
+                   aligned(x) && aligned(z) && aligned(o) && aligned(out) && aligned(weight);
+  hy_dispatch(out, "ssd_out_gate_norm", [&]<typename T>() {
+    auto launch = [&]<int TEAM, int V>() {
+      const long blocks = TEAM == 64 ? (rows + 3) / 4 : rows;
+      hipLaunchKernelGGL((ssd_out_gate_norm_kernel<T, TEAM, V>), dim3(blocks), dim3(256), 0, hy_stream(),
+                         reinterpret_cast<T*>(out.data_ptr()), o.data_ptr<float>(),
+                         reinterpret_cast<const T*>(x.data_ptr()), x.stride(0), D.data_ptr<float>(),
+                         reinterpret_cast<const T*>(z.data_ptr()), z.stride(0),
+                         reinterpret_cast<const T*>(weight.data_ptr()), width, (int)groups, rows, DV,
+                         (float)eps);
+    };
+    if (vec) {
+      if (width <= 1024) launch.template operator()<64, 4>();
+      else launch.template operator()<256, 4>();
+    } else {
+      if (width <= 256) launch.template operator()<64, 1>();
+      else launch.template operator()<256, 1>();
+    }
+  });
+}
+
 }  // namespace
 
 
@@ -1362,10 +1538,10 @@ TORCH_LIBRARY(llmq_amd_hybrid, m) {
   m.def("sandwich_norm_res32(Tensor(a!) x, Tensor(b!) residual, Tensor w_post, Tensor w_pre, float eps, float offset, int groups=1) -> ()");
   m.def("act_and_mul(Tensor(a!) out, Tensor input, bool gelu) -> ()");
   m.def("qknorm_vmix_cache(Tensor(a!) q, Tensor k, Tensor v, Tensor q_w, Tensor k_w, Tensor? v_first, float lam, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, float eps) -> ()");
-  m.def("paged_attn_prefill(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor cu_q, Tensor q_start, int max_q, int span, float scale, int mask_mode, int pos_stride, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0) -> ()");
-  m.def("paged_attn_decode(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor context_lens, int span, float scale, int mask_mode, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0) -> ()");
+  m.def("paged_attn_prefill(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor cu_q, Tensor q_start, int max_q, int span, float scale, int mask_mode, int pos_stride, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0, int weight_fn=0, Tensor? wbias=None) -> ()");
+  m.def("paged_attn_decode(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor context_lens, int span, float scale, int mask_mode, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0, int weight_fn=0, Tensor? wbias=None) -> ()");
   m.def("gla_recurrence(Tensor(a!) o, Tensor q, Tensor? k, Tensor v, Tensor z, Tensor z_bias, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh, float tau, Tensor? lower, bool q_silu, float q_scale) -> ()");
-  m.def("gla_out_norm_gate(Tensor(a!) out, Tensor o, Tensor weight, Tensor? gate, float eps) -> ()");
+  m.def("gla_out_norm_gate(Tensor(a!) out, Tensor o, Tensor weight, Tensor? gate, float eps, bool gate_sigmoid=False) -> ()");
   m.def("latent_rope_pack(Tensor(a!) out, Tensor q, Tensor q_lat, Tensor ckr, Tensor c_w, Tensor inv_freq, Tensor positions, Tensor(b!) k_cache, Tensor slots, int dim, int rot_dims, bool interleaved, float eps) -> ()");
   m.def("gated_residual_add(Tensor(a!) out, Tensor(b!) res, Tensor y1, Tensor g1, Tensor b1, Tensor? y2, Tensor? g2, Tensor? b2) -> ()");
   m.def("side_gate_mul(Tensor(a!) out, Tensor a, Tensor table, Tensor tokens, int offset) -> ()");
@@ -1376,7 +1552,7 @@ TORCH_LIBRARY(llmq_amd_hybrid, m) {
   m.def("moe_combine(Tensor(a!) y, Tensor yk, Tensor? wd) -> ()");
   m.def("moe_gather_combine(Tensor(a!) y, Tensor ys, Tensor pos, Tensor? w, int top) -> ()");
   m.def("embed_sinusoid(Tensor(a!) out, Tensor embedding, Tensor ids, Tensor positions, Tensor inv_freq) -> ()");
-  m.def("scaled_add_norm(Tensor(a!) out, Tensor(b!) res, Tensor y, Tensor? y2, float a1, float a2, Tensor weight, float eps) -> ()");
+  m.def("scaled_add_norm(Tensor(a!) out, Tensor(b!) res, Tensor y, Tensor? y2, float a1, float a2, Tensor weight, float eps, int groups=1) -> ()");
   m.def("depth_mix_norm(Tensor(a!) out, Tensor(b!) stack, int n, Tensor coef, Tensor y, Tensor? y2, float a1, float a2, Tensor weight, float eps) -> ()");
   m.def("kv_scatter(Tensor k, Tensor v, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor slots) -> ()");
   m.def("mingru_scan(Tensor(a!) out, Tensor z, Tensor u, Tensor g, Tensor z_b, Tensor u_b, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh) -> ()");
@@ -1384,13 +1560,16 @@ TORCH_LIBRARY(llmq_amd_hybrid, m) {
   m.def("selective_scan(Tensor(a!) out, Tensor x, Tensor dt, Tensor dt_b, Tensor A, Tensor Bm, Tensor Cm, Tensor D, Tensor z, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh) -> ()");
   m.def("softmax_topk(Tensor(a!) idx, Tensor(b!) w, Tensor logits, int top, float scale, Tensor? correction=None, bool renorm=False) -> ()");
   m.def("clamp_swish_mul(Tensor(a!) out, Tensor input, float limit) -> ()");
-  m.def("qkv_norm_rope_cache(Tensor(a!) q, Tensor k, Tensor? v, Tensor? q_w, Tensor? k_w, Tensor? inv_freq, int rot_dims, Tensor positions, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, float eps, bool v_unit_norm, Tensor? v_inv_freq) -> ()");
+  m.def("qkv_norm_rope_cache(Tensor(a!) q, Tensor k, Tensor? v, Tensor? q_w, Tensor? k_w, Tensor? inv_freq, int rot_dims, Tensor positions, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, float eps, bool v_unit_norm, Tensor? v_inv_freq, bool qk_unit_norm=False, Tensor? head_scale=None, float temp_coef=0.0, int temp_every=1, Tensor? v_first=None, float mix=0.0) -> ()");
   m.def("rotate_heads(Tensor(a!) x, Tensor positions, Tensor inv_freq, bool inverse) -> ()");
   m.def("mlstm_gates(Tensor(a!) out, Tensor gates, float cap, Tensor(b!) m_state, Tensor cu, Tensor slots, Tensor fresh) -> ()");
-  m.def("matrix_memory(Tensor(a!) o, Tensor q, Tensor k, Tensor v, Tensor decay, Tensor write, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh, float q_scale) -> ()");
+  m.def("matrix_memory(Tensor(a!) o, Tensor q, Tensor k, Tensor v, Tensor decay, Tensor write, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh, float q_scale, bool ones_col=True) -> ()");
   m.def("mlstm_out_norm_gate(Tensor(a!) out, Tensor o, Tensor floor, Tensor weight, Tensor gate, float eps) -> ()");
   m.def("dual_norm_mean(Tensor(a!) out, Tensor a, Tensor w_a, Tensor b, Tensor w_b, float eps) -> ()");
   m.def("unary_act(Tensor(a!) out, Tensor input, int act) -> ()");
+  m.def("gated_delta_rule(Tensor(a!) o, Tensor q, Tensor k, Tensor v, Tensor z, Tensor z_bias, Tensor rate, Tensor beta, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh, float q_scale) -> ()");
+  m.def("ssd_gates(Tensor(a!) out, Tensor dt, Tensor dt_bias, Tensor rate) -> ()");
+  m.def("ssd_out_gate_norm(Tensor(a!) out, Tensor o, Tensor x, Tensor D, Tensor z, Tensor weight, float eps, int groups) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(llmq_amd_hybrid, CUDA, m) {
@@ -1427,4 +1606,7 @@ TORCH_LIBRARY_IMPL(llmq_amd_hybrid, CUDA, m) {
   m.impl("mlstm_out_norm_gate", &mlstm_out_norm_gate);
   m.impl("dual_norm_mean", &dual_norm_mean);
   m.impl("unary_act", &unary_act);
+  m.impl("gated_delta_rule", &gated_delta_rule);
+  m.impl("ssd_gates", &ssd_gates);
+  m.impl("ssd_out_gate_norm", &ssd_out_gate_norm);
 }

@@ -7,4 +7,5 @@
 #include "latent_moe.hip"
 #include "scan_mix.hip"
 #include "memory_mix.hip"
+#include "delta_mix.hip"
 #include "hybrid_bindings.cpp"

@@ -17,11 +17,16 @@
 // to kRopePairs pairs and kRopeTail unrotated channels each), so a wave works
 // on 64 / LG heads at once and norm and rotation need no exchange beyond the
 // team's sum of squares.
-//   q [T, H, D] (rows strided): optional RMSNorm x weight, rotation, in place;
-//   k [T, G, D]: the same, into the key cache; with v == null its raw values
-//     go to the value cache (values = keys as projected);
-//   v [T, G, DV]: optional division by the root mean square, rotation over
-//     all DV channels with a table of its own, into the value cache.
+//   q [T, H, D] (rows strided): optional RMSNorm (x weight, or none), rotation,
+//     optional factor per head (head_scale) and per position
+//     (1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)), in place;
+//   k [T, G, D]: norm and rotation alike, into the key cache; with v == null
+//     its raw values go to the value cache (values = keys as projected);
+//   v [T, G, DV]: optional blend (1 - mix) v + mix v_first with another layer's
+//     values of the same token, optional division by the root mean square,
+//     rotation over all DV channels with a table of its own, into the value
+//     cache.
+// A norm without weight and a rotation commute (a rotation keeps the length).
 // cos/sin of a token's angles (position * inv_freq[i], fp32, sincosf) are
 // computed once per workgroup into LDS.
 constexpr int kRopePairs = 4;
@@ -30,7 +35,8 @@ constexpr int kRopeTail = 8;
 template <typename T>
 DEVINL void norm_rope_vector(const T* __restrict__ src, int n, int rd, const T* __restrict__ weight,
                              bool unit_norm, float eps, const float* __restrict__ cs, int sub,
-                             int LG, bool active, T* __restrict__ dst, T* __restrict__ raw_dst) {
+                             int LG, bool active, T* __restrict__ dst, T* __restrict__ raw_dst,
+                             float post, const T* __restrict__ first, float mix) {
   const int half = active ? rd / 2 : 0;
   if (!active) n = 0;
   float u[kRopePairs], v[kRopePairs], t[kRopeTail];
@@ -46,6 +52,10 @@ DEVINL void norm_rope_vector(const T* __restrict__ src, int n, int rd, const T* 
         raw_dst[i] = src[i];
         raw_dst[i + half] = src[i + half];
       }
+      if (first) {
+        u[j] = (1.0f - mix) * u[j] + mix * to_f32(first[i]);
+        v[j] = (1.0f - mix) * v[j] + mix * to_f32(first[i + half]);
+      }
     }
     ss += u[j] * u[j] + v[j] * v[j];
   }
@@ -56,6 +66,7 @@ DEVINL void norm_rope_vector(const T* __restrict__ src, int n, int rd, const T* 
     if (c < n) {
       t[j] = to_f32(src[c]);
       if (raw_dst) raw_dst[c] = src[c];
+      if (first) t[j] = (1.0f - mix) * t[j] + mix * to_f32(first[c]);
     }
     ss += t[j] * t[j];
   }
@@ -64,6 +75,7 @@ DEVINL void norm_rope_vector(const T* __restrict__ src, int n, int rd, const T* 
     for (int off = LG >> 1; off > 0; off >>= 1) ss += __shfl_xor(ss, off, WAVE);
     inv = 1.0f / sqrtf(ss / max(n, 1) + eps);
   }
+  inv *= post;
 #pragma unroll
   for (int j = 0; j < kRopePairs; ++j) {
     const int i = sub + LG * j;
@@ -96,7 +108,8 @@ DEVINL void norm_rope_vector(const T* __restrict__ src, int n, int rd, const T* 
 DEVINL void norm_rope_vec8(const __hip_bfloat16* __restrict__ src, int n, int rd,
                            const __hip_bfloat16* __restrict__ weight, bool unit_norm, float eps,
                            const float* __restrict__ cs, int sub, int LG, bool active,
-                           __hip_bfloat16* __restrict__ dst, __hip_bfloat16* __restrict__ raw_dst) {
+                           __hip_bfloat16* __restrict__ dst, __hip_bfloat16* __restrict__ raw_dst,
+                           float post, const __hip_bfloat16* __restrict__ first, float mix) {
   using bf = __hip_bfloat16;
   const int half = rd / 2;
   const bool has_pair = active && sub * 8 < half;
@@ -115,23 +128,37 @@ DEVINL void norm_rope_vec8(const __hip_bfloat16* __restrict__ src, int n, int rd
     for (int e = 0; e < 8; ++e) {
       u[e] = to_f32(a.data[e]);
       v[e] = to_f32(b.data[e]);
-      ss += u[e] * u[e] + v[e] * v[e];
     }
+    if (first) {
+      const Vec8<bf> fa = load16(first + sub * 8), fb = load16(first + half + sub * 8);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        u[e] = (1.0f - mix) * u[e] + mix * to_f32(fa.data[e]);
+        v[e] = (1.0f - mix) * v[e] + mix * to_f32(fb.data[e]);
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += u[e] * u[e] + v[e] * v[e];
   }
   if (has_tail) {
     const Vec8<bf> a = load16(src + rd + sub * 8);
     if (raw_dst) store16(raw_dst + rd + sub * 8, a);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      t[e] = to_f32(a.data[e]);
-      ss += t[e] * t[e];
+    for (int e = 0; e < 8; ++e) t[e] = to_f32(a.data[e]);
+    if (first) {
+      const Vec8<bf> fa = load16(first + rd + sub * 8);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) t[e] = (1.0f - mix) * t[e] + mix * to_f32(fa.data[e]);
     }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += t[e] * t[e];
   }
   float inv = 1.f;
   if (weight || unit_norm) {         // uniform over the wave: every lane takes part
     for (int off = LG >> 1; off > 0; off >>= 1) ss += __shfl_xor(ss, off, WAVE);
     inv = 1.0f / sqrtf(ss / max(active ? n : 1, 1) + eps);
   }
+  inv *= post;
   if (has_pair) {
     Vec8<bf> wa, wb, oa, ob;
     if (weight) {
@@ -168,9 +195,14 @@ DEVINL void norm_rope_vec8(const __hip_bfloat16* __restrict__ src, int n, int rd
 template <typename T, bool VEC>
 DEVINL void norm_rope_any(const T* __restrict__ src, int n, int rd, const T* __restrict__ weight,
                           bool unit_norm, float eps, const float* __restrict__ cs, int sub, int LG,
-                          bool active, T* __restrict__ dst, T* __restrict__ raw_dst) {
-  if constexpr (VEC) norm_rope_vec8(src, n, rd, weight, unit_norm, eps, cs, sub, LG, active, dst, raw_dst);
-  else norm_rope_vector<T>(src, n, rd, weight, unit_norm, eps, cs, sub, LG, active, dst, raw_dst);
+                          bool active, T* __restrict__ dst, T* __restrict__ raw_dst, float post,
+                          const T* __restrict__ first, float mix) {
+  if constexpr (VEC)
+    norm_rope_vec8(src, n, rd, weight, unit_norm, eps, cs, sub, LG, active, dst, raw_dst, post,
+                   first, mix);
+  else
+    norm_rope_vector<T>(src, n, rd, weight, unit_norm, eps, cs, sub, LG, active, dst, raw_dst, post,
+                        first, mix);
 }
 
 template <typename T, bool VEC>
@@ -182,7 +214,8 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_cache_kernel(
     const float* __restrict__ v_inv_freq,                 // [DV / 2] or null
     const long* __restrict__ positions, T* __restrict__ k_cache, T* __restrict__ v_cache,
     const long* __restrict__ slots, int H, int G, int D, int DV, int block_size, float eps,
-    int v_unit_norm, int LG) {
+    int v_unit_norm, int LG, int qk_unit_norm, const float* __restrict__ head_scale,
+    float temp_coef, int temp_every, const T* __restrict__ v_first, long vf_stride, float mix) {
   extern __shared__ __align__(8) float cs_smem[];
   float* cs = cs_smem;                       // [rot_dims/2][cos, sin]
   float* vcs = cs + rot_dims;                // [DV/2][cos, sin]
@@ -208,18 +241,24 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_cache_kernel(
   const long blk = slot >= 0 ? slot / block_size : 0;
   const int off = slot >= 0 ? (int)(slot % block_size) : 0;
   const int per_wave = 64 / LG, sub = lane % LG, team = lane / LG;
+  float temp = 1.f;
+  if (temp_coef != 0.f)
+    temp += temp_coef * logf((float)((positions[tok] + 1) / temp_every) + 1.0f);
   // three passes, each uniform over the wave in what it norms: q, k, v
   for (int base = w * per_wave; base < H; base += 4 * per_wave) {
     const int h = base + team;
     T* qh = q + tok * q_stride + (long)min(h, H - 1) * D;
-    norm_rope_any<T, VEC>(qh, D, rot_dims, q_w, false, eps, cs, sub, LG, h < H, qh, nullptr);
+    const float post = head_scale ? temp * head_scale[min(h, H - 1)] : temp;
+    norm_rope_any<T, VEC>(qh, D, rot_dims, q_w, qk_unit_norm != 0, eps, cs, sub, LG, h < H, qh,
+                          nullptr, post, nullptr, 0.f);
   }
   for (int base = w * per_wave; base < G; base += 4 * per_wave) {
     const int g = base + team;
     const bool act = g < G && slot >= 0;
     const long row = (blk * G + min(g, G - 1)) * block_size + off;
-    norm_rope_any<T, VEC>(k + tok * k_stride + (long)min(g, G - 1) * D, D, rot_dims, k_w, false,
-                          eps, cs, sub, LG, act, k_cache + row * D, v ? nullptr : v_cache + row * DV);
+    norm_rope_any<T, VEC>(k + tok * k_stride + (long)min(g, G - 1) * D, D, rot_dims, k_w,
+                          qk_unit_norm != 0, eps, cs, sub, LG, act, k_cache + row * D,
+                          v ? nullptr : v_cache + row * DV, 1.f, nullptr, 0.f);
   }
   if (v) {
     for (int base = w * per_wave; base < G; base += 4 * per_wave) {
@@ -228,7 +267,9 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_cache_kernel(
       const long row = (blk * G + min(g, G - 1)) * block_size + off;
       norm_rope_any<T, VEC>(v + tok * v_stride + (long)min(g, G - 1) * DV, DV, v_inv_freq ? DV : 0,
                             nullptr, v_unit_norm != 0, eps, vcs, sub, LG, act, v_cache + row * DV,
-                            nullptr);
+                            nullptr, 1.f,
+                            v_first ? v_first + tok * vf_stride + (long)min(g, G - 1) * DV : nullptr,
+                            mix);
     }
   }
 }

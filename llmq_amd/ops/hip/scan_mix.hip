@@ -32,13 +32,17 @@ __global__ void embed_sinusoid_kernel(float* __restrict__ out, const T* __restri
 
 // ------------------------------------------------------- residual joins ----
 // res (fp32, in place) += a1 * y [+ a2 * y2];  out = rmsnorm(res) * w.
-// One workgroup per row.
+// One workgroup per row. A row normed in `groups` equal consecutive parts is
+// `groups` rows of W elements each to these kernels; part g reads the weights
+// from g * W on.
 template <typename T>
 __global__ __launch_bounds__(256) void scaled_add_norm_kernel(
     T* __restrict__ out, float* __restrict__ res, const T* __restrict__ y,
-    const T* __restrict__ y2, float a1, float a2, const T* __restrict__ w, int W, float eps) {
+    const T* __restrict__ y2, float a1, float a2, const T* __restrict__ w, int W, float eps,
+    int groups) {
   __shared__ float red[4];
   const long row = blockIdx.x;
+  w += (row % groups) * W;
   float* rr = res + row * W;
   const T* yr = y + row * W;
   const T* y2r = y2 ? y2 + row * W : nullptr;
@@ -57,20 +61,25 @@ __global__ __launch_bounds__(256) void scaled_add_norm_kernel(
 
 // The same for bf16 rows of up to CH * 2048 elements, a multiple of 8 wide:
 // the updated residual stays in registers between the two passes and every
-// operand crosses memory once, in 16-byte accesses.
-template <int CH>
+// operand crosses memory once, in 16-byte accesses. PER_WAVE: rows (or parts)
+// of up to CH * 512 elements belong to one wave each, four to a workgroup.
+template <int CH, bool PER_WAVE>
 __global__ __launch_bounds__(256) void scaled_add_norm_vec_kernel(
     __hip_bfloat16* __restrict__ out, float* __restrict__ res,
     const __hip_bfloat16* __restrict__ y, const __hip_bfloat16* __restrict__ y2, float a1,
-    float a2, const __hip_bfloat16* __restrict__ w, int W, float eps) {
+    float a2, const __hip_bfloat16* __restrict__ w, int W, float eps, int groups, long rows) {
   __shared__ float red[4];
-  const long row = blockIdx.x;
+  constexpr int TEAM = PER_WAVE ? 64 : 256;
+  const int member = PER_WAVE ? (threadIdx.x & 63) : threadIdx.x;
+  const long row = PER_WAVE ? blockIdx.x * 4L + (threadIdx.x >> 6) : blockIdx.x;
+  if (PER_WAVE && row >= rows) return;
+  w += (row % groups) * W;
   float* rr = res + row * W;
   float rv[CH][8];
   float ss = 0.f;
 #pragma unroll
   for (int c = 0; c < CH; ++c) {
-    const int i = (c * 256 + threadIdx.x) * 8;
+    const int i = (c * TEAM + member) * 8;
     if (i < W) {
       const Vec8<__hip_bfloat16> v = load16(y + row * W + i);
       const float4 ra = *reinterpret_cast<const float4*>(rr + i);
@@ -90,11 +99,11 @@ __global__ __launch_bounds__(256) void scaled_add_norm_vec_kernel(
       *reinterpret_cast<float4*>(rr + i + 4) = make_float4(rv[c][4], rv[c][5], rv[c][6], rv[c][7]);
     }
   }
-  ss = block_reduce_sum(ss, red);
+  ss = PER_WAVE ? wave_reduce_sum(ss) : block_reduce_sum(ss, red);
   const float inv = 1.0f / sqrtf(ss / W + eps);
 #pragma unroll
   for (int c = 0; c < CH; ++c) {
-    const int i = (c * 256 + threadIdx.x) * 8;
+    const int i = (c * TEAM + member) * 8;
     if (i < W) {
       const Vec8<__hip_bfloat16> wv = load16(w + i);
       Vec8<__hip_bfloat16> ov;

@@ -293,6 +293,26 @@ DEVINL void add_sink(float& m, float& l, float& rescale, float sink) {
   m = m_new;
 }
 
+// What turns a score into a key's weight. Softmax: as above, normalised over
+// the visible keys. Sigmoid: 1 / (1 + e^-(score + wbias[head])) per key on its
+// own, no running maximum and no denominator.
+constexpr int kWeightSoftmax = 0;
+constexpr int kWeightSigmoid = 1;
+
+template <bool FAST>
+DEVINL float sigmoid_weight(float s) {
+  return FAST ? __builtin_amdgcn_rcpf(1.0f + __expf(-s)) : 1.0f / (1.0f + expf(-s));
+}
+
+// Output gate: sigmoid(gate) per head (gate_cols = 1) or per output channel of
+// every head (gate_cols = DV); no gate: 1.
+template <typename T>
+DEVINL float head_gate(const T* __restrict__ gate, long row_off, int gate_cols, int h, int c) {
+  if (!gate) return 1.f;
+  const long i = row_off + (gate_cols == 1 ? (long)h : (long)h * gate_cols + c);
+  return 1.0f / (1.0f + expf(-to_f32(gate[i])));
+}
+
 template <typename T, int NV>
 __global__ __launch_bounds__(256) void chunk_bias_attn_prefill_kernel(
     T* __restrict__ out, long out_stride,
@@ -305,8 +325,10 @@ __global__ __launch_bounds__(256) void chunk_bias_attn_prefill_kernel(
     const int* __restrict__ q_start,       // [B] position of a sequence's first query
     int H, int G, int D, int DV, int block_size, int span, float scale,
     int v_row, int mask_mode, int bias_mode, int keep_first, const float* __restrict__ sink,
-    float softcap) {
+    float softcap, int gate_cols, int weight_fn, const float* __restrict__ wbias) {
   extern __shared__ float smem[];
+  const bool sig = weight_fn == kWeightSigmoid;
+  const float wb = sig && wbias ? wbias[blockIdx.y] : 0.f;
   const int b = blockIdx.z, h = blockIdx.y;
   const int row0 = cu_q[b];
   const int nq = cu_q[b + 1] - row0;
@@ -387,6 +409,10 @@ __global__ __launch_bounds__(256) void chunk_bias_attn_prefill_kernel(
       const float sr = softcap > 0.f ? cap_score<sizeof(T) == 2>(s[r], softcap, inv_cap) : s[r];
       const float sc = !vis ? -INFINITY
           : bias ? sr + dist_bias<sizeof(T) == 2>(bias, bias_len, bias_mode, h, i - key) : sr;
+      if (sig) {
+        Ps[(w * 4 + r) * kAttnKT + lane] = vis ? sigmoid_weight<sizeof(T) == 2>(sc + wb) : 0.f;
+        continue;
+      }
       const float tmax = wave_reduce_max(sc);
       const float m_new = fmaxf(m[r], tmax);
       float p = 0.f, corr = 1.f;
@@ -434,13 +460,13 @@ __global__ __launch_bounds__(256) void chunk_bias_attn_prefill_kernel(
 #pragma unroll
       for (int n = 0; n < NV; ++n) acc[r][n] *= rescale;
     }
-    float gs = 1.f;
-    if (gate) gs = 1.0f / (1.0f + expf(-to_f32(gate[trow * g_stride + h])));
-    const float inv = gs / l[r];
+    const float inv = sig ? 1.f : 1.f / l[r];
 #pragma unroll
     for (int n = 0; n < NV; ++n) {
       const int c = lane + 64 * n;
-      if (c < DV) out[trow * out_stride + (long)h * DV + c] = from_f32<T>(acc[r][n] * inv);
+      if (c < DV)
+        out[trow * out_stride + (long)h * DV + c] =
+            from_f32<T>(acc[r][n] * inv * head_gate(gate, trow * g_stride, gate_cols, h, c));
     }
   }
 }
@@ -464,7 +490,7 @@ constexpr int kMfmaQT = 64;
 constexpr int kMfmaKT = 64;
 constexpr int kMfmaKP = kMfmaKT + 8;   // padded key stride of the V^T and P tiles
 
-template <int KS, int DT>
+template <int KS, int DT, bool SIG>
 __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
     __hip_bfloat16* __restrict__ out, long out_stride,
     const __hip_bfloat16* __restrict__ q, long q_stride,
@@ -475,7 +501,9 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
     const int* __restrict__ cu_q, const int* __restrict__ q_start,
     int H, int G, int D, int DV, int block_size, int span, float scale,
     int v_row, int mask_mode, int ps, int n_split, float* __restrict__ part, int bias_mode,
-    int keep_first, const float* __restrict__ sink, float softcap) {
+    int keep_first, const float* __restrict__ sink, float softcap, int gate_cols,
+    const float* __restrict__ wbias) {
+  // SIG: sigmoid weights (wbias [H] or null), see kWeightSigmoid.
   // n_split > 1: the grid's y dimension carries (key split, head); a
   // workgroup walks only its share of the key tiles and writes its
   // unnormalised output, running maximum and sum to `part`
@@ -535,6 +563,7 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
   const int wave_lo = mask_first_key(wave_first, span, mask_mode);
   const bool wave_rows = w * 16 < rows;
   const int* bt = block_tables + (long)b * bt_stride;
+  const float wb = SIG && wbias ? wbias[h] : 0.f;
   const bool bias_log = bias_mode == kBiasLog;
   const float* bias_h = bias ? bias + (bias_log ? 2L * h : (long)h * bias_len) : nullptr;
   short* Pw = Ps + w * 2 * 16 * kMfmaKP;
@@ -646,25 +675,31 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
           sv[ct] = vis ? sc + brow[-ct * 16] : -INFINITY;
           tmax = fmaxf(tmax, sv[ct]);
         }
-        tmax = fmaxf(tmax, __shfl_xor(tmax, 1, WAVE));
-        tmax = fmaxf(tmax, __shfl_xor(tmax, 2, WAVE));
-        tmax = fmaxf(tmax, __shfl_xor(tmax, 4, WAVE));
-        tmax = fmaxf(tmax, __shfl_xor(tmax, 8, WAVE));
-        const float m_new = fmaxf(m[reg], tmax);
-        float alpha = 1.f, psum = 0.f;
         float pv[4] = {0.f, 0.f, 0.f, 0.f};
-        if (m_new > -INFINITY) {
-          alpha = __expf(m[reg] - m_new);
+        if constexpr (SIG) {
+          // a masked score is -inf and weighs 1 / (1 + inf) = 0
 #pragma unroll
-          for (int ct = 0; ct < 4; ++ct) {
-            pv[ct] = sv[ct] > -INFINITY ? __expf(sv[ct] - m_new) : 0.f;
-            psum += pv[ct];
+          for (int ct = 0; ct < 4; ++ct) pv[ct] = sigmoid_weight<true>(sv[ct] + wb);
+        } else {
+          tmax = fmaxf(tmax, __shfl_xor(tmax, 1, WAVE));
+          tmax = fmaxf(tmax, __shfl_xor(tmax, 2, WAVE));
+          tmax = fmaxf(tmax, __shfl_xor(tmax, 4, WAVE));
+          tmax = fmaxf(tmax, __shfl_xor(tmax, 8, WAVE));
+          const float m_new = fmaxf(m[reg], tmax);
+          float alpha = 1.f, psum = 0.f;
+          if (m_new > -INFINITY) {
+            alpha = __expf(m[reg] - m_new);
+#pragma unroll
+            for (int ct = 0; ct < 4; ++ct) {
+              pv[ct] = sv[ct] > -INFINITY ? __expf(sv[ct] - m_new) : 0.f;
+              psum += pv[ct];
+            }
           }
-        }
-        l[reg] = l[reg] * alpha + psum;   // per-lane partial; reduced at the end
-        m[reg] = m_new;
+          l[reg] = l[reg] * alpha + psum;   // per-lane partial; reduced at the end
+          m[reg] = m_new;
 #pragma unroll
-        for (int dt = 0; dt < DT; ++dt) o[dt][reg] *= alpha;
+          for (int dt = 0; dt < DT; ++dt) o[dt][reg] *= alpha;
+        }
         short* pr = Pw + (kgrp * 4 + reg) * kMfmaKP + col;
 #pragma unroll
         for (int ct = 0; ct < 4; ++ct) {
@@ -725,14 +760,13 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
       }
       continue;
     }
-    float gs = 1.f;
-    if (gate) gs = 1.0f / (1.0f + expf(-__bfloat162float(gate[trow * g_stride + h])));
-    const float inv = gs / ll;
+    const float inv = SIG ? 1.f : 1.f / ll;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       const int c = dt * 16 + col;
       if (dt < dtn && c < DV)
-        out[trow * out_stride + (long)h * DV + c] = __float2bfloat16(o[dt][reg] * inv);
+        out[trow * out_stride + (long)h * DV + c] = __float2bfloat16(
+            o[dt][reg] * inv * head_gate(gate, trow * g_stride, gate_cols, h, c));
     }
   }
 }
@@ -790,8 +824,9 @@ __global__ __launch_bounds__(64 * kDecWaves) void chunk_bias_attn_decode_kernel(
     const int* __restrict__ context_lens,
     int H, int G, int D, int DV, int block_size, int span, float scale,
     int v_row, int mask_mode, int bias_mode, int keep_first, const float* __restrict__ sink,
-    float softcap) {
+    float softcap, int gate_cols, int weight_fn, const float* __restrict__ wbias) {
   extern __shared__ __align__(16) float smem[];
+  const bool sig = weight_fn == kWeightSigmoid;
   const int h0 = blockIdx.x * HPW, b = blockIdx.y;
   const int g = h0 / (H / G);
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
@@ -870,6 +905,12 @@ __global__ __launch_bounds__(64 * kDecWaves) void chunk_bias_attn_decode_kernel(
     float p[HPW];
 #pragma unroll
     for (int hh = 0; hh < HPW; ++hh) {
+      if (sig) {
+        const float wb = wbias ? wbias[h0 + hh] : 0.f;
+        p[hh] = lane < nk ? sigmoid_weight<sizeof(T) == 2>(sc[hh] + wb) : 0.f;
+        m[hh] = 0.f;               // equal in every wave that saw keys: partials add up as they are
+        continue;
+      }
       const float m_new = fmaxf(m[hh], wave_reduce_max(sc[hh]));  // nk >= 1: finite
       const float corr = expf(m[hh] - m_new);
       p[hh] = lane < nk ? expf(sc[hh] - m_new) : 0.f;
@@ -925,8 +966,8 @@ __global__ __launch_bounds__(64 * kDecWaves) void chunk_bias_attn_decode_kernel(
       ll += Ms[(NW + ww) * HPW + hh] * f;
       a += As[((long)ww * HPW + hh) * DV + c] * f;
     }
-    float gs = 1.f;
-    if (gate) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)b * g_stride + h0 + hh])));
+    if (sig) ll = 1.f;
+    const float gs = head_gate(gate, (long)b * g_stride, gate_cols, h0 + hh, c);
     out[(long)b * out_stride + (long)(h0 + hh) * DV + c] = from_f32<T>(a * gs / ll);
   }
 }
@@ -939,9 +980,10 @@ __global__ __launch_bounds__(64 * kDecWaves) void chunk_bias_attn_decode_kernel(
 //     w = k;
 //   HGRN2 (lower != null): a = l + (1 - l) * sigmoid(z + z_bias), w = 1 - a
 //     (no key is read).
-//   matrix memory (hdecay != null): per token and head ONE decay and one
+//   scalar gates (hdecay != null): per token and head ONE decay and one
 //     write strength, computed beforehand (fp32 [T, H]): a = hdecay[t, h] on
-//     every key channel, w = hwrite[t, h] * k; z is not read. With ones_col the
+//     every key channel, w = hwrite[t, h] * k; z is not read. Heads may share
+//     q and k in groups of hpk (a Mamba-2 scan's C and B). With ones_col the
 //     value gets one more column that is always 1, so the state's last column
 //     accumulates the written keys alone (an mLSTM's normaliser vector) and
 //     the output's last column is its product with q.
@@ -978,6 +1020,7 @@ __global__ __launch_bounds__(256) void gla_recurrence_kernel(
     int q_silu,
     const float* __restrict__ hdecay,       // [T, H] or null
     const float* __restrict__ hwrite,       // [T, H] (with hdecay)
+    int hpk,                                // heads per q/k head: head h reads q/k head h / hpk
     int ones_col) {                         // v has DV - 1 columns; column DV - 1 is 1
   constexpr int DP = 16 * DPL;          // padded key channels
   const int DVin = DV - (ones_col ? 1 : 0);
@@ -987,6 +1030,7 @@ __global__ __launch_bounds__(256) void gla_recurrence_kernel(
   __shared__ float vs[kGlaTB * kGlaCols];
   __shared__ float po[kGlaTB * 4 * kGlaCols];
   const int b = blockIdx.z, h = blockIdx.y;
+  const int hk = h / hpk;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   // a column's 4 key groups sit in one lane quad: their reduce is two DPP
   // quad permutes, no LDS traffic
@@ -1018,8 +1062,8 @@ __global__ __launch_bounds__(256) void gla_recurrence_kernel(
       rq[j] = rk[j] = rz[j] = 0.f;
       if (tt < nt && d < D) {
         const long row = row0 + t0 + tt;
-        rq[j] = to_f32(q[row * q_stride + (long)h * D + d]);
-        if (k) rk[j] = to_f32(k[row * k_stride + (long)h * D + d]);
+        rq[j] = to_f32(q[row * q_stride + (long)hk * D + d]);
+        if (k) rk[j] = to_f32(k[row * k_stride + (long)hk * D + d]);
         if (hdecay) {
           rz[j] = hdecay[row * H + h];
           rk[j] *= hwrite[row * H + h];
@@ -1145,13 +1189,14 @@ __global__ __launch_bounds__(256) void gla_recurrence_kernel(
   }
 }
 
-// Per (token, head): out = rmsnorm_DV(o) * w [* silu(gate)], rounded to T.
+// Per (token, head): out = rmsnorm_DV(o) * w [* silu(gate) | * sigmoid(gate)],
+// rounded to T.
 // One wave per head, lanes over value channels.
 template <typename T>
 __global__ __launch_bounds__(256) void gla_out_norm_gate_kernel(
     T* __restrict__ out, long out_stride, const float* __restrict__ o,
     const T* __restrict__ weight, const T* __restrict__ gate, long g_stride,
-    int H, int DV, float eps) {
+    int H, int DV, float eps, int gate_sigmoid) {
   const long tok = blockIdx.x;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   for (int h = w; h < H; h += 4) {
@@ -1164,7 +1209,7 @@ __global__ __launch_bounds__(256) void gla_out_norm_gate_kernel(
       float sg = 1.f;
       if (gate) {
         const float gt = to_f32(gate[tok * g_stride + (long)h * DV + c]);
-        sg = gt / (1.0f + expf(-gt));
+        sg = (gate_sigmoid ? 1.0f : gt) / (1.0f + expf(-gt));
       }
       out[tok * out_stride + (long)h * DV + c] =
           from_f32<T>(oh[c] * inv * to_f32(weight[c]) * sg);

@@ -379,10 +379,11 @@ def gla_recurrence(q, k, v, z, z_bias, state, cu, slots, fresh, tau):
     return o
 
 
-def gla_out_norm_gate(o, weight, gate, eps, out_dtype):
+def gla_out_norm_gate(o, weight, gate, eps, out_dtype, sigmoid=False):
     T, H, DV = o.shape
     y = o * (1.0 / torch.sqrt(o.pow(2).mean(dim=-1, keepdim=True) + eps)) * weight.float()
-    y = y.reshape(T, H * DV) * torch.nn.functional.silu(gate.float())
+    act = torch.sigmoid if sigmoid else torch.nn.functional.silu
+    y = y.reshape(T, H * DV) * act(gate.float())
     return y.to(out_dtype)
 
 
@@ -392,13 +393,14 @@ def gla_out_norm_gate(o, weight, gate, eps, out_dtype):
 
 
 def _window_attend(qb, kc, vc, pos, window, scale, log_bias=None, keep_first=0, sink=None,
-                   softcap=0.0):
+                   softcap=0.0, sigmoid=False, wbias=None):
     """qb [n, H, D] at absolute positions pos [n]; kc [L, G, D], vc [L, G, DV]
     cached keys/values of positions 0..L-1. Query i sees key j iff j <= i
     and (window == 0 or i - j < window or j < keep_first). log_bias [H, 2] =
     (r1, r2) per head takes r1 * ln(1 + r2 * (i - j)) off the scaled score.
     softcap c > 0: the scaled score becomes c * tanh(score / c). sink [H]:
-    the softmax denominator gains exp(sink[h])."""
+    the softmax denominator gains exp(sink[h]). sigmoid: a key's weight is
+    sigmoid(score + wbias[h]), not normalised."""
     n, H, _ = qb.shape
     G = kc.shape[1]
     lo = max(0, int(pos[0]) - window + 1) if window and not keep_first else 0
@@ -417,7 +419,11 @@ def _window_attend(qb, kc, vc, pos, window, scale, log_bias=None, keep_first=0, 
         r1, r2 = log_bias[:, 0].float().view(-1, 1, 1), log_bias[:, 1].float().view(-1, 1, 1)
         scores = scores - r1 * torch.log1p(r2 * dist)
     scores = scores.masked_fill(~vis.unsqueeze(0), float("-inf"))
-    if sink is not None:
+    if sigmoid:
+        if wbias is not None:
+            scores = scores + wbias.float().view(-1, 1, 1)
+        w = torch.sigmoid(scores)
+    elif sink is not None:
         extra = sink.float().view(-1, 1, 1).expand(H, n, 1)
         w = torch.softmax(torch.cat([scores, extra], dim=-1), dim=-1)[..., :-1]
     else:
@@ -425,8 +431,18 @@ def _window_attend(qb, kc, vc, pos, window, scale, log_bias=None, keep_first=0, 
     return torch.einsum("hij,jhd->ihd", w, vv)
 
 
+def _head_gate(y, gate):
+    """y [n, H, DV] times sigmoid(gate), gate [n, H] or [n, H * DV]."""
+    if gate is None:
+        return y
+    n, H, DV = y.shape
+    g = torch.sigmoid(gate.float())
+    return y * (g.unsqueeze(-1) if g.shape[1] == H else g.reshape(n, H, DV))
+
+
 def window_attn_prefill(q, k_cache, v_cache, dv, block_tables, cu_q, q_start, window, scale,
-                        log_bias=None, keep_first=0, sink=None, softcap=0.0):
+                        log_bias=None, keep_first=0, sink=None, softcap=0.0, gate=None,
+                        sigmoid=False, wbias=None):
     """Causal / sliding-window softmax attention of packed prompt portions
     over the paged cache. v_cache None: a key row's first dv channels are
     its value."""
@@ -441,13 +457,15 @@ def window_attn_prefill(q, k_cache, v_cache, dv, block_tables, cu_q, q_start, wi
         kc = _gather_seq(k_cache, block_tables[b], L)
         vc = kc[..., :dv] if v_cache is None else _gather_seq(v_cache, block_tables[b], L)
         pos = torch.arange(p0, L, device=q.device)
-        out[s:e] = _window_attend(q[s:e], kc, vc, pos, window, scale, log_bias, keep_first,
-                                  sink, softcap).to(q.dtype)
+        y = _window_attend(q[s:e], kc, vc, pos, window, scale, log_bias, keep_first, sink, softcap,
+                           sigmoid, wbias)
+        out[s:e] = _head_gate(y, None if gate is None else gate[s:e]).to(q.dtype)
     return out
 
 
 def window_attn_decode(q, k_cache, v_cache, dv, block_tables, context_lens, window, scale,
-                       log_bias=None, keep_first=0, sink=None, softcap=0.0):
+                       log_bias=None, keep_first=0, sink=None, softcap=0.0, gate=None,
+                       sigmoid=False, wbias=None):
     B, H, _ = q.shape
     out = q.new_empty(B, H, dv)
     for b in range(B):
@@ -455,8 +473,9 @@ def window_attn_decode(q, k_cache, v_cache, dv, block_tables, context_lens, wind
         kc = _gather_seq(k_cache, block_tables[b], L)
         vc = kc[..., :dv] if v_cache is None else _gather_seq(v_cache, block_tables[b], L)
         pos = torch.tensor([L - 1], device=q.device)
-        out[b : b + 1] = _window_attend(q[b : b + 1], kc, vc, pos, window, scale,
-                                        log_bias, keep_first, sink, softcap).to(q.dtype)
+        y = _window_attend(q[b : b + 1], kc, vc, pos, window, scale, log_bias, keep_first, sink,
+                           softcap, sigmoid, wbias)
+        out[b : b + 1] = _head_gate(y, None if gate is None else gate[b : b + 1]).to(q.dtype)
     return out
 
 
@@ -582,13 +601,14 @@ def embed_sinusoid(embedding, ids, positions, inv_freq):
     return x + pe
 
 
-def scaled_add_norm(res, y, y2, a1, a2, weight, eps, out_dtype):
-    """res (fp32, in place) += a1 * y [+ a2 * y2]; returns rmsnorm(res) * weight."""
+def scaled_add_norm(res, y, y2, a1, a2, weight, eps, out_dtype, groups=1):
+    """res (fp32, in place) += a1 * y [+ a2 * y2]; returns rmsnorm(res) * weight
+    (the norm on `groups` equal parts of a row)."""
     add = a1 * y.float()
     if y2 is not None:
         add = add + a2 * y2.float()
     res.add_(add)
-    return rmsnorm_cast(res, weight, eps, 0.0, out_dtype)
+    return rmsnorm_cast(res, weight, eps, 0.0, out_dtype, groups)
 
 
 def depth_mix_norm(stack, n, coef, y, y2, a1, a2, weight, eps, out_dtype):
@@ -721,7 +741,8 @@ def softcap(x, cap):
 
 
 def qkv_norm_rope_cache(q, k, v, q_w, k_w, inv_freq, rot_dims, positions, k_cache, v_cache,
-                        slots, eps, v_unit_norm, v_inv_freq):
+                        slots, eps, v_unit_norm, v_inv_freq, qk_unit_norm=False, head_scale=None,
+                        temp_coef=0.0, temp_every=1, v_first=None, mix=0.0):
     """Per token, between the projections and the attention kernel. q [T, H, D]
     (updated in place), k [T, G, D], v [T, G, DV] or None (the values are then
     the keys as they arrive). q_w / k_w [D] or None: per-head RMSNorm with that
@@ -729,11 +750,18 @@ def qkv_norm_rope_cache(q, k, v, q_w, k_w, inv_freq, rot_dims, positions, k_cach
     (i, i + rot_dims/2)) on the first rot_dims channels of q and k.
     v_unit_norm: each head's value divided by its root mean square;
     v_inv_freq [DV/2]: the value turned by its position over all DV channels.
-    k and v go to the paged cache rows `slots` (negative: skipped)."""
+    k and v go to the paged cache rows `slots` (negative: skipped).
+    qk_unit_norm: q and k divided by their root mean square per head, without a
+    weight. q then gains head_scale[h] and, at position p,
+    1 + temp_coef * ln(floor((p + 1) / temp_every) + 1). v_first [T, G, DV]:
+    v becomes (1 - mix) v + mix v_first first."""
     T, H, D = q.shape
     G = k.shape[1]
     raw_k = k.float()
     qf, kf = q.float(), raw_k
+    if qk_unit_norm:
+        qf = qf / torch.sqrt(qf.pow(2).mean(-1, keepdim=True) + eps)
+        kf = kf / torch.sqrt(kf.pow(2).mean(-1, keepdim=True) + eps)
     if q_w is not None:
         qf = qf / torch.sqrt(qf.pow(2).mean(-1, keepdim=True) + eps) * q_w.float()
     if k_w is not None:
@@ -741,7 +769,14 @@ def qkv_norm_rope_cache(q, k, v, q_w, k_w, inv_freq, rot_dims, positions, k_cach
     if rot_dims:
         qf = _rotate(qf, positions, inv_freq, rot_dims, False)
         kf = _rotate(kf, positions, inv_freq, rot_dims, False)
+    if head_scale is not None:
+        qf = qf * head_scale.float().view(1, H, 1)
+    if temp_coef:
+        step = torch.div(positions + 1, temp_every, rounding_mode="floor").float()
+        qf = qf * (1.0 + temp_coef * torch.log(step + 1.0)).view(T, 1, 1)
     vf = raw_k if v is None else v.float()
+    if v_first is not None:
+        vf = (1.0 - mix) * vf + mix * v_first.float()
     if v_unit_norm:
         vf = vf / torch.sqrt(vf.pow(2).mean(-1, keepdim=True) + eps)
     if v_inv_freq is not None:
@@ -841,3 +876,61 @@ def unary_act(x, kind):
     else:
         raise ValueError(f"unknown activation {kind!r}")
     return y.to(x.dtype)
+
+
+# ------------------------------------- gated delta rules, Mamba-2 scans (ref) --
+
+
+def gated_delta_rule(q, k, v, z, z_bias, rate, beta, state, cu, slots, fresh, q_scale):
+    """Token-by-token reference of ops.gated_delta_rule."""
+    T, Hk, D = q.shape
+    H = v.shape[1]
+    qf, kf = q.float(), k.float()
+    qf = qf / torch.sqrt(qf.pow(2).sum(-1, keepdim=True) + 1e-6) * q_scale
+    kf = kf / torch.sqrt(kf.pow(2).sum(-1, keepdim=True) + 1e-6)
+    qf = qf.repeat_interleave(H // Hk, dim=1)
+    kf = kf.repeat_interleave(H // Hk, dim=1)
+    step = torch.nn.functional.softplus(z.float() + z_bias.float().view(1, H, D))
+    g = torch.exp(-rate.float().view(1, H, 1) * step)
+    b = torch.sigmoid(beta.float())
+    vf = v.float()
+    o = torch.empty(v.shape, dtype=torch.float32, device=q.device)
+    for i in range(len(slots)):
+        s, e = int(cu[i]), int(cu[i + 1])
+        slot = int(slots[i])
+        S = torch.zeros_like(state[slot]) if int(fresh[i]) else state[slot].clone()
+        for t in range(s, e):
+            S = g[t].unsqueeze(-1) * S
+            u = b[t].unsqueeze(-1) * (vf[t] - torch.einsum("hdv,hd->hv", S, kf[t]))
+            S = S + kf[t].unsqueeze(-1) * u.unsqueeze(-2)
+            o[t] = torch.einsum("hdv,hd->hv", S, qf[t])
+        state[slot] = S
+    return o
+
+
+def ssd_scan(x, Bm, Cm, dt, dt_bias, rate, state, cu, slots, fresh):
+    """Token-by-token reference of ops.ssd_scan."""
+    T, H, DV = x.shape
+    rep = H // Bm.shape[1]
+    step = torch.nn.functional.softplus(dt.float() + dt_bias.float())
+    decay = torch.exp(-rate.float() * step)
+    Bf = Bm.float().repeat_interleave(rep, dim=1)
+    Cf = Cm.float().repeat_interleave(rep, dim=1)
+    xf = x.float() * step.unsqueeze(-1)
+    o = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    for i in range(len(slots)):
+        s, e = int(cu[i]), int(cu[i + 1])
+        slot = int(slots[i])
+        S = torch.zeros_like(state[slot]) if int(fresh[i]) else state[slot].clone()
+        for t in range(s, e):
+            S = decay[t].view(H, 1, 1) * S + Bf[t].unsqueeze(-1) * xf[t].unsqueeze(-2)
+            o[t] = torch.einsum("hdv,hd->hv", S, Cf[t])
+        state[slot] = S
+    return o
+
+
+def ssd_out_gate_norm(o, x, D, z, weight, eps, groups, out_dtype):
+    T, H, DV = o.shape
+    y = o + D.float().view(1, H, 1) * x.float().reshape(T, H, DV)
+    y = y.reshape(T, H * DV) * torch.nn.functional.silu(z.float())
+    return rmsnorm_cast(y, weight, eps, 0.0, torch.float32, groups).to(out_dtype)
