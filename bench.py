@@ -44,7 +44,8 @@ def compare_hybrid(args) -> None:
     models = args.compare_models.split(",")
     batch, prompt_len = min(args.batch, 64), args.prompt_len
     if not use_gpu:
-        tiny = ["tiny-tefudra", "tiny-muvetar"] if args.compare_tefudra else \
+        tiny = ["tiny-kikurax", "tiny-tefudra"] if args.compare_kikurax else \
+            ["tiny-tefudra", "tiny-muvetar"] if args.compare_tefudra else \
             ["tiny-muvetar", "tiny-kosalorn"] if args.compare_muvetar else \
             ["tiny-kosalorn"] if args.compare_kosalorn else []
         models, batch, prompt_len = tiny + ["tiny-kakovik", "tiny-llama"], 4, 48
@@ -148,7 +149,15 @@ def main() -> None:
                         help="the same comparison for the Tefudra presets (sink attention, "
                         "capped attention beside an mLSTM matrix memory, routed GELU experts) "
                         "beside the Kakovik, Muvetar and Llama presets of equal layer sizes")
+    parser.add_argument("--compare-kikurax", action="store_true",
+                        help="the same comparison for the Kikurax presets (sigmoid attention "
+                        "beside a gated delta rule, Mamba-2 scans, rotary attention, routed "
+                        "clamped experts) beside the Kakovik, Muvetar, Tefudra and Llama presets "
+                        "of equal layer sizes")
     args = parser.parse_args()
+    if args.compare_models is None and args.compare_kikurax:
+        args.compare_models = ("kikurax-1b,kakovik-1b,muvetar-1b,tefudra-1b-moe,llama-3.2-1b,"
+                               "kikurax-3b,muvetar-3b,llama-3.2-3b")
     if args.compare_models is None and args.compare_tefudra:
         args.compare_models = ("tefudra-1b,tefudra-1b-moe,kakovik-1b,muvetar-1b,llama-3.2-1b,"
                                "tefudra-3b,kakovik-3b,llama-3.2-3b")
@@ -158,7 +167,8 @@ def main() -> None:
         args.compare_models = (
             "kosalorn-1b,kosalorn-1b-moe,kakovik-1b,llama-3.2-1b,kosalorn-3b,kakovik-3b,llama-3.2-3b"
             if args.compare_kosalorn else "kakovik-1b,llama-3.2-1b,kakovik-3b,llama-3.2-3b")
-    if args.compare_hybrid or args.compare_kosalorn or args.compare_muvetar or args.compare_tefudra:
+    if (args.compare_hybrid or args.compare_kosalorn or args.compare_muvetar
+            or args.compare_tefudra or args.compare_kikurax):
         compare_hybrid(args)
         return
 

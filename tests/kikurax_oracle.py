@@ -66,12 +66,12 @@ def rotate_half(x, rot, first_pos=0):
     by position * f_i; the rest passes."""
     half = rot["dims"] // 2
     out = x.clone()
-    for r in range(x.shape[0]):
-        for i, f in enumerate(frequencies(rot)):
-            c, s = math.cos((first_pos + r) * f), math.sin((first_pos + r) * f)
-            u, v = x[r, :, i], x[r, :, i + half]
-            out[r, :, i] = u * c - v * s
-            out[r, :, i + half] = v * c + u * s
+    pos = torch.arange(first_pos, first_pos + x.shape[0], dtype=F64).view(-1, 1)
+    for i, f in enumerate(frequencies(rot)):
+        c, s = torch.cos(pos * f), torch.sin(pos * f)
+        u, v = x[:, :, i], x[:, :, i + half]
+        out[:, :, i] = u * c - v * s
+        out[:, :, i + half] = v * c + u * s
     return out
 
 
@@ -101,15 +101,15 @@ def sigmoid_attention(t, p, h, m, eps):
     q = rms((h @ t[p + "q"].T).view(n, H, D), eps)
     k = rms((h @ t[p + "k"].T).view(n, G, D), eps)
     v = (h @ t[p + "v"].T).view(n, G, DV)
+    if m.get("q_temp"):
+        q = q * torch.tensor([query_temperature(i, m["q_temp"]["coef"], m["q_temp"]["every"])
+                              for i in range(n)], dtype=F64).view(n, 1, 1)
+    seen = torch.ones(n, n, dtype=F64).tril()
     out = torch.zeros(n, H, DV, dtype=F64)
     for a in range(H):
         g = a // (H // G)
-        for i in range(n):
-            qi = q[i, a]
-            if m.get("q_temp"):
-                qi = qi * query_temperature(i, m["q_temp"]["coef"], m["q_temp"]["every"])
-            s = (k[:i + 1, g] @ qi) * m["scale"] + t[p + "pb"][a]
-            out[i, a] = sigmoid(s) @ v[:i + 1, g]
+        s = (q[:, a] @ k[:, g].T) * m["scale"] + t[p + "pb"][a]
+        out[:, a] = (sigmoid(s) * seen) @ v[:, g]
     y = out.reshape(n, H * DV) * sigmoid(h @ t[p + "g"].T)
     return y @ t[p + "o"].T
 
@@ -127,15 +127,15 @@ def gated_delta_rule(t, p, h, m, eps):
     beta = sigmoid(h @ t[p + "b"].T)
     z = (h @ t[p + "a1"].T) @ t[p + "a2"].T + t[p + "dt_bias"]
     decay = torch.exp(-torch.exp(t[p + "A_log"]).view(1, H, 1) * softplus(z).view(n, H, D))
+    of = torch.tensor([a // (H // G) for a in range(H)])       # a head's q/k head
     out = torch.zeros(n, H, DV, dtype=F64)
-    for a in range(H):
-        g = a // (H // G)
-        S = torch.zeros(D, DV, dtype=F64)
-        for r in range(n):
-            S = decay[r, a].view(D, 1) * S
-            u = beta[r, a] * (v[r, a] - S.T @ k[r, g])
-            S = S + torch.outer(k[r, g], u)
-            out[r, a] = S.T @ q[r, g]
+    S = torch.zeros(H, D, DV, dtype=F64)
+    for r in range(n):
+        S = decay[r].view(H, D, 1) * S
+        held = (S * k[r, of].view(H, D, 1)).sum(1)
+        u = beta[r].view(H, 1) * (v[r] - held)
+        S = S + k[r, of].view(H, D, 1) * u.view(H, 1, DV)
+        out[r] = (S * q[r, of].view(H, D, 1)).sum(1)
     gate = sigmoid((h @ t[p + "g1"].T) @ t[p + "g2"].T)
     y = (rms(out, eps) * t[p + "norm"]).reshape(n, H * DV) * gate
     return y @ t[p + "o"].T
@@ -160,14 +160,14 @@ def mamba2(t, p, h, m, eps):
     B = xbc[:, inner:inner + G * N].view(n, G, N)
     C = xbc[:, inner + G * N:].view(n, G, N)
     dt = softplus(dt + t[p + "dt_bias"])
+    of = torch.tensor([a // (H // G) for a in range(H)])       # a head's group
+    rate = torch.exp(t[p + "A_log"])
     out = torch.zeros(n, H, DV, dtype=F64)
-    for a in range(H):
-        g = a // (H // G)
-        S = torch.zeros(N, DV, dtype=F64)
-        rate = math.exp(float(t[p + "A_log"][a]))
-        for r in range(n):
-            S = math.exp(-rate * float(dt[r, a])) * S + dt[r, a] * torch.outer(B[r, g], x[r, a])
-            out[r, a] = S.T @ C[r, g] + t[p + "D"][a] * x[r, a]
+    S = torch.zeros(H, N, DV, dtype=F64)
+    for r in range(n):
+        S = torch.exp(-rate * dt[r]).view(H, 1, 1) * S + \
+            dt[r].view(H, 1, 1) * B[r, of].view(H, N, 1) * x[r].view(H, 1, DV)
+        out[r] = (S * C[r, of].view(H, N, 1)).sum(1) + t[p + "D"].view(H, 1) * x[r]
     y = out.reshape(n, inner) * silu(z)
     return group_norm(y, t[p + "norm"], eps, m["norm_groups"]) @ t[p + "o"].T
 
@@ -188,16 +188,17 @@ def rotary_attention(t, p, h, m, eps, v_first):
         v = (1.0 - lam) * own + lam * v_first
     q, k = rms(rotate_half(q, m["rot"]), eps), rms(rotate_half(k, m["rot"]), eps)
     cap = m.get("softcap")
+    seen = torch.ones(n, n, dtype=torch.bool).tril()
     out = torch.zeros(n, H, DV, dtype=F64)
     for a in range(H):
         g = a // (H // G)
-        for i in range(n):
-            s = (k[:i + 1, g] @ q[i, a]) * m["scale"] * t[p + "temp"][a]
-            if cap:
-                s = cap * torch.tanh(s / cap)
-            top = max(float(s.max()), 0.0)
-            e = torch.exp(s - top)
-            out[i, a] = (e @ v[:i + 1, g]) / (math.exp(-top) + e.sum())
+        s = (q[:, a] @ k[:, g].T) * m["scale"] * t[p + "temp"][a]
+        if cap:
+            s = cap * torch.tanh(s / cap)
+        s = s.masked_fill(~seen, float("-inf"))
+        top = torch.clamp(s.max(dim=1, keepdim=True).values, min=0.0)
+        e = torch.exp(s - top)
+        out[:, a] = (e @ v[:, g]) / (torch.exp(-top) + e.sum(dim=1, keepdim=True))
     return out.reshape(n, H * DV) @ t[p + "o"].T, own
 
 
