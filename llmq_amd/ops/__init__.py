@@ -1009,6 +1009,18 @@ def gated_delta_rule(q, k, v, z, z_bias, rate, beta, state, cu, slots, fresh,
                                       q_scale)
 
 
+# average portion length from which a bf16 Mamba-2 scan runs chunk-parallel on
+# the matrix cores; below it (and for fp32 models) token-serial
+SSD_CHUNK_MIN_TOKENS = 24
+
+
+def _ssd_chunkable(x, Bm, Cm) -> bool:
+    """Whole 16-byte granules in bf16 and at most 128 states per head."""
+    return (x.dtype == torch.bfloat16 and Bm.shape[2] % 8 == 0 and Bm.shape[2] <= 128
+            and x.shape[2] % 8 == 0
+            and all(t.stride(0) % 8 == 0 and t.data_ptr() % 16 == 0 for t in (x, Bm, Cm)))
+
+
 def ssd_scan(x, Bm, Cm, dt, dt_bias, rate, state, cu, slots, fresh) -> torch.Tensor:
     """Mamba-2 recurrence over packed sequences, per head h (which reads
     group h // (H / G)): step = softplus(dt + dt_bias),
@@ -1020,7 +1032,10 @@ def ssd_scan(x, Bm, Cm, dt, dt_bias, rate, state, cu, slots, fresh) -> torch.Ten
         gates = torch.empty(2, T, H, dtype=torch.float32, device=x.device)
         _HY.ssd_gates(gates, dt, dt_bias, rate)
         o = torch.empty(x.shape, dtype=torch.float32, device=x.device)
-        _HY.matrix_memory(o, Cm, Bm, x, gates[0], gates[1], state, cu, slots, fresh, 1.0, False)
+        if T >= SSD_CHUNK_MIN_TOKENS * slots.numel() and _ssd_chunkable(x, Bm, Cm):
+            _HY.ssd_chunk_scan(o, Cm, Bm, x, gates[1], rate, state, cu, slots, fresh)
+        else:
+            _HY.matrix_memory(o, Cm, Bm, x, gates[0], gates[1], state, cu, slots, fresh, 1.0, False)
         return o
     return torch_ref.ssd_scan(x, Bm, Cm, dt, dt_bias, rate, state, cu, slots, fresh)
 

@@ -1,7 +1,8 @@
 // Kernels of a gated delta rule and around a Mamba-2 scan (gfx950): the delta
-// rule's recurrence with a decay per key channel, and the gates and the gated,
-// grouped read-out norm of a state-space-duality mixer (whose recurrence is
-// the scalar-gate mode of the diagonal-decay kernel in seqmix.hip).
+// rule's recurrence with a decay per key channel; the gates, the chunk-parallel
+// matrix-core scan and the gated, grouped read-out norm of a state-space-duality
+// mixer (whose token-serial scan, for single tokens, short portions and fp32
+// models, is the scalar-gate mode of the diagonal-decay kernel in seqmix.hip).
 //
 // Numerics as in seqmix.hip: activations arrive in the model dtype T (bf16
 // or fp32); unit norms, decays, step sizes, gates and state are fp32 in
@@ -258,6 +259,236 @@ __global__ void ssd_gates_kernel(float* __restrict__ out, const T* __restrict__ 
     out[i] = FAST ? __expf(-rate[h] * step) : expf(-rate[h] * step);
     out[total + i] = step;
   }
+}
+
+// ------------------------------------- Mamba-2: chunk-parallel scan (bf16) ----
+// S_t = e^(a_t) S_(t-1) + step_t B_t x_t^T, o_t = S_t^T C_t with a_t = -rate step_t
+// has ONE decay per token, so over a chunk of 64 tokens with prefix sums
+// cum_i = a_0 + .. + a_i (all <= 0, every difference below is <= 0 too):
+//   o_i  = e^cum_i C_i S_prev + sum_(j <= i) (C_i . B_j) e^(cum_i - cum_j) step_j x_j
+//   S    = e^cum_last S_prev  + sum_j B_j (e^(cum_last - cum_j) step_j x_j)^T
+// four matrix products on v_mfma_f32_16x16x32_bf16 with fp32 accumulation.
+// B, C and x are bf16 already; every fp32 factor (the state, the weighted
+// scores, the weighted x) enters as TWO bf16 planes (value = hi + lo, lo the
+// rounding remainder), the state itself stays in fp32 accumulators for the
+// whole portion.
+//
+// Workgroup = 64 value columns of one (sequence, head), 8 waves. Wave (rt, hf):
+// output rows 16 rt .. + 15 x columns 32 hf .. + 31 (and the scores of those
+// rows with tokens 32 hf .. + 31), state rows NP/2 hf .. x columns 16 rt .. + 15.
+// The next chunk's rows are fetched into registers during the products. LDS
+// buffers whose lifetimes do not meet share their space (B rows / score planes;
+// state planes / weighted-x planes). Rows past the portion's end carry step 0,
+// which leaves state and prefix sums unchanged.
+constexpr int kSsdQ = 64;
+constexpr int kSsdKP = kSsdQ + 8;            // padded token stride of transposed tiles
+typedef __attribute__((ext_vector_type(4))) short ssd_bf16x4;
+
+DEVINL void split_bf16(float v, short& hi, short& lo) {
+  const __hip_bfloat16 h = __float2bfloat16(v);
+  hi = __bfloat16_as_short(h);
+  lo = __bfloat16_as_short(__float2bfloat16(v - __bfloat162float(h)));
+}
+
+constexpr size_t ssd_chunk_lds(int nk) {
+  const size_t ns = nk * 32 + 8;
+  const size_t u1 = kSsdQ * ns > 8u * 16 * kSsdKP ? kSsdQ * ns : 8u * 16 * kSsdKP;
+  const size_t u2 = 2 * 64 * ns > 2u * 64 * kSsdKP ? 2 * 64 * ns : 2u * 64 * kSsdKP;
+  return 2 * (kSsdQ * ns + u1 + u2 + (size_t)nk * 32 * kSsdKP + 64 * kSsdKP) + 2 * kSsdQ * 4;
+}
+
+template <int NK>                            // states padded to NK * 32
+__global__ __launch_bounds__(512) void ssd_chunk_scan_kernel(
+    float* __restrict__ o,                                   // [T, H, DV]
+    const __hip_bfloat16* __restrict__ Cm, long c_stride, const __hip_bfloat16* __restrict__ Bm,
+    long b_stride, const __hip_bfloat16* __restrict__ x, long x_stride,
+    const float* __restrict__ steps,                         // [T, H]
+    const float* __restrict__ rate,                          // [H]
+    float* __restrict__ state,                               // [slots, H, N, DV]
+    const int* __restrict__ cu, const int* __restrict__ slots, const int* __restrict__ fresh,
+    int H, int hpg, int N, int DV) {
+  extern __shared__ __align__(16) unsigned char ssd_smem[];
+  constexpr int NP = NK * 32, NS = NP + 8, KP = kSsdKP, Q = kSsdQ;
+  constexpr int NG = NK > 1 ? NK / 2 : 1;                    // B / C granules per thread
+  constexpr int U1 = Q * NS > 8 * 16 * KP ? Q * NS : 8 * 16 * KP;
+  constexpr int U2 = 2 * 64 * NS > 2 * 64 * KP ? 2 * 64 * NS : 2 * 64 * KP;
+  short* Cs = reinterpret_cast<short*>(ssd_smem);            // [Q][NS]
+  short* Bs = Cs + Q * NS;                                   // [Q][NS]
+  short* Ps = Bs;                                            // [4 row tiles][hi, lo][16][KP]
+  short* St = Bs + U1;                                       // [hi, lo][64][NS]
+  short* Xw = St;                                            // [hi, lo][64][KP]
+  short* Bt = St + U2;                                       // [NP][KP]
+  short* Xt = Bt + NP * KP;                                  // [64][KP]
+  float* cum = reinterpret_cast<float*>(Xt + 64 * KP);       // [Q]
+  float* stp = cum + Q;                                      // [Q]
+  const int b = blockIdx.z, h = blockIdx.y, c0 = blockIdx.x * 64;
+  const int row0 = cu[b], n = cu[b + 1] - row0;
+  if (n <= 0) return;
+  const int g = h / hpg;
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  const int rt = w & 3, hf = w >> 2, col = lane & 15, kgrp = lane >> 4;
+  const float rt_h = -rate[h];
+  const long sbase = ((long)slots[b] * H + h) * N * (long)DV;
+  const bool use_old = fresh[b] == 0;
+  const int vcol = c0 + rt * 16 + col;                       // this lane's state column
+  sm_f32x4 S[NK];
+#pragma unroll
+  for (int r = 0; r < NK; ++r)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int nn = (hf * NK + r) * 16 + kgrp * 4 + e;
+      S[r][e] = (use_old && nn < N && vcol < DV) ? state[sbase + (long)nn * DV + vcol] : 0.f;
+    }
+  const int sj = tid >> 3, sub = tid & 7;                    // staged token, granule
+  const sm_bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
+  sm_bf16x8 rc[NG], rb[NG], rx = zero8;
+  float rstep = 0.f;
+  auto fetch = [&](int t0) {
+    const bool live = t0 + sj < n;
+    const long row = row0 + t0 + sj;
+#pragma unroll
+    for (int i = 0; i < NG; ++i) {
+      const int d8 = (sub + 8 * i) * 8;
+      rc[i] = rb[i] = zero8;
+      if (live && d8 < N) {
+        rc[i] = *reinterpret_cast<const sm_bf16x8*>(Cm + row * c_stride + (long)g * N + d8);
+        rb[i] = *reinterpret_cast<const sm_bf16x8*>(Bm + row * b_stride + (long)g * N + d8);
+      }
+    }
+    rx = zero8;
+    if (live && c0 + sub * 8 < DV)
+      rx = *reinterpret_cast<const sm_bf16x8*>(x + row * x_stride + (long)h * DV + c0 + sub * 8);
+    rstep = t0 + lane < n ? steps[(long)(row0 + t0 + lane) * H + h] : 0.f;
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < n; t0 += Q) {
+    __syncthreads();                         // the previous chunk's tiles are read
+#pragma unroll
+    for (int i = 0; i < NG; ++i) {
+      const int d8 = (sub + 8 * i) * 8;
+      if (d8 < NP) {
+        *reinterpret_cast<sm_bf16x8*>(Cs + sj * NS + d8) = rc[i];
+        *reinterpret_cast<sm_bf16x8*>(Bs + sj * NS + d8) = rb[i];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) Bt[(d8 + e) * KP + sj] = rb[i][e];
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) Xt[(sub * 8 + e) * KP + sj] = rx[e];
+#pragma unroll
+    for (int r = 0; r < NK; ++r) {
+      ssd_bf16x4 hi, lo;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        short a, c;
+        split_bf16(S[r][e], a, c);
+        hi[e] = a;
+        lo[e] = c;
+      }
+      const int at = (rt * 16 + col) * NS + (hf * NK + r) * 16 + kgrp * 4;
+      *reinterpret_cast<ssd_bf16x4*>(St + at) = hi;
+      *reinterpret_cast<ssd_bf16x4*>(St + 64 * NS + at) = lo;
+    }
+    float cl = rt_h * rstep;                 // inclusive prefix sum over the wave's 64 lanes
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const float up = __shfl_up(cl, off, WAVE);
+      if (lane >= off) cl += up;
+    }
+    if (w == 0) {
+      cum[lane] = cl;
+      stp[lane] = rstep;
+    }
+    const float cum_last = __shfl(cl, 63, WAVE);
+    const sm_bf16x8 xg = rx;                 // this chunk's x granule, weighted below
+    __syncthreads();
+    if (t0 + Q < n) fetch(t0 + Q);
+    sm_f32x4 s[2], y[2];
+#pragma unroll
+    for (int ct = 0; ct < 2; ++ct) s[ct] = y[ct] = sm_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < NK; ++ks) {
+      const sm_bf16x8 cf = *reinterpret_cast<const sm_bf16x8*>(Cs + (rt * 16 + col) * NS + ks * 32 + kgrp * 8);
+#pragma unroll
+      for (int ct = 0; ct < 2; ++ct) {
+        const int at = ((hf * 2 + ct) * 16 + col) * NS + ks * 32 + kgrp * 8;
+        const sm_bf16x8 bf = *reinterpret_cast<const sm_bf16x8*>(Bs + at);
+        const sm_bf16x8 sh = *reinterpret_cast<const sm_bf16x8*>(St + at);
+        const sm_bf16x8 sl = *reinterpret_cast<const sm_bf16x8*>(St + 64 * NS + at);
+        s[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, bf, s[ct], 0, 0, 0);
+        y[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, sh, y[ct], 0, 0, 0);
+        y[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, sl, y[ct], 0, 0, 0);
+      }
+    }
+    float ci[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ci[e] = cum[rt * 16 + kgrp * 4 + e];
+    __syncthreads();                         // B rows and state planes are read
+#pragma unroll
+    for (int ct = 0; ct < 2; ++ct) {
+      const int j = (hf * 2 + ct) * 16 + col;
+      const float cj = cum[j], pj = stp[j];
+      short* pr = Ps + rt * 2 * 16 * KP + j;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int i = kgrp * 4 + e;
+        const float p = j <= rt * 16 + i ? s[ct][e] * __expf(ci[e] - cj) * pj : 0.f;
+        split_bf16(p, pr[i * KP], pr[(16 + i) * KP]);
+        y[ct][e] *= __expf(ci[e]);
+      }
+    }
+    {
+      const float wj = __expf(cum_last - cum[sj]) * stp[sj];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int at = (sub * 8 + e) * KP + sj;
+        split_bf16(__uint_as_float((unsigned)(unsigned short)xg[e] << 16) * wj, Xw[at],
+                   Xw[64 * KP + at]);
+      }
+    }
+    __syncthreads();
+    const float dl = __expf(cum_last);
+#pragma unroll
+    for (int r = 0; r < NK; ++r) S[r] *= dl;
+#pragma unroll
+    for (int k2 = 0; k2 < Q / 32; ++k2) {
+      const int ko = k2 * 32 + kgrp * 8;
+      const short* pr = Ps + (rt * 2 * 16 + col) * KP + ko;
+      const sm_bf16x8 ph = *reinterpret_cast<const sm_bf16x8*>(pr);
+      const sm_bf16x8 pl = *reinterpret_cast<const sm_bf16x8*>(pr + 16 * KP);
+#pragma unroll
+      for (int ct = 0; ct < 2; ++ct) {
+        const sm_bf16x8 xf = *reinterpret_cast<const sm_bf16x8*>(Xt + ((hf * 2 + ct) * 16 + col) * KP + ko);
+        y[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, xf, y[ct], 0, 0, 0);
+        y[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, xf, y[ct], 0, 0, 0);
+      }
+      const short* xr = Xw + (rt * 16 + col) * KP + ko;
+      const sm_bf16x8 wh = *reinterpret_cast<const sm_bf16x8*>(xr);
+      const sm_bf16x8 wl = *reinterpret_cast<const sm_bf16x8*>(xr + 64 * KP);
+#pragma unroll
+      for (int r = 0; r < NK; ++r) {
+        const sm_bf16x8 bf = *reinterpret_cast<const sm_bf16x8*>(Bt + ((hf * NK + r) * 16 + col) * KP + ko);
+        S[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf, wh, S[r], 0, 0, 0);
+        S[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf, wl, S[r], 0, 0, 0);
+      }
+    }
+#pragma unroll
+    for (int ct = 0; ct < 2; ++ct) {
+      const int c = c0 + (hf * 2 + ct) * 16 + col;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int t = t0 + rt * 16 + kgrp * 4 + e;
+        if (t < n && c < DV) o[((long)(row0 + t) * H + h) * DV + c] = y[ct][e];
+      }
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < NK; ++r)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int nn = (hf * NK + r) * 16 + kgrp * 4 + e;
+      if (nn < N && vcol < DV) state[sbase + (long)nn * DV + vcol] = S[r][e];
+    }
 }
 
 // ------------------------------------------------------- Mamba-2: read-out ----

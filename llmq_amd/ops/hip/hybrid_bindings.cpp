@@ -1016,18 +1016,29 @@ void causal_conv_silu(at::Tensor out, at::Tensor x, at::Tensor weight,
   TORCH_CHECK(tail.dim() == 3 && tail.size(1) == K - 1 && tail.size(2) == C, "tail [slots, K-1, C] fp32");
   // few rows (single tokens): a thread per row; prompts: 32 rows per thread
   const int rpt = T_ <= 512 ? 1 : 32;
-  const dim3 grid((C + 255) / 256, (T_ + rpt - 1) / rpt);
+  // bf16 channels in aligned pairs: two per thread
+  const bool pairs = x.scalar_type() == at::kBFloat16 && C % 2 == 0 && x.stride(0) % 2 == 0 &&
+                     reinterpret_cast<uintptr_t>(x.data_ptr()) % 4 == 0;
   hy_dispatch(x, "causal_conv_silu", [&]<typename T>() {
-    hipLaunchKernelGGL(causal_conv_silu_kernel<T>, grid, dim3(256), 0, hy_stream(),
-                       reinterpret_cast<T*>(out.data_ptr()), reinterpret_cast<const T*>(x.data_ptr()),
-                       x.stride(0), weight.data_ptr<float>(), bias_ptr,
-                       tail.data_ptr<float>(), cu.data_ptr<int>(), slots.data_ptr<int>(),
-                       fresh.data_ptr<int>(), d.B, C, K, rpt, (int)silu);
-    if (K > 1)
-      hipLaunchKernelGGL(conv_tail_update_kernel<T>, dim3((C + 255) / 256, d.B), dim3(256), 0,
-                         hy_stream(), reinterpret_cast<const T*>(x.data_ptr()), x.stride(0),
+    auto launch_v = [&]<int MAXK, int V>() {
+      const dim3 grid((C / V + 255) / 256, (T_ + rpt - 1) / rpt);
+      hipLaunchKernelGGL((causal_conv_silu_kernel<T, MAXK, V>), grid, dim3(256), 0, hy_stream(),
+                         reinterpret_cast<T*>(out.data_ptr()), reinterpret_cast<const T*>(x.data_ptr()),
+                         x.stride(0), weight.data_ptr<float>(), bias_ptr,
                          tail.data_ptr<float>(), cu.data_ptr<int>(), slots.data_ptr<int>(),
-                         fresh.data_ptr<int>(), C, K);
+                         fresh.data_ptr<int>(), d.B, C, K, rpt, (int)silu);
+    };
+    auto launch = [&]<int MAXK>() {
+      if (pairs && T_ > 512) launch_v.template operator()<MAXK, 2>();
+      else launch_v.template operator()<MAXK, 1>();
+      if (K > 1)
+        hipLaunchKernelGGL((conv_tail_update_kernel<T, MAXK>), dim3((C + 255) / 256, d.B), dim3(256), 0,
+                           hy_stream(), reinterpret_cast<const T*>(x.data_ptr()), x.stride(0),
+                           tail.data_ptr<float>(), cu.data_ptr<int>(), slots.data_ptr<int>(),
+                           fresh.data_ptr<int>(), C, K);
+    };
+    if (K <= 4) launch.template operator()<4>();
+    else launch.template operator()<kConvMaxTaps>();
   });
 }
 
@@ -1488,6 +1499,52 @@ void ssd_gates(at::Tensor out, at::Tensor dt, at::Tensor dt_bias, at::Tensor rat
   });
 }
 
+// The chunk-parallel scan: Cm, Bm [T, G, N], x [T, H, DV] bf16 (row-strided
+// views, heads packed, 16-byte granules); steps fp32 [T, H]; rate fp32 [H];
+// o fp32 [T, H, DV]; state fp32 [slots, H, N, DV].
+void ssd_chunk_scan(at::Tensor o, at::Tensor Cm, at::Tensor Bm, at::Tensor x, at::Tensor steps,
+                    at::Tensor rate, at::Tensor state, at::Tensor cu, at::Tensor slots,
+                    at::Tensor fresh) {
+  HY_GPU(x);
+  const long T_ = x.size(0);
+  if (T_ == 0) return;
+  TORCH_CHECK(x.dim() == 3 && Bm.dim() == 3 && Cm.sizes() == Bm.sizes() && Bm.size(0) == T_);
+  HY_INNER(x); HY_INNER(Bm); HY_INNER(Cm);
+  const int H = x.size(1), DV = x.size(2), G = Bm.size(1), N = Bm.size(2);
+  TORCH_CHECK(G >= 1 && H % G == 0, "heads must be a multiple of the groups");
+  TORCH_CHECK(x.scalar_type() == at::kBFloat16 && Bm.scalar_type() == at::kBFloat16 &&
+              Cm.scalar_type() == at::kBFloat16, "the chunked scan takes bf16");
+  TORCH_CHECK(x.stride(1) == DV && Bm.stride(1) == N && Cm.stride(1) == N, "heads must be packed");
+  auto granules = [](const at::Tensor& t) {
+    return t.stride(0) % 8 == 0 && reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0;
+  };
+  TORCH_CHECK(N % 8 == 0 && N >= 8 && N <= 128 && DV % 8 == 0 && granules(x) && granules(Bm) &&
+              granules(Cm), "the chunked scan takes whole 16-byte granules and at most 128 states");
+  HY_F32(steps); HY_F32(rate); HY_F32(o);
+  TORCH_CHECK(steps.dim() == 2 && steps.size(0) == T_ && steps.size(1) == H && rate.numel() == H);
+  TORCH_CHECK(o.dim() == 3 && o.sizes() == x.sizes());
+  const SeqDims sd = seq_check(cu, slots, fresh, state);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == N && state.size(3) == DV,
+              "state [slots, H, N, DV] fp32");
+  using bf = __hip_bfloat16;
+  const dim3 grid((DV + 63) / 64, H, sd.B);
+  auto launch = [&]<int NK>() {
+    auto kern = ssd_chunk_scan_kernel<NK>;
+    const size_t lds = ssd_chunk_lds(NK);
+    allow_lds(kern, lds);
+    hipLaunchKernelGGL(kern, grid, dim3(512), lds, hy_stream(), o.data_ptr<float>(),
+                       reinterpret_cast<const bf*>(Cm.data_ptr()), Cm.stride(0),
+                       reinterpret_cast<const bf*>(Bm.data_ptr()), Bm.stride(0),
+                       reinterpret_cast<const bf*>(x.data_ptr()), x.stride(0),
+                       steps.data_ptr<float>(), rate.data_ptr<float>(), state.data_ptr<float>(),
+                       cu.data_ptr<int>(), slots.data_ptr<int>(), fresh.data_ptr<int>(), H, H / G, N,
+                       DV);
+  };
+  if (N <= 32) launch.template operator()<1>();
+  else if (N <= 64) launch.template operator()<2>();
+  else launch.template operator()<4>();
+}
+
 // o fp32 [T, H, DV]; x, z [T, H*DV] row-strided; D fp32 [H]; weight [H*DV]
 void ssd_out_gate_norm(at::Tensor out, at::Tensor o, at::Tensor x, at::Tensor D, at::Tensor z,
                        at::Tensor weight, double eps, int64_t groups) {
@@ -1569,6 +1626,7 @@ TORCH_LIBRARY(llmq_amd_hybrid, m) {
   m.def("unary_act(Tensor(a!) out, Tensor input, int act) -> ()");
   m.def("gated_delta_rule(Tensor(a!) o, Tensor q, Tensor k, Tensor v, Tensor z, Tensor z_bias, Tensor rate, Tensor beta, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh, float q_scale) -> ()");
   m.def("ssd_gates(Tensor(a!) out, Tensor dt, Tensor dt_bias, Tensor rate) -> ()");
+  m.def("ssd_chunk_scan(Tensor(a!) o, Tensor Cm, Tensor Bm, Tensor x, Tensor steps, Tensor rate, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh) -> ()");
   m.def("ssd_out_gate_norm(Tensor(a!) out, Tensor o, Tensor x, Tensor D, Tensor z, Tensor weight, float eps, int groups) -> ()");
 }
 
@@ -1608,5 +1666,6 @@ TORCH_LIBRARY_IMPL(llmq_amd_hybrid, CUDA, m) {
   m.impl("unary_act", &unary_act);
   m.impl("gated_delta_rule", &gated_delta_rule);
   m.impl("ssd_gates", &ssd_gates);
+  m.impl("ssd_chunk_scan", &ssd_chunk_scan);
   m.impl("ssd_out_gate_norm", &ssd_out_gate_norm);
 }

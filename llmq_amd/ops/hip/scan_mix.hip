@@ -366,35 +366,54 @@ __global__ __launch_bounds__(64 * NC) void mingru_scan_chunked_kernel(
 // sequence). Not a recurrence: a thread owns one channel and kConvRows
 // consecutive packed rows, wherever they fall in their sequences. The tail is
 // advanced by a second kernel after every read of the old one has happened.
+// MAXK bounds the taps: the usual short kernels keep 4 weights and inputs per
+// channel in registers instead of kConvMaxTaps.
 constexpr int kConvMaxTaps = 16;
 constexpr int kConvGroup = 8;    // rows whose inputs a thread fetches together
 
-template <typename T>
+// V adjacent channels per thread: 1, or 2 as one 4-byte access for bf16.
+template <typename T, int V>
+DEVINL void load_channels(const T* __restrict__ p, float* v) {
+  if constexpr (V == 2 && sizeof(T) == 2) {
+    const unsigned u = *reinterpret_cast<const unsigned*>(p);
+    v[0] = __uint_as_float(u << 16);
+    v[1] = __uint_as_float(u & 0xffff0000u);
+  } else {
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = to_f32(p[e]);
+  }
+}
+
+template <typename T, int MAXK, int V>
 __global__ __launch_bounds__(256) void causal_conv_silu_kernel(
     T* __restrict__ out, const T* __restrict__ x, long x_stride, const float* __restrict__ w,
     const float* __restrict__ bias, const float* __restrict__ tail,
     const int* __restrict__ cu, const int* __restrict__ slots, const int* __restrict__ fresh,
     int B, int C, int K, int rows_per_thread, int silu) {
   // bias may be null; silu == 0 leaves the convolution's result as it is
-  const int c = blockIdx.x * 256 + threadIdx.x;
+  constexpr bool FAST = sizeof(T) == 2;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * V;    // V divides C
   if (c >= C) return;
   const int total = cu[B];
   const int r0 = blockIdx.y * rows_per_thread;
   if (r0 >= total) return;
   const int r1 = min(total, r0 + rows_per_thread);
-  float wk[kConvMaxTaps], win[kConvMaxTaps];
+  float wk[MAXK][V], win[MAXK][V] = {}, bc[V];
 #pragma unroll
-  for (int k = 0; k < kConvMaxTaps; ++k) wk[k] = k < K ? w[(long)c * K + k] : 0.f;
-  const float bc = bias ? bias[c] : 0.f;
+  for (int e = 0; e < V; ++e) {
+#pragma unroll
+    for (int k = 0; k < MAXK; ++k) wk[k][e] = k < K ? w[(long)(c + e) * K + k] : 0.f;
+    bc[e] = bias ? bias[c + e] : 0.f;
+  }
   int b = 0;
   while (cu[b + 1] <= r0) ++b;   // the sequence of row r0 (empty sequences skipped)
   bool load_window = true;
   for (int g0 = r0; g0 < r1; g0 += kConvGroup) {
     // the group's own inputs first: independent loads, all in flight at once
-    float xg[kConvGroup];
+    float xg[kConvGroup][V];
 #pragma unroll
     for (int i = 0; i < kConvGroup; ++i)
-      xg[i] = to_f32(x[(long)min(g0 + i, r1 - 1) * x_stride + c]);
+      load_channels<T, V>(x + (long)min(g0 + i, r1 - 1) * x_stride + c, xg[i]);
 #pragma unroll
     for (int i = 0; i < kConvGroup; ++i) {
       const int r = g0 + i;
@@ -409,30 +428,47 @@ __global__ __launch_bounds__(256) void causal_conv_silu_kernel(
           const bool fr = fresh[b] != 0;
           // win[k] = V[j - (K-1) + k], k < K-1
 #pragma unroll
-          for (int k = 0; k < kConvMaxTaps - 1; ++k) {
+          for (int k = 0; k < MAXK - 1; ++k) {
             if (k < K - 1) {
               const int jj = j - (K - 1) + k;
-              win[k] = jj >= 0 ? to_f32(x[(long)(s + jj) * x_stride + c])
-                               : (fr ? 0.f : tl[(long)(jj + K - 1) * C]);
+              if (jj >= 0) {
+                load_channels<T, V>(x + (long)(s + jj) * x_stride + c, win[k]);
+              } else {
+#pragma unroll
+                for (int e = 0; e < V; ++e) win[k][e] = fr ? 0.f : tl[(long)(jj + K - 1) * C + e];
+              }
             }
           }
           load_window = false;
         }
-        const float xv = xg[i];
-        float acc = bc;
+        alignas(4) T ov[V];
 #pragma unroll
-        for (int k = 0; k < kConvMaxTaps - 1; ++k)
-          if (k < K - 1) acc += wk[k] * win[k];
+        for (int e = 0; e < V; ++e) {
+          const float xv = xg[i][e];
+          float acc = bc[e];
 #pragma unroll
-        for (int k = 0; k < kConvMaxTaps; ++k)
-          if (k == K - 1) acc += wk[k] * xv;
-        out[(long)r * C + c] = from_f32<T>(silu ? acc * sigmoid_f(acc) : acc);
+          for (int k = 0; k < MAXK - 1; ++k)
+            if (k < K - 1) acc += wk[k][e] * win[k][e];
 #pragma unroll
-        for (int k = 0; k < kConvMaxTaps - 2; ++k)
-          if (k < K - 2) win[k] = win[k + 1];
+          for (int k = 0; k < MAXK; ++k)
+            if (k == K - 1) acc += wk[k][e] * xv;
+          if (silu)
+            acc *= FAST ? __builtin_amdgcn_rcpf(1.0f + __expf(-acc)) : sigmoid_f(acc);
+          ov[e] = from_f32<T>(acc);
 #pragma unroll
-        for (int k = 0; k < kConvMaxTaps - 1; ++k)
-          if (k == K - 2) win[k] = xv;
+          for (int k = 0; k < MAXK - 2; ++k)
+            if (k < K - 2) win[k][e] = win[k + 1][e];
+#pragma unroll
+          for (int k = 0; k < MAXK - 1; ++k)
+            if (k == K - 2) win[k][e] = xv;
+        }
+        T* op = out + (long)r * C + c;
+        if constexpr (V == 2 && sizeof(T) == 2) {
+          *reinterpret_cast<unsigned*>(op) = *reinterpret_cast<const unsigned*>(ov);
+        } else {
+#pragma unroll
+          for (int e = 0; e < V; ++e) op[e] = ov[e];
+        }
       }
     }
   }
@@ -440,7 +476,7 @@ __global__ __launch_bounds__(256) void causal_conv_silu_kernel(
 
 // tail[slot, k, c] <- V[n - (K-1) + k], n = the portion's length: its last
 // K-1 inputs, reaching back into the old tail when the portion is shorter.
-template <typename T>
+template <typename T, int MAXK>
 __global__ __launch_bounds__(256) void conv_tail_update_kernel(
     const T* __restrict__ x, long x_stride, float* __restrict__ tail,
     const int* __restrict__ cu, const int* __restrict__ slots, const int* __restrict__ fresh,
@@ -452,9 +488,9 @@ __global__ __launch_bounds__(256) void conv_tail_update_kernel(
   if (n <= 0) return;
   float* tl = tail + (long)slots[b] * (K - 1) * C + c;
   const bool fr = fresh[b] != 0;
-  float nv[kConvMaxTaps];
+  float nv[MAXK];
 #pragma unroll
-  for (int k = 0; k < kConvMaxTaps - 1; ++k) {
+  for (int k = 0; k < MAXK - 1; ++k) {
     if (k < K - 1) {
       const int jj = n - (K - 1) + k;
       nv[k] = jj >= 0 ? to_f32(x[(long)(s + jj) * x_stride + c])
@@ -462,7 +498,7 @@ __global__ __launch_bounds__(256) void conv_tail_update_kernel(
     }
   }
 #pragma unroll
-  for (int k = 0; k < kConvMaxTaps - 1; ++k)
+  for (int k = 0; k < MAXK - 1; ++k)
     if (k < K - 1) tl[(long)k * C] = nv[k];
 }
 

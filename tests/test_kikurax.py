@@ -768,8 +768,12 @@ def test_gated_delta_rule_against_token_by_token(target, H, G, D, DV, lens):
 @pytest.mark.parametrize("H,G,N,DV,ng,lens", [
     (4, 2, 8, 12, 2, [70, 1, 3, 40]), (1, 1, 1, 24, 1, [100]), (6, 6, 33, 5, 3, [17, 33]),
     (3, 1, 70, 40, 8, [5, 1, 1]), (2, 1, 128, 64, 1, [40, 9]), (2, 2, 200, 31, 2, [1, 1]),
-    (40, 8, 16, 64, 1, [3, 1])])
+    (40, 8, 16, 64, 1, [3, 1]), (4, 2, 24, 72, 2, [130, 64, 1, 65]), (2, 2, 64, 16, 1, [300]),
+    (1, 1, 8, 8, 1, [63, 200]), (8, 1, 96, 136, 1, [150, 31]), (16, 2, 128, 64, 4, [64, 127])])
 def test_ssd_scan_and_read_out_against_token_by_token(target, H, G, N, DV, ng, lens):
+    """Unequal packed sequences, each cut in two calls through its state slot:
+    short portions and odd sizes walk token by token, long bf16 portions of
+    whole granules run in chunks on the matrix cores."""
     device, dtype = dev_dtype(target)
     g = torch.Generator().manual_seed(H * 100 + N)
     B, total, eps = len(lens), [n * 2 + 1 for n in lens], 1e-5
@@ -793,7 +797,7 @@ def test_ssd_scan_and_read_out_against_token_by_token(target, H, G, N, DV, ng, l
                          rate.to(device), S, cu, slots, fresh)
         y = ops.ssd_out_gate_norm(o, x, Dh.to(device), cat("z"), w.to(device), eps, ng, dtype)
         for b in range(B):
-            outs[b].append(y[int(cu[b]):int(cu[b + 1])].cpu())
+            outs[b].append((o[int(cu[b]):int(cu[b + 1])].cpu(), y[int(cu[b]):int(cu[b + 1])].cpu()))
     tol = 2e-2 if dtype == torch.bfloat16 else 2e-4
     for b, d in enumerate(data):
         r = {k: t.to(dtype).double() for k, t in d.items()}
@@ -806,11 +810,45 @@ def test_ssd_scan_and_read_out_against_token_by_token(target, H, G, N, DV, ng, l
             for t in range(n):
                 M = torch.exp(-rate[a].double() * step[t, a]) * M + \
                     step[t, a] * torch.outer(r["B"][t, ga], x[t, a])
-                want[t, a] = M.T @ r["C"][t, ga] + Dh[a].double() * x[t, a]
+                want[t, a] = M.T @ r["C"][t, ga]
+            got_S = S[int(slots[b]), a].double().cpu()
+            assert (got_S - M).abs().max() < 1e-4 * M.abs().max().clamp(min=0.1), (b, a)
+        # inputs are exact in both: the recurrence itself is at fp32 level
+        got_o = torch.cat([oo for oo, _ in outs[b]]).double()
+        assert (got_o - want).abs().max() < 1e-4 * want.abs().max(), b
+        want = want + Dh.double().view(1, H, 1) * x
         want = oracle.group_norm(want.reshape(n, H * DV) * oracle.silu(r["z"]), w.double(), eps, ng)
-        got = torch.cat(outs[b]).double()
+        got = torch.cat([y for _, y in outs[b]]).double()
         err = (got - want).pow(2).mean().sqrt() / want.pow(2).mean().sqrt()
         assert err < tol, (b, float(err))
+
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("decay", [1e-4, 0.3, 40.0], ids=["slow", "middle", "fast"])
+def test_ssd_scan_one_write_far_back(target, decay):
+    """A single write read hundreds of tokens later survives (or fades) by
+    exactly the decays between, across the chunks of a long portion."""
+    device, dtype = dev_dtype(target)
+    T, H, N, DV, at = 400, 2, 16, 8, 37
+    x = torch.zeros(T, H, DV, dtype=dtype)
+    Bm = torch.zeros(T, 1, N, dtype=dtype)
+    x[at], Bm[at, :, 3] = 1.0, 2.0
+    Cm = torch.zeros(T, 1, N, dtype=dtype)
+    Cm[:, :, 3] = 0.5
+    dt = torch.full((T, H), 1.0, dtype=dtype)
+    step = math.log1p(math.exp(1.0))
+    S = torch.zeros(1, H, N, DV, device=device)
+    o = ops.ssd_scan(x.to(device), Bm.to(device), Cm.to(device), dt.to(device),
+                     torch.zeros(H, device=device), torch.full((H,), decay / step, device=device), S,
+                     torch.tensor([0, T], dtype=torch.int32, device=device),
+                     torch.tensor([0], dtype=torch.int32, device=device),
+                     torch.tensor([1], dtype=torch.int32, device=device))
+    o = o.double().cpu()[:, :, 0]
+    for t in (0, at - 1):
+        assert float(o[t].abs().max()) == 0.0
+    for t in (at, at + 1, 63, 64, 65, 127, 128, 399):
+        want = step * math.exp(-decay * (t - at))
+        assert float((o[t] - want).abs().max()) < 2e-4 * want + 1e-30, (t, o[t], want)
 
 
 @pytest.mark.parametrize("target", DEVICES)
