@@ -294,11 +294,11 @@ constexpr size_t ssd_chunk_lds(int nk) {
   const size_t ns = nk * 32 + 8;
   const size_t u1 = kSsdQ * ns > 8u * 16 * kSsdKP ? kSsdQ * ns : 8u * 16 * kSsdKP;
   const size_t u2 = 2 * 64 * ns > 2u * 64 * kSsdKP ? 2 * 64 * ns : 2u * 64 * kSsdKP;
-  return 2 * (kSsdQ * ns + u1 + u2 + (size_t)nk * 32 * kSsdKP + 64 * kSsdKP) + 2 * kSsdQ * 4;
+  return 2 * (u1 + u2 + (size_t)nk * 32 * kSsdKP + 64 * kSsdKP) + 2 * kSsdQ * 4;
 }
 
 template <int NK>                            // states padded to NK * 32
-__global__ __launch_bounds__(512) void ssd_chunk_scan_kernel(
+__global__ __launch_bounds__(512, 4) void ssd_chunk_scan_kernel(
     float* __restrict__ o,                                   // [T, H, DV]
     const __hip_bfloat16* __restrict__ Cm, long c_stride, const __hip_bfloat16* __restrict__ Bm,
     long b_stride, const __hip_bfloat16* __restrict__ x, long x_stride,
@@ -309,11 +309,10 @@ __global__ __launch_bounds__(512) void ssd_chunk_scan_kernel(
     int H, int hpg, int N, int DV) {
   extern __shared__ __align__(16) unsigned char ssd_smem[];
   constexpr int NP = NK * 32, NS = NP + 8, KP = kSsdKP, Q = kSsdQ;
-  constexpr int NG = NK > 1 ? NK / 2 : 1;                    // B / C granules per thread
+  constexpr int NG = NK > 1 ? NK / 2 : 1;                    // B granules per thread
   constexpr int U1 = Q * NS > 8 * 16 * KP ? Q * NS : 8 * 16 * KP;
   constexpr int U2 = 2 * 64 * NS > 2 * 64 * KP ? 2 * 64 * NS : 2 * 64 * KP;
-  short* Cs = reinterpret_cast<short*>(ssd_smem);            // [Q][NS]
-  short* Bs = Cs + Q * NS;                                   // [Q][NS]
+  short* Bs = reinterpret_cast<short*>(ssd_smem);            // [Q][NS]
   short* Ps = Bs;                                            // [4 row tiles][hi, lo][16][KP]
   short* St = Bs + U1;                                       // [hi, lo][64][NS]
   short* Xw = St;                                            // [hi, lo][64][KP]
@@ -339,9 +338,11 @@ __global__ __launch_bounds__(512) void ssd_chunk_scan_kernel(
       const int nn = (hf * NK + r) * 16 + kgrp * 4 + e;
       S[r][e] = (use_old && nn < N && vcol < DV) ? state[sbase + (long)nn * DV + vcol] : 0.f;
     }
-  const int sj = tid >> 3, sub = tid & 7;                    // staged token, granule
+  // staged token and granule: a wave holds one granule of all 64 tokens, so its
+  // transposing LDS stores are 64 adjacent elements
+  const int sj = lane, sub = w;
   const sm_bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
-  sm_bf16x8 rc[NG], rb[NG], rx = zero8;
+  sm_bf16x8 rc[NK], rb[NG], rx = zero8;      // rc: this lane's C operands, straight from memory
   float rstep = 0.f;
   auto fetch = [&](int t0) {
     const bool live = t0 + sj < n;
@@ -349,11 +350,15 @@ __global__ __launch_bounds__(512) void ssd_chunk_scan_kernel(
 #pragma unroll
     for (int i = 0; i < NG; ++i) {
       const int d8 = (sub + 8 * i) * 8;
-      rc[i] = rb[i] = zero8;
-      if (live && d8 < N) {
-        rc[i] = *reinterpret_cast<const sm_bf16x8*>(Cm + row * c_stride + (long)g * N + d8);
+      rb[i] = zero8;
+      if (live && d8 < N)
         rb[i] = *reinterpret_cast<const sm_bf16x8*>(Bm + row * b_stride + (long)g * N + d8);
-      }
+    }
+#pragma unroll
+    for (int ks = 0; ks < NK; ++ks) {
+      const int t = t0 + rt * 16 + col, d8 = ks * 32 + kgrp * 8;
+      rc[ks] = t < n && d8 < N
+          ? *reinterpret_cast<const sm_bf16x8*>(Cm + (row0 + t) * c_stride + (long)g * N + d8) : zero8;
     }
     rx = zero8;
     if (live && c0 + sub * 8 < DV)
@@ -367,7 +372,6 @@ __global__ __launch_bounds__(512) void ssd_chunk_scan_kernel(
     for (int i = 0; i < NG; ++i) {
       const int d8 = (sub + 8 * i) * 8;
       if (d8 < NP) {
-        *reinterpret_cast<sm_bf16x8*>(Cs + sj * NS + d8) = rc[i];
         *reinterpret_cast<sm_bf16x8*>(Bs + sj * NS + d8) = rb[i];
 #pragma unroll
         for (int e = 0; e < 8; ++e) Bt[(d8 + e) * KP + sj] = rb[i][e];
@@ -401,6 +405,9 @@ __global__ __launch_bounds__(512) void ssd_chunk_scan_kernel(
     }
     const float cum_last = __shfl(cl, 63, WAVE);
     const sm_bf16x8 xg = rx;                 // this chunk's x granule, weighted below
+    sm_bf16x8 cf[NK];
+#pragma unroll
+    for (int ks = 0; ks < NK; ++ks) cf[ks] = rc[ks];
     __syncthreads();
     if (t0 + Q < n) fetch(t0 + Q);
     sm_f32x4 s[2], y[2];
@@ -408,16 +415,15 @@ __global__ __launch_bounds__(512) void ssd_chunk_scan_kernel(
     for (int ct = 0; ct < 2; ++ct) s[ct] = y[ct] = sm_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int ks = 0; ks < NK; ++ks) {
-      const sm_bf16x8 cf = *reinterpret_cast<const sm_bf16x8*>(Cs + (rt * 16 + col) * NS + ks * 32 + kgrp * 8);
 #pragma unroll
       for (int ct = 0; ct < 2; ++ct) {
         const int at = ((hf * 2 + ct) * 16 + col) * NS + ks * 32 + kgrp * 8;
         const sm_bf16x8 bf = *reinterpret_cast<const sm_bf16x8*>(Bs + at);
         const sm_bf16x8 sh = *reinterpret_cast<const sm_bf16x8*>(St + at);
         const sm_bf16x8 sl = *reinterpret_cast<const sm_bf16x8*>(St + 64 * NS + at);
-        s[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, bf, s[ct], 0, 0, 0);
-        y[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, sh, y[ct], 0, 0, 0);
-        y[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, sl, y[ct], 0, 0, 0);
+        s[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf[ks], bf, s[ct], 0, 0, 0);
+        y[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf[ks], sh, y[ct], 0, 0, 0);
+        y[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf[ks], sl, y[ct], 0, 0, 0);
       }
     }
     float ci[4];
