@@ -1348,7 +1348,7 @@ def kikurax_spec_from_config(cfg: dict, name: str, shapes: Optional[dict] = None
 
 
 def _kikurax(name, vocab, width, pattern, heads, kv_heads, dim, vdim, experts, top, ff,
-             left=None, delta=None, ssd=None, conv=4, groups=2, limit=7.0, softcap=50.0,
+             left=None, delta=None, ssd=None, conv=4, groups=2, limit=7.0, softcap=30.0,
              rot_dims=None, rank=None, scaling=(8.0, 1.0, 4.0, 8192.0), **kw):
     """Preset builder. pattern: one letter per layer, p = averaged pair,
     m = Mamba-2, a = attention. left (dim, vdim), delta (heads, kv_heads, dim,
@@ -1359,7 +1359,7 @@ def _kikurax(name, vocab, width, pattern, heads, kv_heads, dim, vdim, experts, t
     for c in pattern:
         if c == "p":
             mixer = AveragedPairSpec(
-                SigmoidAttnSpec(heads, kv_heads, ld, lv, 0.125, 0.3, 512),
+                SigmoidAttnSpec(heads, kv_heads, ld, lv, ld ** -0.5, 0.2, 1024),
                 GatedDeltaSpec(dh, dg, dd, dv, conv, rank or dv, rank or dv))
         elif c == "m":
             mh, mv, mn, mg, ng = ssd
