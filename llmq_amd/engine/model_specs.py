@@ -976,8 +976,8 @@ class TefudraSpec:
         return total
 
 
-def _rotary_from(rc: dict, size: int, where: str) -> RotarySpec:
-    rot = RotarySpec(base=float(rc["base"]), dims=int(rc.get("dims", size)), layout="half")
+def _rotary_from(rc: dict, size: int, where: str, layout: str = "half") -> RotarySpec:
+    rot = RotarySpec(base=float(rc["base"]), dims=int(rc.get("dims", size)), layout=layout)
     if rot.dims % 2 or not 0 <= rot.dims <= size:
         raise ValueError(f"{where}: rot.dims must be even and at most the head size")
     return rot
@@ -1391,6 +1391,247 @@ KIKURAX_PRESETS = {
 }
 
 
+# ---------------------------------------------------------------------------
+# Zarisun: a hybrid decoder on an fp32 residual whose sublayers read the
+# stream itself and are RMS-normed on their OUTPUT only. A layer carries one of
+# three mixers: windowed attention whose values are its convolved keys, a gated
+# delta rule with one decay per head, or latent attention that may share
+# another layer's cached latent; then, unless it has none, a dense gated
+# feed-forward. Both kinds of attention have a softmax sink and a gate per head.
+
+
+@dataclass
+class YarnScaling:
+    """Rotary frequencies of a context stretched by `factor`: pairs that turn
+    more than `fast` times within the `original` context keep their frequency,
+    those that turn less than `slow` times are divided by the factor, a linear
+    ramp over the pair index between; cos and sin are multiplied by
+    `amplitude`."""
+
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+    @property
+    def amplitude(self) -> float:
+        return 0.1 * math.log(self.factor) + 1.0
+
+
+@dataclass
+class ConvKeyAttnSpec:
+    """Softmax attention with grouped kv heads: q and k pass a short causal
+    convolution, the values are the keys as they leave it; q and k are then
+    RMS-normed over the whole projection and rotated. The denominator holds
+    exp(sink_head) as well; attended heads pass a sigmoid gate each. window 0
+    = causal."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    conv: int = 1
+    rot: RotarySpec = None
+    rot_scaling: Optional[YarnScaling] = None
+    window: int = 0
+    kind: str = "attention"
+
+    @property
+    def vdim(self) -> int:
+        return self.dim
+
+
+@dataclass
+class HeadDeltaSpec:
+    """Gated delta rule with ONE decay per head and token: S <- g S,
+    u = beta (v - S^T k), S <- S + k u^T, o = S^T q, with unit q/k behind a
+    short convolution."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int = 1
+    kind: str = "delta"
+
+
+@dataclass
+class SharedLatentAttnSpec(LatentAttnSpec):
+    """Latent attention with a softmax sink and a gate per head; kv_from: the
+    layer whose cached latent and rotated key part this one reads (None: its
+    own)."""
+
+    rot_scaling: Optional[YarnScaling] = None
+    kv_from: Optional[int] = None
+
+
+@dataclass
+class ZarisunLayerSpec:
+    mixer: object     # ConvKeyAttnSpec | HeadDeltaSpec | SharedLatentAttnSpec
+    ff: int = 0       # dense feed-forward inner size (0 = none)
+
+
+@dataclass
+class ZarisunSpec:
+    name: str
+    family: str                   # "zarisun"
+    vocab_size: int
+    hidden_size: int
+    layers: list = field(default_factory=list)
+    rms_eps: float = 1e-6
+    logit_scale: float = 1.0
+    max_position_embeddings: int = 1 << 17
+    tied_embeddings: bool = True
+    eos_token_id: int = 2
+    bos_token_id: int = 1
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def cache_layer(self, i: int) -> int:
+        """The layer whose paged cache layer i attends over."""
+        own = getattr(self.layers[i].mixer, "kv_from", None)
+        return i if own is None else own
+
+    def param_count(self) -> int:
+        w = self.hidden_size
+        total = self.vocab_size * w + w
+        for ls in self.layers:
+            m = ls.mixer
+            total += w
+            if m.kind == "attention":
+                n = (m.heads + m.kv_heads) * m.dim
+                total += n * (w + m.conv + 1) + m.heads * (w + 1) + w * m.heads * m.dim
+            elif m.kind == "delta":
+                n = 2 * m.kv_heads * m.dim + m.heads * m.vdim
+                total += n * (w + m.conv) + 2 * m.heads * (w + 1) + m.vdim
+                total += 2 * w * m.heads * m.vdim
+            else:
+                total += m.heads * (m.dim + m.rot_dim) * w
+                if m.kv_from is None:
+                    total += (m.kv_rank + m.rot_dim) * w + m.kv_rank
+                total += m.heads * (m.dim + m.vdim) * m.kv_rank
+                total += m.heads * (w + 1) + w * m.heads * m.vdim
+            if ls.ff:
+                total += 3 * w * ls.ff + w
+        return total
+
+
+def _yarn_from(rc: dict, where: str) -> Optional[YarnScaling]:
+    sc = rc.get("scaling")
+    if not sc:
+        return None
+    out = YarnScaling(factor=float(sc["factor"]), original=float(sc["original"]),
+                      fast=float(sc["fast"]), slow=float(sc["slow"]))
+    if min(out.factor, out.original, out.fast, out.slow) <= 0:
+        raise ValueError(f"{where}: rot.scaling needs positive numbers")
+    return out
+
+
+def zarisun_spec_from_config(cfg: dict, name: str) -> ZarisunSpec:
+    """Zarisun config.json -> ZarisunSpec: every size and constant comes from
+    the config."""
+    layers = []
+    for i, lc in enumerate(cfg["layers"]):
+        mc, kind, where = lc["mixer"], lc["type"], f"layer {i}"
+        window = int((mc.get("mask") or {}).get("size") or 0)
+        heads, dim = int(mc["heads"]), int(mc["dim"])
+        taps = int(mc.get("conv", 1))
+        if taps < 1:
+            raise ValueError(f"{where}: the convolution needs at least one tap")
+        kv_heads = int(mc.get("kv_heads", heads))
+        if heads % kv_heads:
+            raise ValueError(f"{where}: heads must be a multiple of kv_heads")
+        vdim = int(mc.get("vdim", dim))
+        if kind == "attention":
+            if vdim != dim:
+                raise ValueError(f"{where}: values that are keys have the keys' size")
+            mixer = ConvKeyAttnSpec(
+                heads=heads, kv_heads=kv_heads, dim=dim, conv=taps, window=window,
+                scale=float(mc.get("scale", dim ** -0.5)),
+                rot=_rotary_from(mc["rot"], dim, where, "interleaved"),
+                rot_scaling=_yarn_from(mc["rot"], where))
+        elif kind == "delta":
+            mixer = HeadDeltaSpec(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, conv=taps)
+        elif kind == "latent_attention":
+            rot_dim = int(mc["rot_dim"])
+            mixer = SharedLatentAttnSpec(
+                heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=int(mc["kv_rank"]),
+                scale=float(mc.get("scale", (dim + rot_dim) ** -0.5)), window=window,
+                rot=_rotary_from(mc["rot"], rot_dim, where, "interleaved"),
+                rot_scaling=_yarn_from(mc["rot"], where),
+                kv_from=None if mc.get("kv_from") is None else int(mc["kv_from"]))
+            if mixer.rot.dims < 2:
+                raise ValueError(f"{where}: the rotated part needs at least one pair")
+            if mixer.kv_from is not None:
+                j = mixer.kv_from
+                own = layers[j].mixer if 0 <= j < i else None
+                if getattr(own, "kind", "") != "latent_attention" or own.kv_from is not None:
+                    raise ValueError(f"{where}: kv_from must name an earlier latent layer with "
+                                     "a cache of its own")
+                if (own.kv_rank, own.rot_dim) != (mixer.kv_rank, mixer.rot_dim):
+                    raise ValueError(f"{where}: a shared latent needs equal kv_rank and rot_dim")
+                if (own.rot, own.rot_scaling) != (mixer.rot, mixer.rot_scaling):
+                    raise ValueError(f"{where}: a shared rotated key part needs the same rotation")
+        else:
+            raise ValueError(f"{where}: unknown mixer type {kind!r}")
+        mlp, ff = lc.get("mlp"), 0
+        if mlp is not None:
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"{where}: unknown feed-forward kind {mlp.get('kind')!r}")
+            ff = int(mlp["ff"])
+        layers.append(ZarisunLayerSpec(mixer=mixer, ff=ff))
+    return ZarisunSpec(
+        name=name, family="zarisun", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+        layers=layers, rms_eps=float(cfg["norm"]["eps"]),
+        logit_scale=float(cfg.get("logit_scale", 1.0)))
+
+
+def _zarisun(name, vocab, width, pattern, heads, kv_heads, dim, ff, window, latent, delta, conv=4,
+             rot_dims=None, base=500000.0, scaling=(8.0, 4096.0, 32.0, 1.0), **kw):
+    """Preset builder. pattern: one letter per layer, a = windowed attention,
+    d = delta rule, l = latent attention, s = latent attention on the cache of
+    the latest l. latent (dim, rot_dim, vdim, kv_rank), delta (heads, kv_heads,
+    dim, vdim)."""
+    layers, owner = [], None
+    ld, lr, lv, rank = latent
+    sc = YarnScaling(*scaling)
+    for i, c in enumerate(pattern):
+        if c == "a":
+            mixer = ConvKeyAttnSpec(heads, kv_heads, dim, dim ** -0.5, conv,
+                                    RotarySpec(base, rot_dims or dim, "interleaved"), sc, window)
+        elif c == "d":
+            mixer = HeadDeltaSpec(*delta, conv)
+        else:
+            if c == "l":
+                owner = i
+            mixer = SharedLatentAttnSpec(
+                heads, ld, lr, lv, rank, (ld + lr) ** -0.5, RotarySpec(base, lr, "interleaved"),
+                rot_scaling=sc, kv_from=None if c == "l" else owner)
+        layers.append(ZarisunLayerSpec(mixer, ff))
+    return ZarisunSpec(name=name, family="zarisun", vocab_size=vocab, hidden_size=width,
+                       layers=layers, **kw)
+
+
+ZARISUN_PRESETS = {
+    # CPU/GPU test config: every mixer, grouped heads, partial rotation, a
+    # shared latent, a scaling range the short contexts reach
+    "tiny-zarisun": _zarisun("tiny-zarisun", 512, 64, "adlas", 4, 2, 16, 96, 24,
+                             latent=(12, 8, 20, 40), delta=(4, 2, 8, 24), conv=3, rot_dims=8,
+                             base=1000.0, scaling=(4.0, 64.0, 8.0, 1.0), logit_scale=0.5),
+    # benchmark configs at the layer sizes of llama-3.2-1b / -3b and of the
+    # other hybrid presets: same width, head count, feed-forward and depth; of
+    # every eight layers four windowed attention, two delta rules, one latent
+    # attention and one on its cache (latent and delta sizes as in the
+    # Kosalorn and Kikurax presets)
+    "zarisun-1b": _zarisun("zarisun-1b", 128256, 2048, "aadlaads" * 2, 32, 8, 64, 8192, 2048,
+                           latent=(32, 32, 64, 192), delta=(16, 16, 64, 128)),
+    "zarisun-3b": _zarisun("zarisun-3b", 128256, 3072, "aadlaads" * 3 + "aadl", 24, 8, 128, 8192,
+                           2048, latent=(64, 64, 128, 192), delta=(12, 12, 128, 256)),
+}
+
+
 def spec_from_hf_config(path: Path, name: str) -> ModelSpec:
     """Build a spec from a HF checkpoint directory's config.json."""
     with open(path / "config.json", "r", encoding="utf-8") as fh:
@@ -1401,6 +1642,8 @@ def spec_from_hf_config(path: Path, name: str) -> ModelSpec:
         return muvetar_spec_from_config(cfg, name)
     if str(cfg.get("architecture", "")).lower() == "tefudra":
         return tefudra_spec_from_config(cfg, name)
+    if str(cfg.get("architecture", "")).lower() == "zarisun":
+        return zarisun_spec_from_config(cfg, name)
     if str(cfg.get("architecture", "")).lower() == "kikurax":
         st = path / "model.safetensors"
         return kikurax_spec_from_config(
@@ -1490,7 +1733,9 @@ def resolve_spec(model: str) -> ModelSpec:
         return TEFUDRA_PRESETS[key]
     if key in KIKURAX_PRESETS:
         return KIKURAX_PRESETS[key]
+    if key in ZARISUN_PRESETS:
+        return ZARISUN_PRESETS[key]
     raise ValueError(
         f"Unknown model '{model}'. Provide a checkpoint directory with config.json "
-        f"or one of: {sorted(PRESETS) + sorted(HYBRID_PRESETS) + sorted(KOSALORN_PRESETS) + sorted(MUVETAR_PRESETS) + sorted(TEFUDRA_PRESETS) + sorted(KIKURAX_PRESETS) + sorted(ALIASES)}"
+        f"or one of: {sorted(PRESETS) + sorted(HYBRID_PRESETS) + sorted(KOSALORN_PRESETS) + sorted(MUVETAR_PRESETS) + sorted(TEFUDRA_PRESETS) + sorted(KIKURAX_PRESETS) + sorted(ZARISUN_PRESETS) + sorted(ALIASES)}"
     )

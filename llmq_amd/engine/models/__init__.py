@@ -6,6 +6,7 @@ from llmq_amd.engine.models.kosalorn import KosalornLM
 from llmq_amd.engine.models.llama import CausalLM
 from llmq_amd.engine.models.muvetar import MuvetarLM
 from llmq_amd.engine.models.tefudra import TefudraLM
+from llmq_amd.engine.models.zarisun import ZarisunLM
 
 MODEL_CLASSES = {
     "llama": CausalLM,
@@ -17,6 +18,7 @@ MODEL_CLASSES = {
     "kosalorn": KosalornLM,
     "muvetar": MuvetarLM,
     "tefudra": TefudraLM,
+    "zarisun": ZarisunLM,
 }
 
 
@@ -27,4 +29,5 @@ def model_class_for(spec):
         raise ValueError(f"no model class registered for family {spec.family!r}") from None
 
 
-__all__ = ["CausalLM", "KakovikLM", "KikuraxLM", "KosalornLM", "MuvetarLM", "TefudraLM", "MODEL_CLASSES", "model_class_for"]
+__all__ = ["CausalLM", "KakovikLM", "KikuraxLM", "KosalornLM", "MuvetarLM", "TefudraLM",
+           "ZarisunLM", "MODEL_CLASSES", "model_class_for"]

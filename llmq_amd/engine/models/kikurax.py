@@ -59,24 +59,8 @@ import torch.nn.functional as F
 from llmq_amd import ops
 from llmq_amd.engine.forward_meta import DecodeMeta, MixedMeta, PrefillMeta
 from llmq_amd.engine.kv_cache import KVCache
-from llmq_amd.engine.model_specs import KikuraxSpec, RotaryScaling
-from llmq_amd.engine.models.kosalorn import rotary_inv_freq
-
-
-def scaled_inv_freq(base: float, dims: int, scaling: Optional[RotaryScaling]) -> torch.Tensor:
-    """fp32 rotary table base^(-2i/dims) with the wavelength-dependent
-    slowdown applied in float64 and rounded once."""
-    if scaling is None:
-        return rotary_inv_freq(base, dims)
-    i = torch.arange(dims // 2, dtype=torch.float64)
-    f = torch.pow(torch.tensor(base, dtype=torch.float64), -2.0 * i / dims)
-    wave = 2.0 * math.pi / f
-    blend = (scaling.original / wave - scaling.low) / (scaling.high - scaling.low) \
-        if scaling.high != scaling.low else torch.zeros_like(f)
-    mid = (1.0 - blend) * f / scaling.factor + blend * f
-    out = torch.where(wave < scaling.original / scaling.high, f,
-                      torch.where(wave > scaling.original / scaling.low, f / scaling.factor, mid))
-    return out.to(torch.float32)
+from llmq_amd.engine.model_specs import KikuraxSpec
+from llmq_amd.engine.models.rotary import scaled_inv_freq
 
 
 class KikuraxLayerWeights:

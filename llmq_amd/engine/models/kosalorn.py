@@ -53,12 +53,7 @@ from llmq_amd import ops
 from llmq_amd.engine.forward_meta import DecodeMeta, MixedMeta, PrefillMeta
 from llmq_amd.engine.kv_cache import KVCache
 from llmq_amd.engine.model_specs import KosalornSpec
-
-
-def rotary_inv_freq(base: float, dims: int) -> torch.Tensor:
-    """fp32 table base^(-2i/dims), i < dims/2, rounded once from float64."""
-    i = torch.arange(dims // 2, dtype=torch.float64)
-    return torch.pow(torch.tensor(base, dtype=torch.float64), -2.0 * i / dims).to(torch.float32)
+from llmq_amd.engine.models.rotary import rotary_inv_freq
 
 
 class KosalornLayerWeights:
@@ -156,7 +151,7 @@ class KosalornLM:
                 segs.append(("dkv", m.kv_rank + m.rot_dim))
                 t["dkv_norm"] = self._empty(m.kv_rank)
                 t["uk"] = self._empty(m.heads, m.dim, m.kv_rank)     # [H, dim, R]
-                t["uv"] = self._empty(m.heads, m.vdim, m.kv_rank)    # [H, vdim, R]
+                t["uv"] = self._empty(m.heads, m.kv_rank, m.vdim)    # [H, R, vdim]
                 t["o"] = self._empty(W, m.heads * m.vdim)
             segs += [("rg1", W)]
             if ls.ff or ls.moe:
@@ -236,6 +231,8 @@ class KosalornLM:
                     for at, n in lw.seg.values():
                         keep[at:at + n] = True
                     t[~keep.to(t.device)] = 0
+                elif name == "uv":
+                    fill(t, 1.0 / math.sqrt(t.shape[1]))
                 else:
                     fill(t, 1.0 / math.sqrt(t.shape[-1]))
         self.finalize()
@@ -291,7 +288,7 @@ class KosalornLM:
             ctx = ops.window_attn_decode(
                 qf, kc, None, R, meta.block_tables, meta.context_lens, m.window, m.scale)
         # values: W_uv on the attended latent, per head
-        o = torch.bmm(ctx.transpose(0, 1), lw.t["uv"].transpose(1, 2))   # [H, T, vdim]
+        o = torch.bmm(ctx.transpose(0, 1), lw.t["uv"])   # [H, T, vdim]
         return F.linear(o.transpose(0, 1).reshape(T, H * m.vdim), lw.t["o"])
 
     def _hgrn2(self, p, lw, m, run, kv_cache, meta):

@@ -59,7 +59,7 @@ from llmq_amd import ops
 from llmq_amd.engine.forward_meta import DecodeMeta, MixedMeta, PrefillMeta
 from llmq_amd.engine.kv_cache import KVCache
 from llmq_amd.engine.model_specs import TefudraSpec
-from llmq_amd.engine.models.kosalorn import rotary_inv_freq
+from llmq_amd.engine.models.rotary import rotary_inv_freq
 
 
 class TefudraLayerWeights:

@@ -232,7 +232,7 @@ def load_kosalorn_weights(model, path: Path) -> None:
             put("dkv", get(mx + "dkv"))
             copy_(t["dkv_norm"], get(mx + "dkv.norm"))
             copy_(t["uk"], get(mx + "uk").view(m.heads, m.dim, m.kv_rank))
-            copy_(t["uv"], get(mx + "uv").view(m.heads, m.vdim, m.kv_rank))
+            copy_(t["uv"], get(mx + "uv").view(m.heads, m.vdim, m.kv_rank).transpose(1, 2))
         copy_(t["o"], get(mx + "o"))
         put("rg1", get(p + "rg1"))
         copy_(t["rg1_b"], get(p + "rg1.b"))
@@ -533,6 +533,75 @@ def load_kikurax_weights(model, path: Path) -> None:
     logger.info("loaded %d tensors from %s", len(tensors), path)
 
 
+def load_zarisun_weights(model, path: Path) -> None:
+    """Zarisun checkpoint names -> the packed in-tree tensors.
+
+    Checkpoint: 'embed' (also the output head), 'final.norm', and per layer
+    'l<i>.norm1', '.norm2' (of the sublayers' outputs), the mixer under
+    'l<i>.mix.', the feed-forward under 'l<i>.mlp.'; linear weights are
+    [out, in], a projection's norm weight is its name + '.norm', its short
+    convolution's taps its name + '.conv'. Packing: everything that reads the
+    mixer's input -> 'in' (taps -> 'conv_w', segments at multiples of 8 rows),
+    gate‖up -> one tensor, per-head latent maps [H, dim, R] and [H, R, vdim];
+    what enters softmax denominators and decays -> fp32."""
+    tensors = _read_all(path)
+    used = set()
+
+    def get(name: str) -> torch.Tensor:
+        if name not in tensors:
+            raise KeyError(f"missing tensor {name}")
+        used.add(name)
+        return tensors[name]
+
+    def copy_(dst: torch.Tensor, src: torch.Tensor) -> None:
+        if dst.shape != src.shape:
+            raise ValueError(f"shape mismatch: {tuple(dst.shape)} vs {tuple(src.shape)}")
+        dst.copy_(src.to(dst.dtype))
+
+    spec = model.spec
+    copy_(model.embedding, get("embed"))
+    copy_(model.final_norm, get("final.norm"))
+    for i, (ls, lw) in enumerate(zip(spec.layers, model.layers)):
+        p, t, m = f"l{i}.", lw.t, ls.mixer
+        mx = p + "mix."
+        copy_(t["norm1"], get(p + "norm1"))
+
+        def put(seg: str, src: torch.Tensor, dst: str = "in", lw=lw, t=t) -> None:
+            at, n = lw.seg[seg]
+            copy_(t[dst][at:at + n], src)
+
+        for name in ("in", "conv_w"):                       # alignment rows between segments
+            if name in t:
+                t[name].zero_()
+        for seg in lw.seg:
+            put(seg, get(mx + seg))
+            if "conv_w" in t and lw.seg[seg][0] < lw.conv_cols:
+                put(seg, get(mx + seg + ".conv"), "conv_w")
+        copy_(t["o"], get(mx + "o"))
+        if m.kind == "attention":
+            copy_(t["q_norm"], get(mx + "q.norm"))
+            copy_(t["k_norm"], get(mx + "k.norm"))
+            copy_(t["sink"], get(mx + "sink"))
+        elif m.kind == "delta":
+            for name in ("A_log", "dt_bias", "norm"):
+                copy_(t[name], get(mx + name))
+        else:
+            if m.kv_from is None:
+                copy_(t["dkv_norm"], get(mx + "dkv.norm"))
+            copy_(t["uk"], get(mx + "uk").view(m.heads, m.dim, m.kv_rank))
+            copy_(t["uv"], get(mx + "uv").view(m.heads, m.vdim, m.kv_rank).transpose(1, 2))
+            copy_(t["sink"], get(mx + "sink"))
+        if ls.ff:
+            copy_(t["norm2"], get(p + "norm2"))
+            copy_(t["gate_up"], torch.cat([get(p + "mlp.gate"), get(p + "mlp.up")], dim=0))
+            copy_(t["down"], get(p + "mlp.down"))
+    unused = sorted(set(tensors) - used)
+    if unused:
+        logger.warning("checkpoint tensors this configuration does not use: %s", unused[:8])
+    model.finalize()
+    logger.info("loaded %d tensors from %s", len(tensors), path)
+
+
 _FAMILY_LOADERS = {"kakovik": load_kakovik_weights, "kikurax": load_kikurax_weights,
                    "kosalorn": load_kosalorn_weights, "muvetar": load_muvetar_weights,
-                   "tefudra": load_tefudra_weights}
+                   "tefudra": load_tefudra_weights, "zarisun": load_zarisun_weights}

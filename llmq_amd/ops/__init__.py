@@ -413,10 +413,11 @@ def rmsnorm_cast(x: torch.Tensor, weight: torch.Tensor, eps: float, offset: floa
 
 
 def sandwich_norm_res32(x: torch.Tensor, residual: torch.Tensor, w_post: torch.Tensor,
-                        w_pre: torch.Tensor, eps: float, offset: float,
+                        w_pre: Optional[torch.Tensor], eps: float, offset: float,
                         groups: int = 1) -> torch.Tensor:
     """residual (fp32, in place) += rmsnorm(x)·(w_post+offset); returns
-    rmsnorm(residual)·(w_pre+offset) in x's dtype (x's storage on GPU).
+    rmsnorm(residual)·(w_pre+offset) in x's dtype (x's storage on GPU), or with
+    w_pre None the residual itself, rounded (a sublayer that reads the stream).
     groups > 1: both norms work on that many equal parts of a row."""
     if _use_hybrid(x):
         _HY.sandwich_norm_res32(x, residual, w_post, w_pre, eps, offset, int(groups))
@@ -567,17 +568,17 @@ def window_attn_decode(q, k_cache, v_cache, dv: int, block_tables, context_lens,
         bias_mode = _BIAS_LOG if log_bias is not None else _BIAS_TABLE
         keep = int(keep_first) if window else 0
         if (q.dtype == torch.bfloat16 and k_cache.shape[1] == 1 and H >= 8 and D % 8 == 0
-                and D <= 256 and q.is_contiguous() and log_bias is None and not keep
-                and sink is None and not softcap and gate is None and not sigmoid):
+                and D <= 256 and dv <= 256 and q.is_contiguous() and log_bias is None and not keep
+                and not softcap and (gate is None or gate.shape[1] == H) and not sigmoid):
             # one kv head for all query heads: the heads of a token become the
             # rows of one head, all at the token's position, and the step runs
             # on the matrix-core kernel — every key tile staged once for all
-            # heads instead of once per head group
+            # heads instead of once per head group; sink and gate go by row
             cu = _head_row_offsets(B, H, q.device)
-            _HY.paged_attn_prefill(out.view(B * H, 1, dv), q.view(B * H, 1, D), None, k_cache,
+            _HY.paged_attn_prefill(out.view(B * H, 1, dv), q.view(B * H, 1, D), gate, k_cache,
                                    v_cache, None, block_tables, cu, context_lens - 1, H,
                                    int(window) or _NO_WINDOW, float(scale), _MASK_WINDOW, 0,
-                                   _BIAS_TABLE, 0, None, 0.0)
+                                   _BIAS_TABLE, 0, sink, 0.0)
             return out
         _HY.paged_attn_decode(out, q, gate, k_cache, v_cache, log_bias, block_tables,
                               context_lens, int(window) or _NO_WINDOW, float(scale), _MASK_WINDOW,
@@ -603,20 +604,26 @@ def _head_row_offsets(B: int, H: int, device) -> torch.Tensor:
 
 
 def latent_rope_pack(q, q_lat, ckr, c_w, inv_freq, positions, k_cache, slots, dim: int,
-                     rot_dims: int, interleaved: bool, eps: float) -> torch.Tensor:
+                     rot_dims: int, interleaved: bool, eps: float, amplitude: float = 1.0,
+                     out=None) -> torch.Tensor:
     """Latent attention, between the projections and the attention kernel:
-    rotary positions (fp32 angles position * inv_freq[i]) on the rotated part
-    of q [T, H, dim+DR] and of ckr [T, R+DR], RMSNorm of the latent, the
-    packed query q_lat ‖ rotated part [T, H, R+DR] returned, and latent ‖
-    rotated key part scattered into the paged cache [blocks, 1, bs, R+DR]."""
+    rotary positions (fp32 angles position * inv_freq[i], cos and sin times
+    amplitude) on the rotated part of q [T, H, dim+DR] and of ckr [T, R+DR],
+    RMSNorm of the latent, the packed query q_lat ‖ rotated part [T, H, R+DR]
+    returned, and latent ‖ rotated key part scattered into the paged cache
+    [blocks, 1, bs, R+DR]. With out [T, H, R+DR] (its first R channels filled,
+    q_lat None) the query is packed there; ckr None: the layer caches nothing
+    of its own."""
     if _use_hybrid(q):
-        T, H, _ = q.shape
-        out = torch.empty(T, H, ckr.shape[1], dtype=q.dtype, device=q.device)
+        if out is None:
+            T, H, _ = q.shape
+            out = torch.empty(T, H, q_lat.shape[2] + q.shape[2] - dim, dtype=q.dtype, device=q.device)
         _HY.latent_rope_pack(out, q, q_lat, ckr, c_w, inv_freq, positions, k_cache, slots,
-                             int(dim), int(rot_dims), bool(interleaved), float(eps))
+                             int(dim), int(rot_dims), bool(interleaved), float(eps),
+                             float(amplitude))
         return out
     return torch_ref.latent_rope_pack(q, q_lat, ckr, c_w, inv_freq, positions, k_cache, slots,
-                                      dim, rot_dims, interleaved, eps)
+                                      dim, rot_dims, interleaved, eps, amplitude, out)
 
 
 def gated_residual_add(res, y1, g1, b1, y2, g2, b2, out_dtype: torch.dtype) -> torch.Tensor:
@@ -919,6 +926,27 @@ def qkv_norm_rope_cache(q, k, v, q_w, k_w, inv_freq, rot_dims: int, positions, k
                                   head_scale, temp_coef, temp_every, v_first, mix)
 
 
+def rownorm_rope_cache(q, k, q_w, k_w, inv_freq, rot_dims: int, positions, k_cache, v_cache, slots,
+                       eps: float, amplitude: float = 1.0, conv=None) -> None:
+    """Per token, between the projections and the attention kernel, for q
+    [T, H, D] (in place) and k [T, G, D] that are RMS-normed over all their
+    heads at once (weights [H*D], [G*D]): rotary positions on the first
+    rot_dims channels of every head in adjacent pairs (2i, 2i+1), cos and sin
+    times amplitude; k goes to the key cache and the keys as they arrive to the
+    value cache. conv = (weight fp32 [C, K], tail [slots, K-1, C], slots,
+    fresh, q_at, k_at): every row is its sequence's only one, and q and k
+    (channels from q_at / k_at on) first pass the short causal convolution
+    whose tail is advanced in place."""
+    if _use_hybrid(q):
+        w, tail, rec_slots, fresh, q_at, k_at = conv or (None, None, None, None, 0, 0)
+        _HY.rownorm_rope_cache(q, k, q_w, k_w, inv_freq, int(rot_dims), float(amplitude), positions,
+                               k_cache, v_cache, slots, float(eps), w, tail, rec_slots, fresh,
+                               int(q_at), int(k_at))
+        return
+    torch_ref.rownorm_rope_cache(q, k, q_w, k_w, inv_freq, rot_dims, positions, k_cache, v_cache,
+                                 slots, eps, amplitude, conv)
+
+
 def rotate_heads(x, positions, inv_freq, inverse: bool = False) -> torch.Tensor:
     """x [T, H, n] in place: every head turned by its token's position (by
     minus the position if inverse) over all n channels, pairs (i, i + n/2),
@@ -994,11 +1022,11 @@ def unary_act(x, kind: str) -> torch.Tensor:
 def gated_delta_rule(q, k, v, z, z_bias, rate, beta, state, cu, slots, fresh,
                      q_scale: float) -> torch.Tensor:
     """Gated delta rule over packed sequences, per head h (which reads q/k
-    head h // (H / Hk)): g = exp(-rate_h softplus(z + z_bias)) per key channel,
+    head h // (H / Hk)): g = exp(-rate_h softplus(z + z_bias)) per key channel
+    (z [T, H, D], z_bias fp32 [H*D]) or per head (z [T, H], z_bias fp32 [H]),
     S <- diag(g) S, u = sigmoid(beta) (v - S^T k), S <- S + k u^T,
     o = S^T (q_scale q), with q and k divided by sqrt(sum of squares + 1e-6).
-    q, k [T, Hk, D]; v [T, H, DV]; z [T, H, D]; beta [T, H]; z_bias fp32
-    [H*D]; rate fp32 [H]; state [slots, H, D, DV] fp32 advanced in place.
+    q, k [T, Hk, D]; v [T, H, DV]; beta [T, H]; rate fp32 [H]; state [slots, H, D, DV] fp32 advanced in place.
     Returns o [T, H, DV] fp32."""
     if _use_hybrid(q):
         o = torch.empty(v.shape, dtype=torch.float32, device=q.device)

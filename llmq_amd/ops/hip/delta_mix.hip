@@ -13,7 +13,8 @@
 
 // ------------------------------------------------------- gated delta rule ----
 // Per sequence and head, state S [D, DV] fp32 in a per-sequence slot:
-//   g_t = exp(-rate_h * softplus(z_t + z_bias)) per key channel,
+//   g_t = exp(-rate_h * softplus(z_t + z_bias)) per key channel, or one number
+//         for all of them (HEAD_DECAY: z [T, H], z_bias [H]),
 //   S <- diag(g_t) S;  u = sigmoid(beta_t) (v_t - S^T k_t);  S <- S + k_t u^T;
 //   o_t = S^T q_t,
 // with k_t and q_t unit vectors (x / sqrt(sum x^2 + 1e-6), q times q_scale).
@@ -57,12 +58,12 @@ DEVINL float softplus_f(float x) {
   return fmaxf(x, 0.f) + t;
 }
 
-template <typename T, int DPL, int NC>
+template <typename T, int DPL, int NC, bool HEAD_DECAY>
 __global__ __launch_bounds__(256) void gated_delta_kernel(
     float* __restrict__ o,                                  // [T, H, DV]
     const T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride,
     const T* __restrict__ v, long v_stride, const T* __restrict__ z, long z_stride,
-    const float* __restrict__ z_bias,                       // [H * D]
+    const float* __restrict__ z_bias,                       // [H * D] or [H]
     const float* __restrict__ rate,                         // [H]
     const T* __restrict__ beta, long b_stride,              // [T, H]
     float* __restrict__ state,                              // [slots, H, D, DV]
@@ -75,7 +76,7 @@ __global__ __launch_bounds__(256) void gated_delta_kernel(
   constexpr int COLS = 16 * NC;                // value columns per workgroup
   __shared__ __align__(16) float qs[kDeltaTB * DP];
   __shared__ __align__(16) float ks[kDeltaTB * DP];
-  __shared__ __align__(16) float gs[kDeltaTB * DP];
+  __shared__ __align__(16) float gs[HEAD_DECAY ? kDeltaTB : kDeltaTB * DP];
   __shared__ __align__(16) float vs[kDeltaTB * COLS];
   __shared__ float bs[kDeltaTB], kq[kDeltaTB];
   const int b = blockIdx.z, h = blockIdx.y, hk = h / hpk;
@@ -108,24 +109,28 @@ __global__ __launch_bounds__(256) void gated_delta_kernel(
   // staging: thread = (token tid / 16, lane l of its row): the row's granules
   // of q, k and z, NC of the v columns
   const int st = tid >> 4;
-  float zb[DPL];
+  constexpr int NZ = HEAD_DECAY ? 1 : DPL;     // decay logits per lane and token
+  float zb[NZ];
 #pragma unroll
-  for (int i = 0; i < DPL; ++i) zb[i] = chan(i) < D ? z_bias[h * D + chan(i)] : 0.f;
+  for (int i = 0; i < NZ; ++i)
+    zb[i] = HEAD_DECAY ? z_bias[h] : chan(i) < D ? z_bias[h * D + chan(i)] : 0.f;
   const float rt = rate[h];
-  float rq[DPL], rk[DPL], rz[DPL], rv[NC], rb = 0.f;
+  float rq[DPL], rk[DPL], rz[NZ], rv[NC], rb = 0.f;
   auto fetch = [&](int t0) {
     const bool live = t0 + st < n;
     const long row = row0 + t0 + st;
 #pragma unroll
     for (int i = 0; i < DPL; ++i) {
       const int d = chan(i);
-      rq[i] = rk[i] = rz[i] = 0.f;
+      rq[i] = rk[i] = 0.f;
+      if constexpr (!HEAD_DECAY) rz[i] = 0.f;
       if (live && d < D) {
         rq[i] = to_f32(q[row * q_stride + (long)hk * D + d]);
         rk[i] = to_f32(k[row * k_stride + (long)hk * D + d]);
-        rz[i] = to_f32(z[row * z_stride + (long)h * D + d]);
+        if constexpr (!HEAD_DECAY) rz[i] = to_f32(z[row * z_stride + (long)h * D + d]);
       }
     }
+    if constexpr (HEAD_DECAY) rz[0] = live ? to_f32(z[row * z_stride + h]) : 0.f;
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       const int gc = blockIdx.x * COLS + l * NC + c;
@@ -152,16 +157,22 @@ __global__ __launch_bounds__(256) void gated_delta_kernel(
 #pragma unroll
       for (int i = 0; i < DPL; ++i) {
         const int at = st * DP + chan(i);
-        const float sp = softplus_f<FAST>(rz[i] + zb[i]);
         qs[at] = rq[i] * iq;
         ks[at] = rk[i] * ik;
-        gs[at] = FAST ? __expf(-rt * sp) : expf(-rt * sp);
+        if constexpr (!HEAD_DECAY) {
+          const float sp = softplus_f<FAST>(rz[i] + zb[i]);
+          gs[at] = FAST ? __expf(-rt * sp) : expf(-rt * sp);
+        }
       }
 #pragma unroll
       for (int c = 0; c < NC; ++c) vs[st * COLS + l * NC + c] = rv[c];
       if (l == 0) {
         bs[st] = 1.0f / (1.0f + (FAST ? __expf(-rb) : expf(-rb)));
         kq[st] = sqk * iq * ik;
+        if constexpr (HEAD_DECAY) {
+          const float sp = softplus_f<FAST>(rz[0] + zb[0]);
+          gs[st] = FAST ? __expf(-rt * sp) : expf(-rt * sp);
+        }
       }
     }
     __syncthreads();
@@ -170,12 +181,15 @@ __global__ __launch_bounds__(256) void gated_delta_kernel(
       float kk[DPL], pk[NC], pq[NC];
 #pragma unroll
       for (int c = 0; c < NC; ++c) pk[c] = pq[c] = 0.f;
+      float gh = 1.f;
+      if constexpr (HEAD_DECAY) gh = gs[tt];
 #pragma unroll
       for (int g = 0; g < NG; ++g) {
         const int at = tt * DP + (g * 16 + l) * GW;
         float ga[GW], qa[GW];
         if constexpr (GW == 4) {
-          const float4 g4 = *reinterpret_cast<const float4*>(gs + at);
+          const float4 g4 = HEAD_DECAY ? make_float4(gh, gh, gh, gh)
+                                       : *reinterpret_cast<const float4*>(gs + at);
           const float4 k4 = *reinterpret_cast<const float4*>(ks + at);
           const float4 q4 = *reinterpret_cast<const float4*>(qs + at);
           ga[0] = g4.x; ga[1] = g4.y; ga[2] = g4.z; ga[3] = g4.w;
@@ -184,7 +198,7 @@ __global__ __launch_bounds__(256) void gated_delta_kernel(
         } else {
 #pragma unroll
           for (int e = 0; e < GW; ++e) {
-            ga[e] = gs[at + e];
+            ga[e] = HEAD_DECAY ? gh : gs[at + e];
             kk[g * GW + e] = ks[at + e];
             qa[e] = qs[at + e];
           }

@@ -68,9 +68,13 @@ void rmsnorm_cast(at::Tensor out, at::Tensor in, at::Tensor weight, double eps, 
   });
 }
 
-void sandwich_norm_res32(at::Tensor x, at::Tensor residual, at::Tensor w_post, at::Tensor w_pre,
-                         double eps, double offset, int64_t groups_arg) {
+// w_pre none: x becomes the residual itself, rounded
+void sandwich_norm_res32(at::Tensor x, at::Tensor residual, at::Tensor w_post,
+                         const std::optional<at::Tensor>& w_pre_opt, double eps, double offset,
+                         int64_t groups_arg) {
   HY_GPU(x);
+  const bool has_pre = w_pre_opt.has_value();
+  const at::Tensor& w_pre = has_pre ? *w_pre_opt : w_post;   // stands in for the checks
   TORCH_CHECK(x.is_contiguous() && residual.is_contiguous());
   TORCH_CHECK(residual.scalar_type() == at::kFloat, "residual must be fp32");
   const int width = x.size(-1);
@@ -89,8 +93,8 @@ void sandwich_norm_res32(at::Tensor x, at::Tensor residual, at::Tensor w_post, a
       hipLaunchKernelGGL((sandwich_norm_res32_vec_kernel<CH, PER_WAVE>), dim3(blocks), dim3(256), 0,
                          hy_stream(), reinterpret_cast<bf*>(x.data_ptr()), residual.data_ptr<float>(),
                          reinterpret_cast<const bf*>(w_post.data_ptr()),
-                         reinterpret_cast<const bf*>(w_pre.data_ptr()), hidden, (float)eps,
-                         (float)offset, groups, rows);
+                         has_pre ? reinterpret_cast<const bf*>(w_pre.data_ptr()) : nullptr, hidden,
+                         (float)eps, (float)offset, groups, rows);
     };
     // short rows (and the parts of rows normed in groups): a wave per row
     if (hidden <= 512) launch.template operator()<1, true>();
@@ -104,8 +108,8 @@ void sandwich_norm_res32(at::Tensor x, at::Tensor residual, at::Tensor w_post, a
     hipLaunchKernelGGL(sandwich_norm_res32_kernel<T>, dim3(rows), dim3(256), 0, hy_stream(),
                        reinterpret_cast<T*>(x.data_ptr()), residual.data_ptr<float>(),
                        reinterpret_cast<const T*>(w_post.data_ptr()),
-                       reinterpret_cast<const T*>(w_pre.data_ptr()), hidden, (float)eps,
-                       (float)offset, groups);
+                       has_pre ? reinterpret_cast<const T*>(w_pre.data_ptr()) : nullptr, hidden,
+                       (float)eps, (float)offset, groups);
   });
 }
 
@@ -273,16 +277,28 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
                         int64_t keep_first, const std::optional<at::Tensor>& sink, double softcap,
                         int64_t weight_fn, const std::optional<at::Tensor>& wbias) {
   if (q.size(0) == 0) return;
-  const float* sink_ptr = sink_check(sink, q);
+  TORCH_CHECK(pos_stride == 0 || pos_stride == 1, "pos_stride is 0 (rows share a position) or 1");
+  // rows that share a position are the query heads of one token per sequence:
+  // sink [rows] and gate [sequences, rows] belong to the rows
+  const bool shared = pos_stride == 0;
+  if (shared) {
+    TORCH_CHECK(q.size(1) == 1 && q.size(0) == q_start.numel() * max_q,
+                "rows that share a position: max_q rows of one head per sequence");
+    TORCH_CHECK(!sink.has_value() || (sink->is_cuda() && sink->scalar_type() == at::kFloat &&
+                sink->is_contiguous() && sink->numel() == max_q), "sink must be fp32 [rows] on the GPU");
+    TORCH_CHECK(!gate.has_value() || (gate->is_cuda() && gate->dim() == 2 &&
+                gate->size(0) == q_start.numel() && gate->size(1) == max_q && gate->stride(1) == 1 &&
+                gate->scalar_type() == q.scalar_type()), "gate must be [sequences, rows]");
+  }
+  const float* sink_ptr = !shared ? sink_check(sink, q)
+                                  : sink.has_value() ? sink->data_ptr<float>() : nullptr;
   const float* wbias_ptr = wbias_check(weight_fn, wbias, sink, q);
   TORCH_CHECK(pos_stride == 1 || weight_fn == kWeightSoftmax,
               "rows that share a position take softmax weights");
   TORCH_CHECK(keep_first >= 0 && softcap >= 0.0);
   TORCH_CHECK(keep_first == 0 || mask_mode == kMaskWindow, "kept first tokens go with the window mask");
-  TORCH_CHECK(pos_stride == 1 || (keep_first == 0 && !sink_ptr),
-              "rows that share a position take no kept tokens and no sink");
-  TORCH_CHECK(pos_stride == 0 || pos_stride == 1, "pos_stride is 0 (rows share a position) or 1");
-  const AttnDims a = attn_check(out, q, gate, k_cache, v_cache, bias, block_tables, span, mask_mode,
+  TORCH_CHECK(!shared || keep_first == 0, "rows that share a position take no kept tokens");
+  const AttnDims a = attn_check(out, q, shared ? std::optional<at::Tensor>() : gate, k_cache, v_cache, bias, block_tables, span, mask_mode,
                                 bias_mode);
   HY_I32(cu_q); HY_I32(q_start);
   const int B = q_start.numel();
@@ -294,7 +310,7 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
     return e && e[0] == '1';
   }();
   TORCH_CHECK(pos_stride == 1 || (q.scalar_type() == at::kBFloat16 && a.D % 8 == 0 && a.D <= 256 &&
-                                  q.stride(0) % 8 == 0 && !gate.has_value()),
+                                  a.DV <= 256 && q.stride(0) % 8 == 0),
               "rows that share a position run on the matrix-core kernel only");
   if (q.scalar_type() == at::kBFloat16 && (!force_valu || pos_stride == 0) && a.D % 8 == 0 && a.D <= 256 &&
       a.DV <= 256 &&   // 16 channel tiles of 16 per wave; wider values run on the fp32 ALUs
@@ -345,14 +361,20 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
       const long pairs = q.size(0) * (long)a.H;
       hipLaunchKernelGGL(attn_merge_splits_kernel, dim3((pairs + 3) / 4), dim3(256), 0, hy_stream(),
                          reinterpret_cast<bf*>(out.data_ptr()), out.stride(0),
-                         part.data_ptr<float>(), pairs, a.H, a.DV, n_split);
+                         part.data_ptr<float>(), pairs, a.H, a.DV, n_split, sink_ptr,
+                         gate.has_value() ? reinterpret_cast<const bf*>(gate->data_ptr()) : nullptr,
+                         gate.has_value() ? gate->stride(0) : 0L, (int)max_q);
     }
     return;
   }
   const bool alias = a.vptr == k_cache.data_ptr();
-  const size_t lds = sizeof(float) * ((size_t)kAttnKT * (a.D + 1) +
-                                      (alias ? 0 : (size_t)kAttnKT * a.DV) +
-                                      (size_t)kAttnQT * a.D + (size_t)kAttnQT * kAttnKT);
+  TORCH_CHECK(!shared, "rows that share a position run on the matrix-core kernel only");
+  auto lds_for = [&](int keys) {
+    return sizeof(float) * ((size_t)keys * (a.D + 1) + (alias ? 0 : (size_t)keys * a.DV) +
+                            (size_t)kAttnQT * a.D + (size_t)kAttnQT * kAttnKT);
+  };
+  const int kt_n = lds_for(kAttnKT) <= 160 * 1024 ? kAttnKT : kAttnKT / 2;
+  const size_t lds = lds_for(kt_n);
   const dim3 grid((max_q + kAttnQT - 1) / kAttnQT, a.H, B);
   hy_dispatch(q, "chunk_bias_attn_prefill", [&]<typename T>() {
     dispatch_nv(a.DV, [&]<int NV>() {
@@ -369,7 +391,7 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
                          cu_q.data_ptr<int>(), q_start.data_ptr<int>(), a.H, a.G, a.D, a.DV, a.bs,
                          (int)span, (float)scale, a.v_row, (int)mask_mode, (int)bias_mode,
                          (int)keep_first, sink_ptr, (float)softcap, a.gate_cols, (int)weight_fn,
-                         wbias_ptr);
+                         wbias_ptr, kt_n);
     });
   });
 }
@@ -514,43 +536,55 @@ void gla_out_norm_gate(at::Tensor out, at::Tensor o, at::Tensor weight,
   });
 }
 
-// ---- latent attention: rotary + latent norm + packed query + cache scatter
-void latent_rope_pack(at::Tensor out, at::Tensor q, at::Tensor q_lat, at::Tensor ckr,
-                      at::Tensor c_w, at::Tensor inv_freq, at::Tensor positions,
-                      at::Tensor k_cache, at::Tensor slots, int64_t dim, int64_t rot_dims,
-                      bool interleaved, double eps) {
+// ---- latent attention: rotary + latent norm + packed query + cache scatter.
+// q_lat none: out[..., :R] is written already. ckr (and c_w, k_cache) none: the
+// layer reads rows another layer cached, only the query is packed.
+void latent_rope_pack(at::Tensor out, at::Tensor q, const std::optional<at::Tensor>& q_lat,
+                      const std::optional<at::Tensor>& ckr, const std::optional<at::Tensor>& c_w,
+                      at::Tensor inv_freq, at::Tensor positions,
+                      const std::optional<at::Tensor>& k_cache, at::Tensor slots, int64_t dim,
+                      int64_t rot_dims, bool interleaved, double eps, double amplitude) {
   HY_GPU(q);
   const long T_ = q.size(0);
   if (T_ == 0) return;
-  TORCH_CHECK(q.dim() == 3 && q_lat.dim() == 3 && ckr.dim() == 2 && out.dim() == 3);
-  HY_INNER(q); HY_INNER(q_lat); HY_INNER(ckr);
-  const int H = q.size(1), R = q_lat.size(2);
-  const int DR = (int)q.size(2) - (int)dim;
-  TORCH_CHECK(dim >= 0 && DR >= 1, "q must be [T, H, dim + rot part]");
-  TORCH_CHECK(q_lat.size(0) == T_ && q_lat.size(1) == H && ckr.size(0) == T_ && ckr.size(1) == R + DR);
-  TORCH_CHECK(out.is_contiguous() && out.size(0) == T_ && out.size(1) == H && out.size(2) == R + DR);
+  TORCH_CHECK(q.dim() == 3 && out.dim() == 3);
+  HY_INNER(q);
+  const int H = q.size(1);
+  const int DR = (int)q.size(2) - (int)dim, R = (int)out.size(2) - DR;
+  const auto dt = q.scalar_type();
+  TORCH_CHECK(dim >= 0 && DR >= 1 && R >= 1, "q must be [T, H, dim + rot part]");
+  TORCH_CHECK(out.is_contiguous() && out.size(0) == T_ && out.size(1) == H && out.scalar_type() == dt);
   TORCH_CHECK(rot_dims >= 2 && rot_dims % 2 == 0 && rot_dims <= DR, "rot_dims must be even, at most the rotated part");
   TORCH_CHECK(inv_freq.scalar_type() == at::kFloat && inv_freq.is_contiguous() &&
               inv_freq.numel() == rot_dims / 2 && inv_freq.is_cuda());
-  TORCH_CHECK(c_w.numel() == R && c_w.is_contiguous());
   TORCH_CHECK(positions.scalar_type() == at::kLong && positions.is_contiguous() && positions.numel() == T_);
   TORCH_CHECK(slots.scalar_type() == at::kLong && slots.is_contiguous() && slots.numel() == T_);
-  TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous() && k_cache.size(1) == 1 &&
-              k_cache.size(3) == R + DR, "latent cache must be [blocks, 1, block, R + rot part]");
-  const auto dt = q.scalar_type();
-  TORCH_CHECK(q_lat.scalar_type() == dt && ckr.scalar_type() == dt && c_w.scalar_type() == dt &&
-              out.scalar_type() == dt && k_cache.scalar_type() == dt,
-              "latent_rope_pack: one dtype for activations, weights and cache");
+  if (q_lat.has_value())
+    TORCH_CHECK(q_lat->dim() == 3 && q_lat->size(0) == T_ && q_lat->size(1) == H &&
+                q_lat->size(2) == R && q_lat->stride(2) == 1 && q_lat->scalar_type() == dt,
+                "q_lat must be [T, H, latent]");
+  if (ckr.has_value()) {
+    TORCH_CHECK(c_w.has_value() && k_cache.has_value(), "a latent needs its norm weight and its cache");
+    TORCH_CHECK(ckr->dim() == 2 && ckr->size(0) == T_ && ckr->size(1) == R + DR && ckr->stride(1) == 1);
+    TORCH_CHECK(c_w->numel() == R && c_w->is_contiguous());
+    TORCH_CHECK(k_cache->dim() == 4 && k_cache->is_contiguous() && k_cache->size(1) == 1 &&
+                k_cache->size(3) == R + DR, "latent cache must be [blocks, 1, block, R + rot part]");
+    TORCH_CHECK(ckr->scalar_type() == dt && c_w->scalar_type() == dt && k_cache->scalar_type() == dt,
+                "latent_rope_pack: one dtype for activations, weights and cache");
+  }
   hy_dispatch(q, "latent_rope_pack", [&]<typename T>() {
-    hipLaunchKernelGGL(latent_rope_pack_kernel<T>, dim3(T_), dim3(256), 0, hy_stream(),
-                       reinterpret_cast<T*>(out.data_ptr()),
-                       reinterpret_cast<const T*>(q.data_ptr()), q.stride(0), q.stride(1),
-                       reinterpret_cast<const T*>(q_lat.data_ptr()), q_lat.stride(0), q_lat.stride(1),
-                       reinterpret_cast<const T*>(ckr.data_ptr()), ckr.stride(0),
-                       reinterpret_cast<const T*>(c_w.data_ptr()), inv_freq.data_ptr<float>(),
-                       positions.data_ptr<long>(), reinterpret_cast<T*>(k_cache.data_ptr()),
-                       slots.data_ptr<long>(), H, (int)dim, DR, R, (int)rot_dims,
-                       (int)interleaved, (float)eps);
+    auto ptr = [](const std::optional<at::Tensor>& x) -> T* {
+      return x.has_value() ? reinterpret_cast<T*>(x->data_ptr()) : nullptr;
+    };
+    hipLaunchKernelGGL(latent_rope_pack_kernel<T>, dim3(T_), dim3(256), sizeof(float) * rot_dims,
+                       hy_stream(), reinterpret_cast<T*>(out.data_ptr()),
+                       reinterpret_cast<const T*>(q.data_ptr()), q.stride(0), q.stride(1), ptr(q_lat),
+                       q_lat.has_value() ? q_lat->stride(0) : 0L,
+                       q_lat.has_value() ? q_lat->stride(1) : 0L, ptr(ckr),
+                       ckr.has_value() ? ckr->stride(0) : 0L, ckr.has_value() ? ptr(c_w) : nullptr,
+                       inv_freq.data_ptr<float>(), positions.data_ptr<long>(),
+                       ckr.has_value() ? ptr(k_cache) : nullptr, slots.data_ptr<long>(), H, (int)dim,
+                       DR, R, (int)rot_dims, (int)interleaved, (float)eps, (float)amplitude);
   });
 }
 
@@ -1264,6 +1298,86 @@ void qkv_norm_rope_cache(at::Tensor q, at::Tensor k, const std::optional<at::Ten
   else hy_dispatch(q, "qkv_norm_rope_cache", [&]<typename T>() { launch.template operator()<T, false>(); });
 }
 
+// q [T, H, D], k [T, G, D]: row-strided views with packed heads, normed over the
+// whole row, rotated in adjacent pairs; raw keys become the values. conv_w given:
+// every row is its sequence's only one and q / k are first convolved (q's and
+// k's channels start at q_at / k_at of conv_w and tail), the tail advanced.
+void rownorm_rope_cache(at::Tensor q, at::Tensor k, at::Tensor q_w, at::Tensor k_w,
+                        const std::optional<at::Tensor>& inv_freq, int64_t rot_dims,
+                        double amplitude, at::Tensor positions, at::Tensor k_cache,
+                        at::Tensor v_cache, at::Tensor slots, double eps,
+                        const std::optional<at::Tensor>& conv_w,
+                        const std::optional<at::Tensor>& tail,
+                        const std::optional<at::Tensor>& rec_slots,
+                        const std::optional<at::Tensor>& rec_fresh, int64_t q_at, int64_t k_at) {
+  HY_GPU(q);
+  const long T_ = q.size(0);
+  if (T_ == 0) return;
+  TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && k.size(0) == T_ && k.size(2) == q.size(2));
+  HY_INNER(q); HY_INNER(k);
+  const int H = q.size(1), G = k.size(1), D = q.size(2);
+  TORCH_CHECK(H >= 1 && G >= 1 && D >= 1 && q.stride(1) == D && k.stride(1) == D, "heads must be packed");
+  const auto dt = q.scalar_type();
+  TORCH_CHECK(k.scalar_type() == dt && k_cache.scalar_type() == dt && v_cache.scalar_type() == dt &&
+              q_w.scalar_type() == dt && k_w.scalar_type() == dt,
+              "rownorm_rope_cache: one dtype for activations, weights and cache");
+  TORCH_CHECK(q_w.is_cuda() && q_w.is_contiguous() && q_w.numel() == (long)H * D && k_w.is_cuda() &&
+              k_w.is_contiguous() && k_w.numel() == (long)G * D, "norm weights span the whole row");
+  TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous() && k_cache.size(1) == G &&
+              k_cache.size(3) == D, "key cache must be [blocks, G, block, D]");
+  TORCH_CHECK(v_cache.is_contiguous() && v_cache.sizes() == k_cache.sizes(),
+              "values that are the raw keys have the keys' cache shape");
+  TORCH_CHECK(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= D, "rot_dims must be even, at most D");
+  const float* table = nullptr;
+  if (rot_dims) {
+    TORCH_CHECK(inv_freq.has_value() && inv_freq->is_cuda() && inv_freq->scalar_type() == at::kFloat &&
+                inv_freq->is_contiguous() && inv_freq->numel() == rot_dims / 2,
+                "a rotary table must be fp32 [dims / 2]");
+    table = inv_freq->data_ptr<float>();
+  }
+  TORCH_CHECK(positions.scalar_type() == at::kLong && positions.is_contiguous() &&
+              positions.numel() == T_ && positions.is_cuda());
+  TORCH_CHECK(slots.scalar_type() == at::kLong && slots.is_contiguous() && slots.numel() == T_ &&
+              slots.is_cuda());
+  const bool step = conv_w.has_value();
+  ConvStep cv{nullptr, nullptr, nullptr, nullptr, 0, 1, 0, 0};
+  if (step) {
+    TORCH_CHECK(tail.has_value() && rec_slots.has_value() && rec_fresh.has_value(),
+                "a convolution step needs the tail, the state slots and the fresh flags");
+    HY_F32((*conv_w)); HY_F32((*tail)); HY_I32((*rec_slots)); HY_I32((*rec_fresh));
+    TORCH_CHECK(conv_w->dim() == 2 && conv_w->size(1) >= 1 && tail->dim() == 3 && conv_w->is_cuda() &&
+                tail->is_cuda() && tail->size(1) == conv_w->size(1) - 1 &&
+                tail->size(2) == conv_w->size(0), "conv_w [C, K], tail [slots, K - 1, C]");
+    TORCH_CHECK(rec_slots->numel() == T_ && rec_fresh->numel() == T_, "one row per sequence");
+    const long C = conv_w->size(0);
+    TORCH_CHECK(q_at >= 0 && q_at + (long)H * D <= C && k_at >= 0 && k_at + (long)G * D <= C,
+                "q and k must lie within the convolved channels");
+    cv = ConvStep{conv_w->data_ptr<float>(), tail->data_ptr<float>(), rec_slots->data_ptr<int>(),
+                  rec_fresh->data_ptr<int>(), (int)C, (int)conv_w->size(1), (int)q_at, (int)k_at};
+  }
+  auto aligned = [](const at::Tensor& x) { return reinterpret_cast<uintptr_t>(x.data_ptr()) % 16 == 0; };
+  const bool vec = dt == at::kBFloat16 && D % 8 == 0 && q.stride(0) % 8 == 0 && k.stride(0) % 8 == 0 &&
+                   aligned(q) && aligned(k) && aligned(q_w) && aligned(k_w) && aligned(k_cache) &&
+                   aligned(v_cache);
+  auto launch = [&]<typename T, int V, bool STEP>() {
+    hipLaunchKernelGGL((rownorm_rope_cache_kernel<T, V, STEP>), dim3(T_), dim3(256),
+                       sizeof(float) * rot_dims, hy_stream(), reinterpret_cast<T*>(q.data_ptr()),
+                       q.stride(0), reinterpret_cast<const T*>(k.data_ptr()), k.stride(0),
+                       reinterpret_cast<const T*>(q_w.data_ptr()),
+                       reinterpret_cast<const T*>(k_w.data_ptr()), table, (int)rot_dims,
+                       (float)amplitude, positions.data_ptr<long>(),
+                       reinterpret_cast<T*>(k_cache.data_ptr()),
+                       reinterpret_cast<T*>(v_cache.data_ptr()), slots.data_ptr<long>(), H, G, D,
+                       (int)k_cache.size(2), (float)eps, cv);
+  };
+  auto by_step = [&]<typename T, int V>() {
+    if (step) launch.template operator()<T, V, true>();
+    else launch.template operator()<T, V, false>();
+  };
+  if (vec) by_step.template operator()<__hip_bfloat16, 8>();
+  else hy_dispatch(q, "rownorm_rope_cache", [&]<typename T>() { by_step.template operator()<T, 2>(); });
+}
+
 void rotate_heads(at::Tensor x, at::Tensor positions, at::Tensor inv_freq, bool inverse) {
   HY_GPU(x);
   const long T_ = x.size(0);
@@ -1427,7 +1541,8 @@ void unary_act(at::Tensor out, at::Tensor in, int64_t act) {
 // ---- gated delta rule and Mamba-2 gates / read-out ---------------------------
 
 // q, k [T, Hk, D], v [T, H, DV], z [T, H, D]: row-strided views, heads packed;
-// beta [T, H] row-strided; z_bias fp32 [H*D]; rate fp32 [H] (> 0); o fp32
+// z [T, H, D] with z_bias fp32 [H*D] (a decay per key channel) or z [T, H] with
+// z_bias fp32 [H] (one per head); beta [T, H] row-strided; rate fp32 [H] (> 0); o fp32
 // [T, H, DV]; state fp32 [slots, H, D, DV].
 void gated_delta_rule(at::Tensor o, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor z,
                       at::Tensor z_bias, at::Tensor rate, at::Tensor beta, at::Tensor state,
@@ -1435,16 +1550,19 @@ void gated_delta_rule(at::Tensor o, at::Tensor q, at::Tensor k, at::Tensor v, at
   HY_GPU(q);
   const long T_ = q.size(0);
   if (T_ == 0) return;
-  TORCH_CHECK(q.dim() == 3 && k.sizes() == q.sizes() && v.dim() == 3 && z.dim() == 3 && beta.dim() == 2);
+  TORCH_CHECK(q.dim() == 3 && k.sizes() == q.sizes() && v.dim() == 3 && beta.dim() == 2 &&
+              (z.dim() == 3 || z.dim() == 2));
+  const bool head_decay = z.dim() == 2;
   HY_INNER(q); HY_INNER(k); HY_INNER(v); HY_INNER(z); HY_INNER(beta);
   const int Hk = q.size(1), D = q.size(2), H = v.size(1), DV = v.size(2);
   TORCH_CHECK(Hk >= 1 && H % Hk == 0, "heads must be a multiple of the q/k heads");
-  TORCH_CHECK(v.size(0) == T_ && z.size(0) == T_ && z.size(1) == H && z.size(2) == D &&
+  TORCH_CHECK(v.size(0) == T_ && z.size(0) == T_ && z.size(1) == H && (head_decay || z.size(2) == D) &&
               beta.size(0) == T_ && beta.size(1) == H);
-  TORCH_CHECK(q.stride(1) == D && k.stride(1) == D && v.stride(1) == DV && z.stride(1) == D,
+  TORCH_CHECK(q.stride(1) == D && k.stride(1) == D && v.stride(1) == DV &&
+              (head_decay || z.stride(1) == D),
               "heads must be packed");
   HY_F32(z_bias); HY_F32(rate);
-  TORCH_CHECK(z_bias.numel() == (long)H * D && rate.numel() == H);
+  TORCH_CHECK(z_bias.numel() == (head_decay ? (long)H : (long)H * D) && rate.numel() == H);
   TORCH_CHECK(o.scalar_type() == at::kFloat && o.is_contiguous() && o.dim() == 3 && o.size(0) == T_ &&
               o.size(1) == H && o.size(2) == DV);
   const SeqDims sd = seq_check(cu, slots, fresh, state);
@@ -1457,9 +1575,9 @@ void gated_delta_rule(at::Tensor o, at::Tensor q, at::Tensor k, at::Tensor v, at
   // 4 value columns per thread while that still fills the chip, else 1
   const long wide = (long)((DV + 63) / 64) * H * sd.B;
   hy_dispatch(q, "gated_delta_rule", [&]<typename T>() {
-    auto launch = [&]<int DPL, int NC>() {
+    auto launch_as = [&]<int DPL, int NC, bool HD>() {
       const dim3 grid((DV + 16 * NC - 1) / (16 * NC), H, sd.B);
-      hipLaunchKernelGGL((gated_delta_kernel<T, DPL, NC>), grid, dim3(256), 0, hy_stream(),
+      hipLaunchKernelGGL((gated_delta_kernel<T, DPL, NC, HD>), grid, dim3(256), 0, hy_stream(),
                          o.data_ptr<float>(), reinterpret_cast<const T*>(q.data_ptr()), q.stride(0),
                          reinterpret_cast<const T*>(k.data_ptr()), k.stride(0),
                          reinterpret_cast<const T*>(v.data_ptr()), v.stride(0),
@@ -1468,6 +1586,10 @@ void gated_delta_rule(at::Tensor o, at::Tensor q, at::Tensor k, at::Tensor v, at
                          reinterpret_cast<const T*>(beta.data_ptr()), beta.stride(0),
                          state.data_ptr<float>(), cu.data_ptr<int>(), slots.data_ptr<int>(),
                          fresh.data_ptr<int>(), H, H / Hk, D, DV, (float)q_scale);
+    };
+    auto launch = [&]<int DPL, int NC>() {
+      if (head_decay) launch_as.template operator()<DPL, NC, true>();
+      else launch_as.template operator()<DPL, NC, false>();
     };
     auto by_d = [&]<int NC>() {
       if (D <= 32) launch.template operator()<2, NC>();
@@ -1592,14 +1714,14 @@ void ssd_out_gate_norm(at::Tensor out, at::Tensor o, at::Tensor x, at::Tensor D,
 
 TORCH_LIBRARY(llmq_amd_hybrid, m) {
   m.def("rmsnorm_cast(Tensor(a!) out, Tensor input, Tensor weight, float eps, float offset, int groups=1) -> ()");
-  m.def("sandwich_norm_res32(Tensor(a!) x, Tensor(b!) residual, Tensor w_post, Tensor w_pre, float eps, float offset, int groups=1) -> ()");
+  m.def("sandwich_norm_res32(Tensor(a!) x, Tensor(b!) residual, Tensor w_post, Tensor? w_pre, float eps, float offset, int groups=1) -> ()");
   m.def("act_and_mul(Tensor(a!) out, Tensor input, bool gelu) -> ()");
   m.def("qknorm_vmix_cache(Tensor(a!) q, Tensor k, Tensor v, Tensor q_w, Tensor k_w, Tensor? v_first, float lam, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, float eps) -> ()");
   m.def("paged_attn_prefill(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor cu_q, Tensor q_start, int max_q, int span, float scale, int mask_mode, int pos_stride, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0, int weight_fn=0, Tensor? wbias=None) -> ()");
   m.def("paged_attn_decode(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor context_lens, int span, float scale, int mask_mode, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0, int weight_fn=0, Tensor? wbias=None) -> ()");
   m.def("gla_recurrence(Tensor(a!) o, Tensor q, Tensor? k, Tensor v, Tensor z, Tensor z_bias, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh, float tau, Tensor? lower, bool q_silu, float q_scale) -> ()");
   m.def("gla_out_norm_gate(Tensor(a!) out, Tensor o, Tensor weight, Tensor? gate, float eps, bool gate_sigmoid=False) -> ()");
-  m.def("latent_rope_pack(Tensor(a!) out, Tensor q, Tensor q_lat, Tensor ckr, Tensor c_w, Tensor inv_freq, Tensor positions, Tensor(b!) k_cache, Tensor slots, int dim, int rot_dims, bool interleaved, float eps) -> ()");
+  m.def("latent_rope_pack(Tensor(a!) out, Tensor q, Tensor? q_lat, Tensor? ckr, Tensor? c_w, Tensor inv_freq, Tensor positions, Tensor(b!)? k_cache, Tensor slots, int dim, int rot_dims, bool interleaved, float eps, float amplitude=1.0) -> ()");
   m.def("gated_residual_add(Tensor(a!) out, Tensor(b!) res, Tensor y1, Tensor g1, Tensor b1, Tensor? y2, Tensor? g2, Tensor? b2) -> ()");
   m.def("side_gate_mul(Tensor(a!) out, Tensor a, Tensor table, Tensor tokens, int offset) -> ()");
   m.def("sigmoid_topk(Tensor(a!) idx, Tensor(b!) w, Tensor logits, int top) -> ()");
@@ -1618,6 +1740,7 @@ TORCH_LIBRARY(llmq_amd_hybrid, m) {
   m.def("softmax_topk(Tensor(a!) idx, Tensor(b!) w, Tensor logits, int top, float scale, Tensor? correction=None, bool renorm=False) -> ()");
   m.def("clamp_swish_mul(Tensor(a!) out, Tensor input, float limit) -> ()");
   m.def("qkv_norm_rope_cache(Tensor(a!) q, Tensor k, Tensor? v, Tensor? q_w, Tensor? k_w, Tensor? inv_freq, int rot_dims, Tensor positions, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, float eps, bool v_unit_norm, Tensor? v_inv_freq, bool qk_unit_norm=False, Tensor? head_scale=None, float temp_coef=0.0, int temp_every=1, Tensor? v_first=None, float mix=0.0) -> ()");
+  m.def("rownorm_rope_cache(Tensor(a!) q, Tensor k, Tensor q_w, Tensor k_w, Tensor? inv_freq, int rot_dims, float amplitude, Tensor positions, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, float eps, Tensor? conv_w=None, Tensor(d!)? tail=None, Tensor? rec_slots=None, Tensor? rec_fresh=None, int q_at=0, int k_at=0) -> ()");
   m.def("rotate_heads(Tensor(a!) x, Tensor positions, Tensor inv_freq, bool inverse) -> ()");
   m.def("mlstm_gates(Tensor(a!) out, Tensor gates, float cap, Tensor(b!) m_state, Tensor cu, Tensor slots, Tensor fresh) -> ()");
   m.def("matrix_memory(Tensor(a!) o, Tensor q, Tensor k, Tensor v, Tensor decay, Tensor write, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh, float q_scale, bool ones_col=True) -> ()");
@@ -1658,6 +1781,7 @@ TORCH_LIBRARY_IMPL(llmq_amd_hybrid, CUDA, m) {
   m.impl("softmax_topk", &softmax_topk);
   m.impl("clamp_swish_mul", &clamp_swish_mul);
   m.impl("qkv_norm_rope_cache", &qkv_norm_rope_cache);
+  m.impl("rownorm_rope_cache", &rownorm_rope_cache);
   m.impl("rotate_heads", &rotate_heads);
   m.impl("mlstm_gates", &mlstm_gates);
   m.impl("matrix_memory", &matrix_memory);

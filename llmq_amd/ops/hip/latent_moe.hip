@@ -12,12 +12,12 @@
 // ------------------------------------------------------ latent attention --
 // Rotary positions on the first rot_dims channels of a vector x (n channels
 // in all, the rest pass unchanged), channel j of the result. Pair i turns by
-// angle pos * inv_freq[i]: (u, v) -> (u cos - v sin, v cos + u sin). Half
-// layout: pair (i, i + rot_dims/2); interleaved: pair (2i, 2i + 1).
+// the angle whose (cos, sin) is cs[2i], cs[2i+1]: (u, v) -> (u cos - v sin,
+// v cos + u sin). Half layout: pair (i, i + rot_dims/2); interleaved: pair
+// (2i, 2i + 1).
 template <typename T>
-DEVINL float rotary_channel(const T* __restrict__ x, int j, float pos,
-                            const float* __restrict__ inv_freq, int rot_dims,
-                            bool interleaved) {
+DEVINL float rotary_channel(const T* __restrict__ x, int j, const float* __restrict__ cs,
+                            int rot_dims, bool interleaved) {
   const float xj = to_f32(x[j]);
   if (j >= rot_dims) return xj;
   const int half = rot_dims >> 1;
@@ -32,59 +32,73 @@ DEVINL float rotary_channel(const T* __restrict__ x, int j, float pos,
     i = first ? j : j - half;
     partner = first ? j + half : j - half;
   }
-  const float a = pos * inv_freq[i];
-  const float c = cosf(a), s = sinf(a);
+  const float c = cs[2 * i], s = cs[2 * i + 1];
   const float xp = to_f32(x[partner]);
   return first ? xj * c - xp * s : xj * c + xp * s;
 }
 
 // Per token, between the projections and the attention kernel:
-//   out[t, h, :R]  = q_lat[t, h, :]            (query mapped into the latent)
+//   out[t, h, :R]  = q_lat[t, h, :]            (query mapped into the latent;
+//                    q_lat null: those channels of out hold it already)
 //   out[t, h, R:]  = rotary(q[t, h, dim:])     (rotated query part)
 //   cache row      = rmsnorm(ckr[t, :R]) * c_w ‖ rotary(ckr[t, R:])
+//                    (ckr null: the layer reads another layer's rows)
 // The cache is [blocks, 1, block_size, R + DR]: one row per token, shared by
-// all heads; a negative slot writes nothing (padding rows).
+// all heads; a negative slot writes nothing (padding rows). Angles are
+// position * inv_freq[i], cos and sin times amp, once per token into LDS.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_rope_pack_kernel(
     T* __restrict__ out,                       // [T, H, R+DR] contiguous
     const T* __restrict__ q, long q_s0, long q_s1,          // [T, H, dim+DR]
-    const T* __restrict__ q_lat, long l_s0, long l_s1,      // [T, H, R]
-    const T* __restrict__ ckr, long c_s0,                   // [T, R+DR]
+    const T* __restrict__ q_lat, long l_s0, long l_s1,      // [T, H, R] or null
+    const T* __restrict__ ckr, long c_s0,                   // [T, R+DR] or null
     const T* __restrict__ c_w,                              // [R]
     const float* __restrict__ inv_freq,                     // [rot_dims/2]
     const long* __restrict__ positions, T* __restrict__ k_cache,
     const long* __restrict__ slots, int H, int dim, int DR, int R, int rot_dims,
-    int interleaved, float eps) {
+    int interleaved, float eps, float amp) {
+  extern __shared__ float lat_cs[];            // [rot_dims/2][cos, sin]
   __shared__ float red[4];
   const long tok = blockIdx.x;
   const float pos = (float)positions[tok];
   const int RW = R + DR;
-  const T* cr = ckr + tok * c_s0;
-  float ss = 0.f;
-  for (int i = threadIdx.x; i < R; i += blockDim.x) {
-    const float f = to_f32(cr[i]);
-    ss += f * f;
+  for (int i = threadIdx.x; i < rot_dims / 2; i += blockDim.x) {
+    float sn, c;
+    sincosf(pos * inv_freq[i], &sn, &c);
+    lat_cs[2 * i] = c * amp;
+    lat_cs[2 * i + 1] = sn * amp;
   }
-  ss = block_reduce_sum(ss, red);
-  const float inv = 1.0f / sqrtf(ss / R + eps);
-  for (int idx = threadIdx.x; idx < H * RW; idx += blockDim.x) {
-    const int h = idx / RW, c = idx % RW;
-    float val;
-    if (c < R) {
-      val = to_f32(q_lat[tok * l_s0 + (long)h * l_s1 + c]);
-    } else {
-      val = rotary_channel(q + tok * q_s0 + (long)h * q_s1 + dim, c - R, pos, inv_freq,
-                           rot_dims, interleaved != 0);
+  const T* cr = ckr + tok * c_s0;
+  float inv = 0.f;
+  if (ckr) {
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < R; i += blockDim.x) {
+      const float f = to_f32(cr[i]);
+      ss += f * f;
     }
-    out[(tok * H + h) * RW + c] = from_f32<T>(val);
+    ss = block_reduce_sum(ss, red);            // its barriers publish the table too
+    inv = 1.0f / sqrtf(ss / R + eps);
+  } else {
+    __syncthreads();
+  }
+  if (q_lat) {
+    for (int idx = threadIdx.x; idx < H * R; idx += blockDim.x) {
+      const int h = idx / R, c = idx % R;
+      out[(tok * H + h) * RW + c] = q_lat[tok * l_s0 + (long)h * l_s1 + c];
+    }
+  }
+  for (int idx = threadIdx.x; idx < H * DR; idx += blockDim.x) {
+    const int h = idx / DR, c = idx % DR;
+    out[(tok * H + h) * RW + R + c] = from_f32<T>(rotary_channel(
+        q + tok * q_s0 + (long)h * q_s1 + dim, c, lat_cs, rot_dims, interleaved != 0));
   }
   const long slot = slots[tok];
-  if (slot < 0) return;
+  if (!ckr || slot < 0) return;
   T* row = k_cache + slot * RW;   // [blocks, 1, bs, RW]: slot = block * bs + offset
   for (int c = threadIdx.x; c < RW; c += blockDim.x) {
     float val;
     if (c < R) val = to_f32(cr[c]) * inv * to_f32(c_w[c]);
-    else val = rotary_channel(cr + R, c - R, pos, inv_freq, rot_dims, interleaved != 0);
+    else val = rotary_channel(cr + R, c - R, lat_cs, rot_dims, interleaved != 0);
     row[c] = from_f32<T>(val);
   }
 }

@@ -274,6 +274,208 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_cache_kernel(
   }
 }
 
+// ------------------------------- q / k normed over the whole projection ----
+// One workgroup per token. q [H, D] and k [G, D] of a token are each RMS-normed
+// over ALL their channels (weights [H * D] and [G * D]), then every head is
+// rotated on its first rot_dims channels in ADJACENT pairs (2i, 2i + 1), cos and
+// sin times amp; q in place, k into the key cache, and the keys as they arrive
+// (before norm and rotation) into the value cache.
+//
+// STEP: the token is its sequence's only row of this launch, and the kernel
+// first runs the short causal convolution in front of the norm: output channel
+// = sum_k w[c, k] V[k], the K - 1 earlier inputs from the sequence's tail
+// [slots, K - 1, C] fp32 (zeros if fresh), which is advanced in place. The
+// result is rounded to T like that of the convolution kernel, so a token's
+// q, k and values do not depend on which of the two ways it came.
+//
+// A thread owns granules of V adjacent channels of one head (8 as one 16-byte
+// access for bf16, else 2); up to kRowKeep granules stay in registers between
+// the sums and the stores, what lies beyond is read (and convolved) again.
+constexpr int kRowKeep = 4;
+
+struct ConvStep {
+  const float* w;       // [C, K]
+  float* tail;          // [slots, K - 1, C]
+  const int* slots;     // [B]
+  const int* fresh;     // [B]
+  int C, K, q_at, k_at; // q's and k's first channel among the C
+};
+
+template <typename T, int V>
+DEVINL void load_granule(const T* __restrict__ p, int live, float* v) {
+  if constexpr (V == 8) {
+    const Vec8<T> a = load16(p);
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = to_f32(a.data[e]);
+  } else {
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = e < live ? to_f32(p[e]) : 0.f;
+  }
+}
+
+template <typename T, int V>
+DEVINL void store_granule(T* __restrict__ p, int live, const float* v) {
+  if constexpr (V == 8) {
+    Vec8<T> a;
+#pragma unroll
+    for (int e = 0; e < V; ++e) a.data[e] = from_f32<T>(v[e]);
+    store16(p, a);
+  } else {
+#pragma unroll
+    for (int e = 0; e < V; ++e)
+      if (e < live) p[e] = from_f32<T>(v[e]);
+  }
+}
+
+// v: the current inputs of channels c .. c + live - 1 -> their convolution
+// outputs; commit: the tail moves on by one token.
+template <typename T, int V>
+DEVINL void conv_one_step(const ConvStep& cv, int c, long slot, bool fresh, int live, bool commit,
+                          float* v) {
+  float acc[V];
+#pragma unroll
+  for (int e = 0; e < V; ++e) acc[e] = 0.f;
+  float* tl = cv.tail + slot * (cv.K - 1) * cv.C + c;
+  for (int k = 0; k < cv.K - 1; ++k) {
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      if (e >= live) continue;
+      const float old = fresh ? 0.f : tl[(long)k * cv.C + e];
+      acc[e] += cv.w[(long)(c + e) * cv.K + k] * old;
+      if (commit && k > 0) tl[(long)(k - 1) * cv.C + e] = old;
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < V; ++e) {
+    if (e >= live) continue;
+    if (commit && cv.K > 1) tl[(long)(cv.K - 2) * cv.C + e] = v[e];
+    v[e] = to_f32(from_f32<T>(acc[e] + cv.w[(long)(c + e) * cv.K + cv.K - 1] * v[e]));
+  }
+}
+
+template <typename T, int V, bool STEP>
+__global__ __launch_bounds__(256) void rownorm_rope_cache_kernel(
+    T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride,
+    const T* __restrict__ q_w, const T* __restrict__ k_w, // [H * D], [G * D]
+    const float* __restrict__ inv_freq, int rot_dims,     // [rot_dims / 2] (rot_dims may be 0)
+    float amp, const long* __restrict__ positions, T* __restrict__ k_cache,
+    T* __restrict__ v_cache, const long* __restrict__ slots, int H, int G, int D, int block_size,
+    float eps, ConvStep cv) {
+  extern __shared__ __align__(8) float row_cs[];   // [rot_dims / 2][cos, sin]
+  __shared__ float red[8];
+  const long tok = blockIdx.x;
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  const float pos = (float)positions[tok];
+  for (int i = tid; i < rot_dims / 2; i += 256) {
+    float sn, c;
+    sincosf(pos * inv_freq[i], &sn, &c);
+    row_cs[2 * i] = c * amp;
+    row_cs[2 * i + 1] = sn * amp;
+  }
+  const int per_head = (D + V - 1) / V;
+  const int nq = H * per_head, nk = G * per_head;
+  long rslot = 0;
+  bool fr = true;
+  if constexpr (STEP) {
+    rslot = cv.slots[tok];
+    fr = cv.fresh[tok] != 0;
+  }
+  auto fetch = [&](const T* base, int item, int first_channel, bool commit, float* v) {
+    const int h = item / per_head, d = (item % per_head) * V, live = min(V, D - d);
+    load_granule<T, V>(base + (long)h * D + d, live, v);
+    if constexpr (STEP) conv_one_step<T, V>(cv, first_channel + h * D + d, rslot, fr, live, commit, v);
+  };
+  T* qt = q + tok * q_stride;
+  const T* kt = k + tok * k_stride;
+  float kq[kRowKeep][V], kk[kRowKeep][V];
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int s = 0; s < kRowKeep; ++s) {
+    const int item = s * 256 + tid;
+    if (item < nq) {
+      fetch(qt, item, cv.q_at, true, kq[s]);
+#pragma unroll
+      for (int e = 0; e < V; ++e) sq += kq[s][e] * kq[s][e];
+    }
+    if (item < nk) {
+      fetch(kt, item, cv.k_at, true, kk[s]);
+#pragma unroll
+      for (int e = 0; e < V; ++e) sk += kk[s][e] * kk[s][e];
+    }
+  }
+  for (int item = kRowKeep * 256 + tid; item < nq || item < nk; item += 256) {
+    float v[V];
+    if (item < nq) {
+      fetch(qt, item, cv.q_at, false, v);
+#pragma unroll
+      for (int e = 0; e < V; ++e) sq += v[e] * v[e];
+    }
+    if (item < nk) {
+      fetch(kt, item, cv.k_at, false, v);
+#pragma unroll
+      for (int e = 0; e < V; ++e) sk += v[e] * v[e];
+    }
+  }
+  sq = wave_reduce_sum(sq);
+  sk = wave_reduce_sum(sk);
+  if (lane == 0) {
+    red[w] = sq;
+    red[4 + w] = sk;
+  }
+  __syncthreads();
+  const float iq = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (H * D) + eps);
+  const float ik = 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (G * D) + eps);
+  auto finish = [&](const T* wt, float inv, int item, float* v) {   // norm, weight, rotation
+    const int h = item / per_head, d = (item % per_head) * V, live = min(V, D - d);
+    float wv[V];
+    load_granule<T, V>(wt + (long)h * D + d, live, wv);
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] *= inv * wv[e];
+#pragma unroll
+    for (int e = 0; e < V; e += 2) {
+      if (d + e < rot_dims) {
+        const float2 c_s = *reinterpret_cast<const float2*>(row_cs + d + e);
+        const float a = v[e], b = v[e + 1];
+        v[e] = a * c_s.x - b * c_s.y;
+        v[e + 1] = b * c_s.x + a * c_s.y;
+      }
+    }
+  };
+  auto put_q = [&](int item, float* v) {
+    finish(q_w, iq, item, v);
+    const int h = item / per_head, d = (item % per_head) * V;
+    store_granule<T, V>(qt + (long)h * D + d, min(V, D - d), v);
+  };
+  const long slot = slots[tok];
+  const long blk = slot >= 0 ? slot / block_size : 0;
+  const int off = slot >= 0 ? (int)(slot % block_size) : 0;
+  auto put_k = [&](int item, float* v) {
+    if (slot < 0) return;
+    const int g = item / per_head, d = (item % per_head) * V;
+    const long at = ((blk * G + g) * block_size + off) * D + d;
+    store_granule<T, V>(v_cache + at, min(V, D - d), v);
+    finish(k_w, ik, item, v);
+    store_granule<T, V>(k_cache + at, min(V, D - d), v);
+  };
+#pragma unroll
+  for (int s = 0; s < kRowKeep; ++s) {
+    const int item = s * 256 + tid;
+    if (item < nq) put_q(item, kq[s]);
+    if (item < nk) put_k(item, kk[s]);
+  }
+  for (int item = kRowKeep * 256 + tid; item < nq || item < nk; item += 256) {
+    float v[V];
+    if (item < nq) {
+      fetch(qt, item, cv.q_at, true, v);
+      put_q(item, v);
+    }
+    if (item < nk) {
+      fetch(kt, item, cv.k_at, true, v);
+      put_k(item, v);
+    }
+  }
+}
+
 // x [T, H, n] contiguous, in place: head vectors turned by sign * position over
 // all n channels, pairs (i, i + n/2).
 template <typename T>

@@ -42,7 +42,8 @@ __global__ void rmsnorm_cast_kernel(TO* __restrict__ out, const TI* __restrict__
 // Norm sandwich around an fp32 residual:
 //   residual += rmsnorm(x) * (w_post + offset)        (fp32, in place)
 //   x         = rmsnorm(residual) * (w_pre + offset)  (T, in place)
-// One launch closes a sublayer and opens the next.
+// One launch closes a sublayer and opens the next. w_pre null: the next
+// sublayer reads the stream itself, x = residual rounded to T.
 template <typename T>
 __global__ void sandwich_norm_res32_kernel(T* __restrict__ x, float* __restrict__ residual,
                                            const T* __restrict__ w_post,
@@ -51,7 +52,7 @@ __global__ void sandwich_norm_res32_kernel(T* __restrict__ x, float* __restrict_
   __shared__ float red[4];
   const long row = blockIdx.x;
   w_post += (row % groups) * hidden;
-  w_pre += (row % groups) * hidden;
+  if (w_pre) w_pre += (row % groups) * hidden;
   T* xr = x + row * hidden;
   float* rr = residual + row * hidden;
   float ss = 0.f;
@@ -65,8 +66,10 @@ __global__ void sandwich_norm_res32_kernel(T* __restrict__ x, float* __restrict_
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
     const float r = rr[i] + to_f32(xr[i]) * inv1 * (to_f32(w_post[i]) + offset);
     rr[i] = r;
+    if (!w_pre) xr[i] = from_f32<T>(r);
     ss2 += r * r;
   }
+  if (!w_pre) return;
   ss2 = block_reduce_sum(ss2, red);
   const float inv2 = 1.0f / sqrtf(ss2 / hidden + eps);
   for (int i = threadIdx.x; i < hidden; i += blockDim.x)
@@ -90,7 +93,7 @@ __global__ __launch_bounds__(256) void sandwich_norm_res32_vec_kernel(
   const long row = PER_WAVE ? blockIdx.x * 4L + (threadIdx.x >> 6) : blockIdx.x;
   if (PER_WAVE && row >= rows) return;
   w_post += (row % groups) * hidden;
-  w_pre += (row % groups) * hidden;
+  if (w_pre) w_pre += (row % groups) * hidden;
   __hip_bfloat16* xr = x + row * hidden;
   float* rr = residual + row * hidden;
   float xv[CH][8], rv[CH][8];
@@ -126,8 +129,15 @@ __global__ __launch_bounds__(256) void sandwich_norm_res32_vec_kernel(
       }
       *reinterpret_cast<float4*>(rr + i) = make_float4(rv[c][0], rv[c][1], rv[c][2], rv[c][3]);
       *reinterpret_cast<float4*>(rr + i + 4) = make_float4(rv[c][4], rv[c][5], rv[c][6], rv[c][7]);
+      if (!w_pre) {
+        Vec8<__hip_bfloat16> ov;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ov.data[j] = __float2bfloat16(rv[c][j]);
+        store16(xr + i, ov);
+      }
     }
   }
+  if (!w_pre) return;
   ss2 = PER_WAVE ? wave_reduce_sum(ss2) : block_reduce_sum(ss2, red);
   const float inv2 = 1.0f / sqrtf(ss2 / hidden + eps);
 #pragma unroll
@@ -233,8 +243,8 @@ __global__ void qknorm_vmix_cache_kernel(
 // bias[i - j, h]; softmax over the visible keys; the head's output is
 // multiplied by sigmoid(gate[i, h]).
 //
-// Workgroup = 16 query rows x 1 head, 4 waves x 4 rows. Key tiles of 64 are
-// staged in LDS as fp32; in the score phase a lane owns one key (4 rows
+// Workgroup = 16 query rows x 1 head, 4 waves x 4 rows. Key tiles of kt_n (64,
+// or 32 where wide keys would not fit the LDS) are staged in LDS as fp32; in the score phase a lane owns one key (4 rows
 // register-blocked), in the PV phase a lane owns value channels.
 constexpr int kAttnQT = 16;
 constexpr int kAttnKT = 64;
@@ -325,7 +335,7 @@ __global__ __launch_bounds__(256) void chunk_bias_attn_prefill_kernel(
     const int* __restrict__ q_start,       // [B] position of a sequence's first query
     int H, int G, int D, int DV, int block_size, int span, float scale,
     int v_row, int mask_mode, int bias_mode, int keep_first, const float* __restrict__ sink,
-    float softcap, int gate_cols, int weight_fn, const float* __restrict__ wbias) {
+    float softcap, int gate_cols, int weight_fn, const float* __restrict__ wbias, int kt_n) {
   extern __shared__ float smem[];
   const bool sig = weight_fn == kWeightSigmoid;
   const float wb = sig && wbias ? wbias[blockIdx.y] : 0.f;
@@ -343,9 +353,9 @@ __global__ __launch_bounds__(256) void chunk_bias_attn_prefill_kernel(
   // K tile: no V tile of their own
   const bool v_alias = v_cache == k_cache;
   const int VP = v_alias ? DP : DV;         // row stride of the V tile
-  float* Ks = smem;                         // [KT][D+1]
-  float* Vs = v_alias ? Ks : Ks + kAttnKT * DP;            // [KT][DV]
-  float* Qs = Ks + kAttnKT * DP + (v_alias ? 0 : kAttnKT * DV);   // [QT][D]
+  float* Ks = smem;                         // [kt_n][D+1]
+  float* Vs = v_alias ? Ks : Ks + kt_n * DP;               // [kt_n][DV]
+  float* Qs = Ks + kt_n * DP + (v_alias ? 0 : kt_n * DV);  // [QT][D]
   float* Ps = Qs + kAttnQT * D;             // [QT][KT]
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
 
@@ -369,8 +379,8 @@ __global__ __launch_bounds__(256) void chunk_bias_attn_prefill_kernel(
   const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
   for (int kt = first_end > 0 ? 0 : lo; kt <= pos_last;) {
     const bool in_first = kt < first_end;
-    const int kt_next = (in_first && kt + kAttnKT >= first_end) ? lo : kt + kAttnKT;
-    const int nk = min(kAttnKT, (in_first ? first_end : pos_last + 1) - kt);
+    const int kt_next = (in_first && kt + kt_n >= first_end) ? lo : kt + kt_n;
+    const int nk = min(kt_n, (in_first ? first_end : pos_last + 1) - kt);
     __syncthreads();
     for (int idx = tid; idx < nk * D; idx += 256) {
       const int jj = idx / D, d = idx % D;
@@ -512,7 +522,8 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
   // portion). ps = 0: all rows of a sequence sit at q_start — the rows are the
   // query HEADS of one new token that share one kv head, laid out as rows of
   // a single head, so a decode step over a latent cache runs on the matrix
-  // cores with every key tile staged once for all heads.
+  // cores with every key tile staged once for all heads. sink and the gate
+  // (one per head) are then indexed by the row: sink[row], gate[b, row].
   extern __shared__ __align__(16) unsigned char smem_raw[];
   constexpr int VG = DT / 2;             // 32-channel groups of V per thread
   const int b = blockIdx.z, h = blockIdx.y % H, sp = blockIdx.y / H;
@@ -743,7 +754,7 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
     const long trow = row0 + r0 + r;
     if (sink && n_split == 1) {
       float rescale;
-      add_sink(m[reg], ll, rescale, sink[h]);
+      add_sink(m[reg], ll, rescale, sink[ps ? h : r0 + r]);
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) o[dt][reg] *= rescale;
     }
@@ -766,37 +777,47 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
       const int c = dt * 16 + col;
       if (dt < dtn && c < DV)
         out[trow * out_stride + (long)h * DV + c] = __float2bfloat16(
-            o[dt][reg] * inv * head_gate(gate, trow * g_stride, gate_cols, h, c));
+            o[dt][reg] * inv * (ps ? head_gate(gate, trow * g_stride, gate_cols, h, c)
+                                   : head_gate(gate, (long)b * g_stride, 1, r0 + r, c)));
     }
   }
 }
 
 // Merge of key splits: out[row, head] = sum_s o_s e^(m_s - M) / sum_s l_s e^(m_s - M),
-// M = max_s m_s; a split that saw no key has m = -inf and counts nothing.
-// One wave per (row, head), lanes over value channels.
+// M = max_s m_s; a split that saw no key has m = -inf and counts nothing. A
+// sink joins as one more l; rows are the hps query heads of one sequence each
+// (sink [hps], gate [sequence, hps]). One wave per (row, head), lanes over
+// value channels.
 __global__ __launch_bounds__(256) void attn_merge_splits_kernel(
     __hip_bfloat16* __restrict__ out, long out_stride, const float* __restrict__ part,
-    long pairs, int H, int DV, int n_split) {
+    long pairs, int H, int DV, int n_split, const float* __restrict__ sink,
+    const __hip_bfloat16* __restrict__ gate, long g_stride, int hps) {
   const long pair = blockIdx.x * 4L + (threadIdx.x >> 6);
   if (pair >= pairs) return;
   const int lane = threadIdx.x & 63;
   const float* pp = part + pair * n_split * (long)(DV + 2);
   float M = -INFINITY;
   for (int sidx = 0; sidx < n_split; ++sidx) M = fmaxf(M, pp[sidx * (DV + 2) + DV]);
+  const long row = pair / H;
+  const int h = (int)(pair % H);
   float L = 0.f;
+  if (sink) {
+    const float sk = sink[row % hps];
+    M = fmaxf(M, sk);
+    L = expf(sk - M);
+  }
   for (int sidx = 0; sidx < n_split; ++sidx) {
     const float ms = pp[sidx * (DV + 2) + DV];
     if (ms > -INFINITY) L += pp[sidx * (DV + 2) + DV + 1] * expf(ms - M);
   }
-  const long row = pair / H;
-  const int h = (int)(pair % H);
+  const float gs = head_gate(gate, (row / hps) * g_stride, 1, (int)(row % hps), 0) / L;
   for (int c = lane; c < DV; c += 64) {
     float a = 0.f;
     for (int sidx = 0; sidx < n_split; ++sidx) {
       const float ms = pp[sidx * (DV + 2) + DV];
       if (ms > -INFINITY) a += pp[sidx * (DV + 2) + c] * expf(ms - M);
     }
-    out[row * out_stride + (long)h * DV + c] = __float2bfloat16(a / L);
+    out[row * out_stride + (long)h * DV + c] = __float2bfloat16(a * gs);
   }
 }
 

@@ -263,8 +263,11 @@ def rmsnorm_cast(x: torch.Tensor, weight: torch.Tensor, eps: float, offset: floa
 
 def sandwich_norm_res32(x, residual, w_post, w_pre, eps, offset, groups=1):
     """residual(fp32) += rmsnorm(x)*(w_post+offset); returns
-    rmsnorm(residual)*(w_pre+offset) in x's dtype. residual updated in place."""
+    rmsnorm(residual)*(w_pre+offset) in x's dtype (w_pre None: the residual
+    itself). residual updated in place."""
     residual.add_(rmsnorm_cast(x, w_post, eps, offset, torch.float32, groups))
+    if w_pre is None:
+        return residual.to(x.dtype, copy=True)
     return rmsnorm_cast(residual, w_pre, eps, offset, x.dtype, groups)
 
 
@@ -479,11 +482,12 @@ def window_attn_decode(q, k_cache, v_cache, dv, block_tables, context_lens, wind
     return out
 
 
-def _rotate(x, positions, inv_freq, rot_dims, interleaved):
-    """x [T, ..., n] fp32: rotary positions on its first rot_dims channels."""
+def _rotate(x, positions, inv_freq, rot_dims, interleaved, amplitude=1.0):
+    """x [T, ..., n] fp32: rotary positions on its first rot_dims channels,
+    cos and sin times amplitude."""
     half = rot_dims // 2
     ang = positions.float().view(-1, *([1] * (x.dim() - 2)), 1) * inv_freq.float()
-    cos, sin = torch.cos(ang), torch.sin(ang)
+    cos, sin = torch.cos(ang) * amplitude, torch.sin(ang) * amplitude
     out = x.clone()
     if interleaved:
         u, v = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
@@ -497,18 +501,26 @@ def _rotate(x, positions, inv_freq, rot_dims, interleaved):
 
 
 def latent_rope_pack(q, q_lat, ckr, c_w, inv_freq, positions, k_cache, slots, dim, rot_dims,
-                     interleaved, eps):
+                     interleaved, eps, amplitude=1.0, out=None):
     """q [T, H, dim+DR] (projection), q_lat [T, H, R] (its unrotated part
-    mapped into the latent), ckr [T, R+DR] (latent ‖ rotated key part).
-    Returns the packed query [T, H, R+DR] = q_lat ‖ rotate(q[..., dim:]) and
-    scatters rmsnorm(latent)*c_w ‖ rotate(key part) into the paged cache
+    mapped into the latent; None: out's first R channels hold it), ckr
+    [T, R+DR] (latent ‖ rotated key part; None: nothing is cached). Returns
+    the packed query [T, H, R+DR] = q_lat ‖ rotate(q[..., dim:]) and scatters
+    rmsnorm(latent)*c_w ‖ rotate(key part) into the paged cache
     [blocks, 1, bs, R+DR]."""
     T, H, _ = q.shape
-    R = q_lat.shape[2]
-    q_rot = _rotate(q[..., dim:].float(), positions, inv_freq, rot_dims, interleaved)
-    out = torch.cat([q_lat.float(), q_rot], dim=-1).to(q.dtype)
+    DR = q.shape[2] - dim
+    if out is None:
+        out = q.new_empty(T, H, q_lat.shape[2] + DR)
+    R = out.shape[2] - DR
+    if q_lat is not None:
+        out[..., :R] = q_lat
+    out[..., R:] = _rotate(q[..., dim:].float(), positions, inv_freq, rot_dims, interleaved,
+                           amplitude).to(q.dtype)
+    if ckr is None:
+        return out
     c = rmsnorm_cast(ckr[:, :R], c_w, eps, 0.0, torch.float32)
-    k_rot = _rotate(ckr[:, R:].float(), positions, inv_freq, rot_dims, interleaved)
+    k_rot = _rotate(ckr[:, R:].float(), positions, inv_freq, rot_dims, interleaved, amplitude)
     row = torch.cat([c, k_rot], dim=-1)
     bs = k_cache.shape[2]
     keep = slots >= 0
@@ -789,6 +801,43 @@ def qkv_norm_rope_cache(q, k, v, q_w, k_w, inv_freq, rot_dims, positions, k_cach
     v_cache[s // bs, :, s % bs, :] = vf[keep].to(v_cache.dtype)
 
 
+def rownorm_rope_cache(q, k, q_w, k_w, inv_freq, rot_dims, positions, k_cache, v_cache, slots, eps,
+                       amplitude=1.0, conv=None):
+    """q [T, H, D] (updated in place) and k [T, G, D] normed over all their
+    heads at once, rotated in adjacent pairs on the first rot_dims channels of
+    every head, k and the raw keys (as values) scattered into the paged cache
+    (negative slots: skipped). conv: the short convolution in front, for rows
+    that are their sequence's only one."""
+    T, H, D = q.shape
+    G = k.shape[1]
+    if conv is not None:
+        w, tail, rec_slots, fresh, q_at, k_at = conv
+        cu = torch.arange(T + 1)
+
+        def step(x, at):
+            n = x.shape[1] * D
+            part = tail[:, :, at:at + n].contiguous()
+            y = causal_conv_silu(x.reshape(T, n), w[at:at + n], None, part, cu, rec_slots, fresh,
+                                 silu=False)
+            tail[:, :, at:at + n] = part
+            return y.view(x.shape)
+
+        q.copy_(step(q, q_at))
+        k = step(k, k_at)
+
+    def normed(x, weight):
+        y = rmsnorm_cast(x.reshape(T, -1), weight, eps, 0.0, torch.float32).view(x.shape)
+        return _rotate(y, positions, inv_freq, rot_dims, True, amplitude) if rot_dims else y
+
+    q.copy_(normed(q, q_w).to(q.dtype))
+    kn = normed(k, k_w)
+    bs = k_cache.shape[2]
+    keep = slots >= 0
+    s = slots[keep].long()
+    k_cache[s // bs, :, s % bs, :] = kn[keep].to(k_cache.dtype)
+    v_cache[s // bs, :, s % bs, :] = k[keep].to(v_cache.dtype)
+
+
 def rotate_heads(x, positions, inv_freq, inverse):
     """x [T, H, n] in place: every head turned by (minus, if inverse) its
     token's position over all n channels, pairs (i, i + n/2)."""
@@ -890,7 +939,8 @@ def gated_delta_rule(q, k, v, z, z_bias, rate, beta, state, cu, slots, fresh, q_
     kf = kf / torch.sqrt(kf.pow(2).sum(-1, keepdim=True) + 1e-6)
     qf = qf.repeat_interleave(H // Hk, dim=1)
     kf = kf.repeat_interleave(H // Hk, dim=1)
-    step = torch.nn.functional.softplus(z.float() + z_bias.float().view(1, H, D))
+    zf = z.float() if z.dim() == 3 else z.float().unsqueeze(-1)      # one decay per head
+    step = torch.nn.functional.softplus(zf + z_bias.float().view(1, H, -1))
     g = torch.exp(-rate.float().view(1, H, 1) * step)
     b = torch.sigmoid(beta.float())
     vf = v.float()
