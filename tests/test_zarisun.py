@@ -1,0 +1,903 @@
+"""Zarisun (windowed attention on convolved keys, a delta rule with one decay
+per head, latent attention on shared caches) against the plain oracle in
+zarisun_oracle.py.
+
+Every test builds its own small configuration and random checkpoint, loads
+it through the engine's own entry points (config reader, weight loader,
+scheduler, cache and state managers) and compares logits with the oracle.
+The scenarios run on the CPU (torch reference ops) and, marked ``gpu``, on
+the HIP kernels in fp32 (sharp) and bf16.
+"""
+
+from __future__ import annotations
+
+import json
+import math
+
+import pytest
+import torch
+
+import zarisun_oracle as oracle
+from llmq_amd import ops
+from llmq_amd.engine.config import EngineConfig
+from llmq_amd.engine.engine import LLMEngine
+from llmq_amd.engine.sampling_params import SamplingParams
+
+
+# --------------------------------------------------------------- fixtures --
+
+def rot_cfg(base, dims, scaling):
+    rot = {"base": base, "dims": dims}
+    if scaling:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    return rot
+
+
+def attn(heads=4, kv_heads=2, dim=16, rot_dims=8, base=900.0, scale=0.4, window=13, conv=3,
+         scaling=(4.0, 60, 6.0, 0.7), ff=40):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": scale, "conv": conv,
+         "rot": rot_cfg(base, rot_dims, scaling)}
+    if window:
+        m["mask"] = {"size": window}
+    return {"type": "attention", "mixer": m, "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def delta(heads=4, kv_heads=2, dim=8, vdim=12, conv=4, ff=40):
+    return {"type": "delta", "mlp": {"kind": "dense", "ff": ff} if ff else None,
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}}
+
+
+def lat(heads=4, dim=12, rot_dim=8, vdim=20, rank=24, base=3000.0, scale=0.35, kv_from=None,
+        window=0, scaling=(8.0, 100, 16.0, 1.0), ff=40):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": rank,
+         "scale": scale, "rot": rot_cfg(base, rot_dim, scaling)}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    if window:
+        m["mask"] = {"size": window}
+    return {"type": "latent_attention", "mixer": m,
+            "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def make_config(layers, width=48, vocab=128, eps=1e-5, logit_scale=0.7):
+    return {"architecture": "Zarisun", "layers": layers, "norm": {"eps": eps}, "vocab": vocab,
+            "width": width, "logit_scale": logit_scale}
+
+
+def make_tensors(cfg, seed=0):
+    g = torch.Generator().manual_seed(seed)
+
+    def rnd(*shape, std=1.0, mean=0.0):
+        return (torch.randn(shape, generator=g) * std + mean).to(torch.bfloat16)
+
+    def lin(out, inn, gain=1.0):
+        return rnd(out, inn, std=gain / math.sqrt(inn))
+
+    W, V = cfg["width"], cfg["vocab"]
+    t = {"embed": rnd(V, W), "final.norm": rnd(W, std=0.1, mean=0.9)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        mx, H, D, DV = p + "mix.", m["heads"], m["dim"], m["vdim"]
+        t[p + "norm1"] = rnd(W, std=0.1, mean=0.6)
+        if layer["type"] == "attention":
+            for name, rows in (("q", H * D), ("k", m["kv_heads"] * D)):
+                t[mx + name] = lin(rows, W)
+                t[mx + name + ".conv"] = rnd(rows, m["conv"], std=0.9 / math.sqrt(m["conv"]))
+                t[mx + name + ".norm"] = rnd(rows, std=0.2, mean=1.0)
+            t[mx + "sink"], t[mx + "g"] = rnd(H, std=1.5), lin(H, W)
+        elif layer["type"] == "delta":
+            G = m["kv_heads"]
+            for name, rows in (("q", G * D), ("k", G * D), ("v", H * DV)):
+                t[mx + name] = lin(rows, W)
+                t[mx + name + ".conv"] = rnd(rows, m["conv"], std=0.9 / math.sqrt(m["conv"]))
+            t[mx + "b"], t[mx + "a"], t[mx + "g"] = lin(H, W), lin(H, W, 0.7), lin(H * DV, W)
+            t[mx + "A_log"], t[mx + "dt_bias"] = rnd(H, std=0.7, mean=-1.0), rnd(H, std=0.7, mean=-1.0)
+            t[mx + "norm"] = rnd(DV, std=0.1, mean=1.0)
+        else:
+            R, DR = m["kv_rank"], m["rot_dim"]
+            t[mx + "q"] = lin(H * (D + DR), W)
+            if m.get("kv_from") is None:
+                t[mx + "dkv"], t[mx + "dkv.norm"] = lin(R + DR, W), rnd(R, std=0.2, mean=1.0)
+            t[mx + "uk"], t[mx + "uv"] = lin(H * D, R), lin(H * DV, R)
+            t[mx + "sink"], t[mx + "g"] = rnd(H, std=1.5), lin(H, W)
+        t[mx + "o"] = lin(W, H * DV)
+        if layer["mlp"]:
+            ff = layer["mlp"]["ff"]
+            t[p + "norm2"] = rnd(W, std=0.1, mean=0.6)
+            t[p + "mlp.gate"], t[p + "mlp.up"] = lin(ff, W), lin(ff, W)
+            t[p + "mlp.down"] = lin(W, ff)
+    return t
+
+
+def write_checkpoint(path, cfg, tensors):
+    from safetensors.torch import save_file
+
+    path.mkdir(parents=True, exist_ok=True)
+    (path / "config.json").write_text(json.dumps(cfg))
+    save_file({k: v.contiguous() for k, v in tensors.items()}, str(path / "model.safetensors"))
+    return str(path)
+
+
+def mixed_layers():
+    """Every switch at once: the three mixers, grouped, single and ungrouped kv
+    heads, partial and whole rotation with and without stretched context, a
+    cache shared by two layers while another latent layer has its own, several
+    windows, layers with and without a feed-forward."""
+    return [
+        lat(heads=3, dim=8, rot_dim=4, vdim=16, rank=12, scaling=None),
+        attn(),
+        delta(),
+        lat(),
+        attn(heads=8, kv_heads=1, dim=24, rot_dims=24, window=40, conv=2, scale=0.3, scaling=None),
+        lat(heads=6, dim=8, vdim=12, kv_from=3, scale=0.4, ff=0),
+        delta(heads=3, kv_heads=3, dim=20, vdim=8, conv=2, ff=17),
+        lat(heads=8, dim=16, vdim=8, kv_from=0, rot_dim=4, rank=12, scale=0.3, scaling=None,
+            ff=24),
+        attn(heads=3, kv_heads=3, dim=12, rot_dims=4, window=0, conv=4, ff=0),
+        lat(heads=2, dim=10, vdim=10, kv_from=3, window=21),
+    ]
+
+
+def tokens_for(n, vocab, seed):
+    g = torch.Generator().manual_seed(5000 + seed)
+    return torch.randint(0, vocab, (n,), generator=g).tolist()
+
+
+DEVICES = [
+    pytest.param(("cpu", "float32"), id="cpu"),
+    pytest.param(("cuda", "float32"), id="hip-fp32", marks=pytest.mark.gpu),
+    pytest.param(("cuda", "bfloat16"), id="hip-bf16", marks=pytest.mark.gpu),
+]
+
+
+def make_engine(path, target, blocks=64, block_size=16, max_seqs=4, prefill_budget=4096,
+                max_len=1024):
+    device, dtype = target
+    return LLMEngine(EngineConfig(
+        model=path, device=device, dtype=dtype, max_num_seqs=max_seqs, max_model_len=max_len,
+        num_kv_blocks=blocks, kv_block_size=block_size, max_prefill_tokens=prefill_budget))
+
+
+def assert_close(got, want, target, what=""):
+    """Relative rms error per row: fp32 is the sharp comparison; bf16 rounds
+    every GEMM input and output of a deep stack and has to stay at rounding
+    level (nine rows in ten, and the median)."""
+    got, want = got.double().cpu(), want.double()
+    err = (got - want).pow(2).mean(-1).sqrt() / want.pow(2).mean(-1).sqrt()
+    if target[1] == "bfloat16":
+        worst = float(err.quantile(0.9)) if err.numel() >= 10 else float(err.min())
+        mean, lim_worst, lim_mean = float(err.median()), 6e-2, 3e-2
+    else:
+        worst, mean, lim_worst, lim_mean = float(err.max()), float(err.mean()), 1e-4, 3e-5
+    assert worst < lim_worst, f"{what}: worst row error {worst:.3e} at row {int(err.argmax())}"
+    assert mean < lim_mean, f"{what}: mean row error {mean:.3e}"
+
+
+def replay(engine, rid, toks, cuts, end=True):
+    """One request alone, cut into the given portion sizes; all logits."""
+    out, at = [], 0
+    for n in cuts:
+        last = at + n == len(toks)
+        out.append(engine.replay_step(
+            [{"id": rid, "tokens": toks[at:at + n], "want": list(range(n))}],
+            end=[rid] if (last and end) else []))
+        at += n
+    assert at == len(toks)
+    return torch.cat(out)
+
+
+def f64(tensors):
+    return {k: v.double() for k, v in tensors.items()}
+
+
+@pytest.fixture(scope="module")
+def mixed_model(tmp_path_factory):
+    """(config, float64 tensors, path) of the all-switches model."""
+    cfg = make_config(mixed_layers())
+    tensors = make_tensors(cfg, seed=11)
+    return cfg, f64(tensors), write_checkpoint(tmp_path_factory.mktemp("zs") / "m", cfg, tensors)
+
+
+_WANT = {}
+
+
+def oracle_logits(cfg, tensors, toks):
+    key = (id(tensors), tuple(toks))
+    if key not in _WANT:
+        _WANT[key] = oracle.forward(cfg, tensors, toks)
+    return _WANT[key]
+
+
+def dev_dtype(target):
+    return target[0], (torch.bfloat16 if target[1] == "bfloat16" else torch.float32)
+
+
+# ------------------------------------------------------ config and layout --
+
+def test_config_reader_takes_everything_from_config(tmp_path):
+    from llmq_amd.engine.model_specs import resolve_spec
+
+    cfg = make_config(mixed_layers())
+    tensors = make_tensors(cfg)
+    path = write_checkpoint(tmp_path / "m", cfg, tensors)
+    spec = resolve_spec(path)
+    assert spec.family == "zarisun" and spec.num_layers == 10 and spec.hidden_size == 48
+    assert (spec.vocab_size, spec.rms_eps, spec.logit_scale) == (128, 1e-5, 0.7)
+    assert [ls.mixer.kind for ls in spec.layers] == [
+        "latent_attention", "attention", "delta", "latent_attention", "attention",
+        "latent_attention", "delta", "latent_attention", "attention", "latent_attention"]
+    assert [ls.ff for ls in spec.layers] == [40, 40, 40, 40, 40, 0, 17, 24, 0, 40]
+    a = spec.layers[1].mixer
+    assert (a.heads, a.kv_heads, a.dim, a.vdim, a.scale, a.conv, a.window) == \
+        (4, 2, 16, 16, 0.4, 3, 13)
+    assert (a.rot.base, a.rot.dims, a.rot.layout) == (900.0, 8, "interleaved")
+    sc = a.rot_scaling
+    assert (sc.factor, sc.original, sc.fast, sc.slow) == (4.0, 60.0, 6.0, 0.7)
+    assert abs(sc.amplitude - (1 + 0.1 * math.log(4.0))) < 1e-12
+    assert spec.layers[4].mixer.rot_scaling is None and spec.layers[8].mixer.window == 0
+    d = spec.layers[6].mixer
+    assert (d.heads, d.kv_heads, d.dim, d.vdim, d.conv) == (3, 3, 20, 8, 2)
+    m = spec.layers[9].mixer
+    assert (m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank, m.scale, m.window, m.kv_from) == \
+        (2, 10, 8, 10, 24, 0.35, 21, 3)
+    assert [spec.cache_layer(i) for i in range(10)] == [0, 1, 2, 3, 4, 3, 6, 0, 8, 3]
+    assert spec.param_count() == sum(v.numel() for v in tensors.values())
+    eng = make_engine(path, ("cpu", "float32"))
+    # only owners of a latent hold rows; a delta layer holds none
+    assert [kc is None for kc in eng.kv_cache.k] == [False, False, True, False, False, True, True,
+                                                     True, False, True]
+    assert eng.kv_cache.k[3].shape[1:] == (1, 16, 32) and eng.kv_cache.v[3] is None
+    assert eng.kv_cache.k[1].shape[1:] == eng.kv_cache.v[1].shape[1:] == (2, 16, 16)
+    tail, = eng.state_cache.state[1]
+    assert tail.shape[1:] == (2, 96) and eng.state_cache.state[3] is None
+    S, tail = eng.state_cache.state[2]
+    assert S.shape[1:] == (4, 8, 12) and tail.shape[1:] == (3, 80)
+    vd = attn()
+    vd["mixer"]["vdim"] = 8
+    for bad in ([dict(attn(), type="lstm")], [attn(heads=4, kv_heads=3)], [attn(conv=0)],
+                [attn(rot_dims=7)], [vd], [lat(kv_from=0)], [attn(), lat(kv_from=0)],
+                [lat(), lat(kv_from=0), lat(kv_from=1)], [lat(), lat(rank=16, kv_from=0)],
+                [lat(), lat(kv_from=0, base=7.0)], [lat(), lat(kv_from=0, scaling=None)],
+                [lat(kv_from=1), lat()], [dict(attn(), mlp={"kind": "moe", "ff": 3})]):
+        with pytest.raises(ValueError):
+            resolve_spec(write_checkpoint(tmp_path / "bad", make_config(bad), {}))
+
+
+@pytest.mark.parametrize("name", ["l0.mix.k.conv", "l0.mix.q.norm", "l1.mix.sink", "l1.mix.dkv.norm",
+                                  "l2.mix.dt_bias", "l0.norm2", "embed"])
+def test_a_missing_tensor_is_refused(tmp_path, name):
+    cfg = make_config([attn(), lat(), delta()])
+    tensors = make_tensors(cfg)
+    del tensors[name]
+    with pytest.raises(KeyError):
+        make_engine(write_checkpoint(tmp_path / "m", cfg, tensors), ("cpu", "float32"))
+
+
+@pytest.mark.parametrize("base,dims,scaling", [
+    (900.0, 8, None), (10000.0, 64, (8.0, 4096, 32.0, 1.0)), (900.0, 8, (4.0, 60, 6.0, 0.7)),
+    (500000.0, 32, (40.0, 8192, 32.0, 1.0)), (100.0, 16, (2.0, 10, 32.0, 1.0)),
+    (50.0, 4, (16.0, 1 << 20, 2.0, 1.0)), (1000.0, 2, (8.0, 512, 1.0, 1.0)),
+    (10.0, 24, (1.0, 300, 9.0, 2.0)), (20000.0, 16, (3.0, 128, 1.5, 1.4))])
+def test_stretched_frequencies(base, dims, scaling):
+    """A ramp inside, ends cut at the first and last index, a ramp past every
+    pair, a context so short that every pair slows down, a factor of 1."""
+    from llmq_amd.engine.model_specs import YarnScaling
+    from llmq_amd.engine.models.rotary import yarn_inv_freq
+
+    got = yarn_inv_freq(base, dims, YarnScaling(*map(float, scaling)) if scaling else None)
+    want = torch.tensor(oracle.frequencies(rot_cfg(base, dims, scaling)), dtype=torch.float64)
+    assert ((got.double() - want).abs() / want).max() < 1e-6
+
+
+# ------------------------------------------------------ mechanisms alone --
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("layers,kw", [
+    ([attn()], {}),
+    ([attn(heads=3, kv_heads=3, dim=8, rot_dims=8, window=1, conv=1, scaling=None)], {}),
+    ([attn(heads=8, kv_heads=1, dim=16, rot_dims=2, scale=1.0, window=0, conv=8)], {}),
+    ([attn(heads=1, kv_heads=1, dim=2, rot_dims=2, window=2, conv=2, ff=0)], {"logit_scale": 1.0}),
+    ([attn(heads=6, kv_heads=2, dim=24, rot_dims=0, window=36, ff=3)], {"logit_scale": 3.0}),
+    ([attn(window=5), attn(window=30), attn(window=16)], {}),
+    ([delta()], {}),
+    ([delta(heads=1, kv_heads=1, dim=32, vdim=32, conv=1, ff=0)], {}),
+    ([delta(heads=6, kv_heads=1, dim=5, vdim=70, conv=2)], {}),
+    ([delta(heads=2, kv_heads=2, dim=130, vdim=3, conv=6)], {}),
+    ([lat()], {}),
+    ([lat(heads=1, dim=4, rot_dim=2, vdim=4, rank=4, scaling=None, ff=0)], {"eps": 1e-3}),
+    ([lat(heads=8, dim=20, rot_dim=12, vdim=8, rank=40)], {}),
+    ([lat(heads=16, dim=8, rot_dim=8, vdim=24, rank=56, window=9)], {}),
+    ([lat(), lat(heads=2, dim=20, vdim=8, kv_from=0, scale=0.6), lat(heads=8, kv_from=0, ff=0)], {}),
+], ids=["attn", "attn-window-1-no-conv", "attn-causal-one-kv-head", "attn-ones", "attn-unrotated",
+        "attn-windows", "delta", "delta-no-conv", "delta-one-key-head", "delta-wide-key", "latent",
+        "latent-ones", "latent-one-tile", "latent-16-heads-window", "latent-shared"])
+def test_mechanism_alone(tmp_path, target, layers, kw):
+    cfg = make_config(layers, **kw)
+    tensors = make_tensors(cfg, seed=3)
+    path = write_checkpoint(tmp_path / "m", cfg, tensors)
+    toks = tokens_for(37, cfg["vocab"], 1)
+    eng = make_engine(path, target)
+    eng.model.taps = []
+    got = replay(eng, "a", toks, [37])
+    taps = []
+    want = oracle.forward(cfg, f64(tensors), toks, taps)
+    for i, (g, w) in enumerate(zip(eng.model.taps, taps)):
+        assert_close(g, w, target, f"stream after layer {i}")
+    assert_close(got, want, target, "logits")
+    eng.model.taps = None
+    assert_close(replay(eng, "b", toks, [5, 1, 2, 20, 1, 1, 7]), want, target, "portions")
+
+
+@pytest.mark.parametrize("target", DEVICES)
+def test_sizes_that_fit_no_vector_width(tmp_path, target):
+    layers = [attn(heads=3, kv_heads=1, dim=7, rot_dims=6, conv=3, ff=9),
+              delta(heads=3, kv_heads=1, dim=5, vdim=7, conv=5, ff=11),
+              lat(heads=5, dim=3, rot_dim=6, vdim=7, rank=13, ff=5),
+              lat(heads=9, dim=11, rot_dim=6, vdim=5, rank=13, kv_from=2),
+              attn(heads=9, kv_heads=1, dim=10, rot_dims=10, window=7)]
+    cfg = make_config(layers, width=27, vocab=61)
+    tensors = make_tensors(cfg, seed=5)
+    path = write_checkpoint(tmp_path / "m", cfg, tensors)
+    toks = tokens_for(41, 61, 2)
+    want = oracle.forward(cfg, f64(tensors), toks)
+    eng = make_engine(path, target)
+    assert_close(replay(eng, "a", toks, [41]), want, target, "whole")
+    assert_close(replay(eng, "b", toks, [7, 1, 1, 30, 2]), want, target, "portions")
+
+
+@pytest.mark.parametrize("target", DEVICES)
+def test_wider_model_with_other_sizes(tmp_path, target):
+    """Head sizes that take the 16-byte paths and the matrix-core tiles, more
+    keys than one tile, a key row wider than a tile of the matrix cores, whole,
+    cut and in a batch."""
+    layers = [attn(heads=8, kv_heads=2, dim=48, rot_dims=32, window=100, scale=0.15, ff=96),
+              delta(heads=4, kv_heads=2, dim=48, vdim=64, ff=64),
+              lat(heads=8, dim=32, rot_dim=16, vdim=40, rank=112, scale=0.2, ff=80),
+              attn(heads=16, kv_heads=1, dim=64, rot_dims=64, window=70, scale=0.12),
+              lat(heads=4, dim=40, rot_dim=16, vdim=72, rank=112, scale=0.18, kv_from=2),
+              lat(heads=2, dim=16, rot_dim=24, vdim=16, rank=264, scale=0.2)]
+    cfg = make_config(layers, width=160, vocab=300)
+    tensors = make_tensors(cfg, seed=9)
+    path = write_checkpoint(tmp_path / "m", cfg, tensors)
+    t64 = f64(tensors)
+    a, b = tokens_for(200, 300, 80), tokens_for(90, 300, 81)
+    want_a, want_b = oracle.forward(cfg, t64, a), oracle.forward(cfg, t64, b)
+    eng = make_engine(path, target, blocks=24)
+    assert_close(replay(eng, "w", a, [200]), want_a, target, "whole")
+    assert_close(replay(eng, "c", a, [63, 2, 65, 1, 1, 1, 1, 30, 36]), want_a, target, "cut")
+    # b's portions beside a's single tokens, then b's single tokens beside a's portion
+    got_a = [eng.replay_step([{"id": "a", "tokens": a[:120], "want": list(range(120))}])]
+    got_b = []
+    for k in range(40):
+        out = eng.replay_step([{"id": "a", "tokens": [a[120 + k]], "want": [0]},
+                               {"id": "b", "tokens": b[2 * k:2 * k + 2], "want": [0, 1]}])
+        got_a.append(out[:1])
+        got_b.append(out[1:])
+    out = eng.replay_step([{"id": "b", "tokens": [b[80]], "want": [0]},
+                           {"id": "a", "tokens": a[160:], "want": list(range(40))}])
+    got_b.append(out[:1])
+    got_a.append(out[1:])
+    got_b.append(eng.replay_step([{"id": "b", "tokens": b[81:], "want": list(range(9))}],
+                                 end=["a", "b"]))
+    assert_close(torch.cat(got_a), want_a, target, "a in the batch")
+    assert_close(torch.cat(got_b), want_b, target, "b in the batch")
+    assert eng.allocator.num_free == 24
+
+
+# ------------------------------------------- schedules: cuts, batches, reuse --
+
+@pytest.mark.parametrize("target", DEVICES)
+def test_prefill_equals_token_by_token(mixed_model, target):
+    cfg, tensors, path = mixed_model
+    toks = tokens_for(90, cfg["vocab"], 2)
+    want = oracle_logits(cfg, tensors, toks)
+    eng = make_engine(path, target)
+    assert_close(replay(eng, "w", toks, [90]), want, target, "whole prompt")
+    assert_close(replay(eng, "d", toks, [1] * 90), want, target, "token by token")
+    assert eng.allocator.num_free == eng.allocator.num_blocks
+    assert eng.slot_allocator.num_free == 4
+
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("cuts", [
+    [2] * 45,
+    [1, 2, 3, 5, 8, 13, 21, 34, 3],
+    [16, 16, 16, 16, 16, 10],                  # at page borders
+    [15, 2, 15, 17, 31, 1, 1, 8],              # around page borders
+    [13, 13, 1, 13, 27, 23],                   # at the smallest window's edge
+    [64, 1, 1, 1, 1, 1, 1, 1, 1, 1, 17],
+    [3, 87],
+], ids=["twos", "growing", "pages", "around-pages", "windows", "decode-then-portion", "short-first"])
+def test_portions(mixed_model, target, cuts):
+    cfg, tensors, path = mixed_model
+    toks = tokens_for(90, cfg["vocab"], 3)
+    want = oracle_logits(cfg, tensors, toks)
+    eng = make_engine(path, target)
+    assert_close(replay(eng, "c", toks, cuts), want, target, f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("target", DEVICES)
+def test_mixed_batches_equal_alone_and_reuse(mixed_model, target):
+    """Six unequal requests through four slots and a pool that cannot hold
+    them all at once: portions beside single tokens, requests that pause,
+    blocks and slots handed on to later requests."""
+    cfg, tensors, path = mixed_model
+    lens = {"a": 70, "b": 9, "c": 41, "d": 130, "e": 25, "f": 3}
+    toks = {r: tokens_for(n, cfg["vocab"], 10 + i) for i, (r, n) in enumerate(lens.items())}
+    want = {r: oracle_logits(cfg, tensors, t) for r, t in toks.items()}
+    eng = make_engine(path, target, blocks=14, block_size=16)
+    at = {r: 0 for r in lens}
+    got = {r: [] for r in lens}
+    plan = [
+        {"a": 33, "b": 2, "c": 17},
+        {"a": 1, "b": 1, "c": 24, "d": 40},
+        {"a": 1, "b": 6, "d": 2},              # c pauses at its end; b ends
+        {"a": 35, "d": 1, "e": 25},            # e takes b's slot and blocks
+        {"d": 1},
+        {"d": 86, "f": 3},                     # a, c, e ended; f reuses
+    ]
+    ends = [[], [], ["b"], ["a", "e"], ["c"], ["d", "f"]]
+    slots_seen = set()
+    for step, end in zip(plan, ends):
+        entries = [{"id": r, "tokens": toks[r][at[r]:at[r] + n], "want": list(range(n))}
+                   for r, n in step.items()]
+        out = eng.replay_step(entries, end=[])
+        for s in eng._seqs.values():
+            slots_seen.add(s.state_slot)
+        eng.replay_step([], end=end)
+        k = 0
+        for ent in entries:
+            n = len(ent["tokens"])
+            got[ent["id"]].append(out[k:k + n])
+            at[ent["id"]] += n
+            k += n
+    assert at == lens
+    assert slots_seen <= {0, 1, 2, 3}
+    for r in lens:
+        assert_close(torch.cat(got[r]), want[r], target, f"request {r}")
+    assert eng.allocator.num_free == 14 and eng.slot_allocator.num_free == 4
+
+
+@pytest.mark.parametrize("target", DEVICES)
+def test_stale_pages_and_slots_do_not_leak(mixed_model, target):
+    """A request that runs in blocks and a slot another one just left sees
+    nothing of it: same logits as in a fresh engine."""
+    cfg, tensors, path = mixed_model
+    first = tokens_for(64, cfg["vocab"], 30)
+    second = tokens_for(50, cfg["vocab"], 31)
+    want = oracle_logits(cfg, tensors, second)
+    eng = make_engine(path, target, blocks=4, max_seqs=1)
+    replay(eng, "x", first, [60, 1, 1, 1, 1])
+    assert_close(replay(eng, "y", second, [3, 1, 1, 45]), want, target, "after reuse")
+
+
+@pytest.mark.parametrize("target", DEVICES)
+def test_long_decode_across_pages_and_windows(mixed_model, target):
+    cfg, tensors, path = mixed_model
+    toks = tokens_for(5 + 150, cfg["vocab"], 4)
+    want = oracle_logits(cfg, tensors, toks)
+    eng = make_engine(path, target)
+    assert_close(replay(eng, "l", toks, [5] + [1] * 150), want, target, "long decode")
+
+
+@pytest.mark.parametrize("target", DEVICES)
+def test_first_tokens(mixed_model, target):
+    """Requests of one to four tokens: nothing before the start, no
+    convolution full."""
+    cfg, tensors, path = mixed_model
+    eng = make_engine(path, target)
+    for n in (1, 2, 3, 4):
+        toks = tokens_for(n, cfg["vocab"], 70 + n)
+        want = oracle_logits(cfg, tensors, toks)
+        assert_close(replay(eng, f"n{n}", toks, [n]), want, target, f"{n} tokens")
+        assert_close(replay(eng, f"s{n}", toks, [1] * n), want, target, f"{n} single tokens")
+
+
+# ------------------------------------------ edges made visible by design --
+
+def _needle(device, dtype, key_pos, query_pos, decode, window=0, H=2, G=1, D=16, DV=8, raw=8.0,
+            page=16, sink=None, gate=None, latent=False):
+    """Every key scores 0 and has value 0, but the needle at key_pos: raw
+    score `raw`, value 1 in channel 1; behind the query lie stale rows of score
+    30 and value 50. The output's channel 1 is then the weight the needle gets.
+    Pages are handed out in reverse order. latent: values are the first
+    channels of the key rows (the score sits in the last one)."""
+    n = query_pos + 1
+    nblocks = (n + page - 1) // page
+    kc = torch.zeros(nblocks + 2, G, page, D, dtype=dtype)
+    vc = kc if latent else torch.zeros(nblocks + 2, G, page, DV, dtype=dtype)
+    table = torch.arange(nblocks + 1, 0, -1, dtype=torch.int32).view(1, -1)
+    at = D - 1 if latent else 0
+    for pos, score, value in [(j, 30.0, 50.0) for j in range(n, nblocks * page)] + \
+            [(key_pos, raw, 1.0)]:
+        b, o = int(table[0, pos // page]), pos % page
+        kc[b, :, o, at] = score
+        vc[b, :, o, 1] = value
+    kc, table = kc.to(device), table.to(device)
+    vc = None if latent else vc.to(device)
+    if decode:
+        q = torch.zeros(1, H, D, dtype=dtype, device=device)
+        q[0, :, at] = 1.0
+        out = ops.window_attn_decode(
+            q, kc, vc, DV, table, torch.tensor([n], dtype=torch.int32, device=device), window, 1.0,
+            sink=sink, gate=gate)
+        return out[0, :, 1].double().cpu()
+    start = max(0, query_pos - 4)            # a portion whose last row is the query
+    rows = query_pos - start + 1
+    q = torch.zeros(rows, H, D, dtype=dtype, device=device)
+    q[:, :, at] = 1.0
+    out = ops.window_attn_prefill(
+        q, kc, vc, DV, table, torch.tensor([0, rows], dtype=torch.int32, device=device),
+        torch.tensor([start], dtype=torch.int32, device=device), rows, window, 1.0, sink=sink,
+        gate=None if gate is None else gate.expand(rows, -1).contiguous())
+    return out[-1, :, 1].double().cpu()
+
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("decode", [False, True], ids=["portion", "single"])
+@pytest.mark.parametrize("H,G,D,DV,latent", [
+    (2, 1, 16, 8, False), (8, 1, 64, 64, False), (6, 2, 72, 72, False), (3, 3, 10, 10, False),
+    (8, 1, 48, 40, True), (20, 1, 136, 112, True), (70, 1, 40, 24, True), (4, 1, 26, 20, True)])
+def test_one_key_among_many_at_window_edges(target, decode, H, G, D, DV, latent):
+    """The needle just inside the window, just outside (weight 0), at page and
+    tile borders, far back; a sink per head and a gate per head in the result."""
+    device, dtype = dev_dtype(target)
+    tol = 2e-2 if dtype == torch.bfloat16 else 1e-5
+    sink = torch.linspace(-3.0, 9.0, H)
+    gate = torch.linspace(2.0, -1.0, H).to(dtype)
+    sg = torch.sigmoid(gate.double())
+    for window, query_pos in ((0, 0), (0, 700), (1, 40), (7, 100), (16, 79), (64, 64), (65, 200),
+                              (300, 1030)):
+        seen = min(query_pos + 1, window) if window else query_pos + 1
+        first = query_pos + 1 - seen
+        for key_pos in sorted({first - 1, first, first + 1, 0, 15, 16, 63, 64, query_pos - 1,
+                               query_pos}):
+            if not 0 <= key_pos <= query_pos:
+                continue
+            got = _needle(device, dtype, key_pos, query_pos, decode, window, H, G, D, DV,
+                          sink=sink.to(device), gate=gate.view(1, H).to(device), latent=latent)
+            want = torch.zeros(H, dtype=torch.float64)
+            if key_pos >= first:
+                want = sg * math.exp(8.0) / (torch.exp(sink.double()) + math.exp(8.0) + seen - 1)
+            assert ((got - want).abs() <= tol * want).all(), (window, query_pos, key_pos)
+
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("H,G,D,DV,window", [(8, 1, 64, 64, 0), (32, 1, 80, 64, 50), (9, 1, 16, 8, 0),
+                                             (64, 1, 224, 192, 0), (8, 2, 32, 32, 20)])
+def test_decode_batch_with_sink_and_gate(target, H, G, D, DV, window):
+    """Unequal contexts in one decode batch (short ones beside contexts whose
+    keys are split over workgroups) against dense rows, gates in a column
+    slice of a wider matrix."""
+    device, dtype = dev_dtype(target)
+    g = torch.Generator().manual_seed(H + D)
+    ctx = [1, 5, 64, 65, 130, 600]
+    B, page, width = len(ctx), 16, 38
+    kc = torch.randn(B * width + 1, G, page, D, generator=g).to(dtype)
+    vc = torch.randn(B * width + 1, G, page, DV, generator=g).to(dtype)
+    q = torch.randn(B, H, D, generator=g).to(dtype)
+    sink = torch.randn(H, generator=g) * 2
+    gate = torch.randn(B, H + 8, generator=g).to(dtype)[:, 8:]
+    table = (torch.randperm(B * width, generator=g) + 1).view(B, width).int()
+    scale = 2.0 * D ** -0.5
+    wide = torch.zeros(B, H + 8, dtype=dtype)
+    wide[:, 8:] = gate
+    got = ops.window_attn_decode(
+        q.to(device), kc.to(device), vc.to(device), DV, table.to(device),
+        torch.tensor(ctx, dtype=torch.int32, device=device), window, scale,
+        sink=sink.to(device), gate=wide.to(device)[:, 8:])
+    tol = 2e-2 if dtype == torch.bfloat16 else 1e-5
+    for b, n in enumerate(ctx):
+        rows = [int(table[b, j // page]) for j in range(n)]
+        k = torch.stack([kc[r, :, j % page] for j, r in enumerate(rows)]).double()   # [n, G, D]
+        v = torch.stack([vc[r, :, j % page] for j, r in enumerate(rows)]).double()
+        seen = oracle.visible(n, window)[-1:]
+        for a in range(H):
+            s = (q[b, a].double() @ k[:, a // (H // G)].T).view(1, n) * scale
+            w = oracle.softmax_with_sink(s, seen, sink[a].double())
+            want = (w @ v[:, a // (H // G)])[0] * torch.sigmoid(gate[b, a].double())
+            err = (got[b, a].double().cpu() - want).abs().max()
+            assert err < tol * want.abs().max().clamp(min=0.05), (b, a, float(err))
+
+
+# ------------------------------------------------------ ops against oracle --
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("step", [False, True], ids=["rows", "conv-step"])
+@pytest.mark.parametrize("H,G,D,rot,K", [(4, 2, 64, 32, 4), (3, 1, 40, 8, 3), (2, 2, 16, 6, 2),
+                                         (5, 1, 7, 6, 5), (1, 1, 2, 2, 1), (6, 3, 24, 0, 16),
+                                         (80, 9, 128, 128, 4), (70, 70, 33, 10, 3)])
+def test_whole_row_norm_rotate_scatter_op(target, step, H, G, D, rot, K):
+    """The per-token kernel between projections and attention, on column
+    slices of a wider matrix; a padding row writes nothing. step: each row is
+    the next token of its own sequence, convolved with the inputs its tail
+    holds; the tail moves on. Rows longer than what a workgroup holds in
+    registers included."""
+    device, dtype = dev_dtype(target)
+    g = torch.Generator().manual_seed(D + K)
+    T, page, eps, base, first = 9, 16, 1e-5, 300.0, 93
+    scaling = (4.0, 100, 8.0, 1.0)
+    rotc = rot_cfg(base, rot, scaling)
+    nq, nk = H * D, G * D
+    k_at = -(-nq // 8) * 8
+    C = k_at + -(-nk // 8) * 8
+    wide = torch.randn(T, C + 16, generator=g).to(dtype).to(device)
+    x0 = wide[:, 8:8 + C].double().cpu()
+    q = wide[:, 8:8 + nq].unflatten(1, (H, D))
+    k = wide[:, 8 + k_at:8 + k_at + nk].unflatten(1, (G, D))
+    qw = (torch.randn(nq, generator=g) * 0.2 + 1).to(dtype)
+    kw = (torch.randn(nk, generator=g) * 0.2 + 1).to(dtype)
+    table = torch.tensor(oracle.frequencies(rotc), dtype=torch.float64).float().to(device)
+    kc = torch.zeros(3, G, page, D, dtype=dtype, device=device)
+    vc = torch.zeros(3, G, page, D, dtype=dtype, device=device)
+    pos = torch.arange(first, first + T, dtype=torch.long, device=device)
+    slots = torch.arange(5, 5 + T, dtype=torch.long, device=device)
+    slots[4] = -1
+    conv, y0 = None, x0
+    if step:
+        w = torch.randn(C, K, generator=g) / math.sqrt(K)
+        tail = torch.randn(T + 1, K - 1, C, generator=g)
+        order = list(range(T - 1, -1, -1))
+        fresh = [int(b % 3 == 1) for b in range(T)]
+        tail_dev = tail.clone().to(device)
+        conv = (w.to(device), tail_dev, torch.tensor(order, dtype=torch.int32, device=device),
+                torch.tensor(fresh, dtype=torch.int32, device=device), 0, k_at)
+        past = [torch.zeros(K - 1, C, dtype=torch.float64) if fresh[b] else tail[order[b]].double()
+                for b in range(T)]
+        y0 = torch.stack([oracle.causal_conv(torch.cat([past[b], x0[b:b + 1]]), w.double())[-1]
+                          for b in range(T)])
+    ops.rownorm_rope_cache(q, k, qw.to(device), kw.to(device), table if rot else None, rot, pos, kc,
+                           vc, slots, eps, oracle.amplitude(rotc), conv)
+    yq, yk = y0[:, :nq], y0[:, k_at:k_at + nk]
+    want_q = oracle.rotate_pairs((oracle.rms(yq, eps) * qw.double()).view(T, H, D), rotc, first)
+    want_k = oracle.rotate_pairs((oracle.rms(yk, eps) * kw.double()).view(T, G, D), rotc, first)
+    want_v = yk.reshape(T, G, D).clone()
+    for w_ in (want_k, want_v):
+        w_[4] = 0.0
+    got_k = kc.permute(0, 2, 1, 3).reshape(-1, G, D)[5:5 + T].double().cpu()
+    got_v = vc.permute(0, 2, 1, 3).reshape(-1, G, D)[5:5 + T].double().cpu()
+    tol = 1e-2 if dtype == torch.bfloat16 else 5e-5
+    for got, want in ((q.double().cpu(), want_q), (got_k, want_k), (got_v, want_v)):
+        assert (got - want).abs().max().item() < tol * want.abs().max().item()
+    assert float(kc.reshape(-1, G, page, D)[0, :, :5].abs().max()) == 0.0   # rows before the slots
+    if step and K > 1:
+        cols = list(range(nq)) + list(range(k_at, k_at + nk))
+        for b in range(T):
+            want_t = torch.cat([past[b], x0[b:b + 1]])[1:][:, cols]
+            assert (tail_dev[order[b]].double().cpu()[:, cols] - want_t).abs().max() < 1e-6
+        assert torch.equal(tail_dev[T].cpu(), tail[T])      # nobody's slot
+
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("own", [True, False], ids=["own-rows", "shared-rows"])
+@pytest.mark.parametrize("H,D,DR,R,rot", [(4, 12, 8, 24, 8), (3, 5, 6, 13, 6), (8, 32, 32, 192, 32),
+                                          (2, 8, 10, 16, 4)])
+def test_latent_query_and_row_op(target, own, H, D, DR, R, rot):
+    """Packed query beside a pre-filled latent part, and the cached row
+    (latent normed, key part rotated with the amplitude) or none."""
+    device, dtype = dev_dtype(target)
+    g = torch.Generator().manual_seed(R)
+    T, page, eps, first = 11, 16, 1e-5, 50
+    rotc = rot_cfg(700.0, rot, (8.0, 64, 8.0, 1.0))
+    q = torch.randn(T, H * (D + DR) + 8, generator=g).to(dtype)
+    ckr = torch.randn(T, R + DR + 8, generator=g).to(dtype)
+    cw = (torch.randn(R, generator=g) * 0.2 + 1).to(dtype)
+    out = torch.randn(T, H, R + DR, generator=g).to(dtype)
+    cache = torch.zeros(2, 1, page, R + DR, dtype=dtype, device=device)
+    table = torch.tensor(oracle.frequencies(rotc), dtype=torch.float64).float().to(device)
+    pos = torch.arange(first, first + T, device=device)
+    slots = torch.arange(3, 3 + T, device=device)
+    slots[2] = -1
+    q3 = q.to(device)[:, 8:].unflatten(1, (H, D + DR))
+    got = ops.latent_rope_pack(q3, None, ckr.to(device)[:, 8:] if own else None,
+                               cw.to(device) if own else None, table, pos, cache if own else None,
+                               slots, D, rot, True, eps, oracle.amplitude(rotc), out=out.to(device))
+    want = out.double().clone()
+    want[:, :, R:] = oracle.rotate_pairs(q[:, 8:].double().view(T, H, D + DR)[:, :, D:], rotc, first)
+    tol = 1e-2 if dtype == torch.bfloat16 else 5e-5
+    assert (got.double().cpu() - want).abs().max() < tol * want.abs().max()
+    rows = cache.view(-1, R + DR)[3:3 + T].double().cpu()
+    c = ckr[:, 8:].double()
+    want_rows = torch.cat([oracle.rms(c[:, :R], eps) * cw.double(),
+                           oracle.rotate_pairs(c[:, R:].reshape(T, 1, DR), rotc, first)[:, 0]], -1)
+    want_rows[2] = 0.0
+    if not own:
+        want_rows.zero_()
+    assert (rows - want_rows).abs().max() <= tol * want_rows.abs().max()
+
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("H,G,D,DV,lens", [
+    (2, 1, 8, 12, [70, 1, 3, 40]), (1, 1, 32, 32, [300]), (6, 2, 5, 7, [17, 33]),
+    (4, 4, 64, 48, [5, 1, 1]), (2, 2, 16, 31, [1, 1, 1]), (2, 1, 128, 68, [21, 16]),
+    (1, 1, 200, 20, [18]), (16, 8, 40, 64, [1] * 20), (32, 16, 64, 128, [80, 3, 17, 64])])
+def test_delta_rule_with_one_decay_per_head(target, H, G, D, DV, lens):
+    """Unequal packed sequences, each cut in two calls through its state slot
+    (whose stale contents a fresh sequence ignores), against the plain
+    recurrence over the whole sequence."""
+    device, dtype = dev_dtype(target)
+    g = torch.Generator().manual_seed(H * 100 + D)
+    B, total = len(lens), [n * 2 + 1 for n in lens]
+    data = [dict(q=torch.randn(n, G, D, generator=g), k=torch.randn(n, G, D, generator=g),
+                 v=torch.randn(n, H, DV, generator=g), z=torch.randn(n, H, generator=g) * 2,
+                 b=torch.randn(n, H, generator=g) * 2) for n in total]
+    zb, rate = torch.randn(H, generator=g) - 1.0, torch.rand(H, generator=g) + 0.1
+    S = torch.full((B + 1, H, D, DV), 7.0, device=device)
+    slots = torch.tensor(list(range(B - 1, -1, -1)), dtype=torch.int32, device=device)
+    outs = [[] for _ in range(B)]
+    for part in range(2):
+        spans = [(0, n) if part == 0 else (n, f) for n, f in zip(lens, total)]
+        cu = torch.tensor([0] + list(torch.tensor([e - s for s, e in spans]).cumsum(0)),
+                          dtype=torch.int32, device=device)
+        cat = lambda key: torch.cat([d[key][s:e] for d, (s, e) in zip(data, spans)]).to(dtype).to(device)
+        fresh = torch.full((B,), 1 - part, dtype=torch.int32, device=device)
+        o = ops.gated_delta_rule(cat("q"), cat("k"), cat("v"), cat("z"), zb.to(device),
+                                 rate.to(device), cat("b"), S, cu, slots, fresh, D ** -0.5)
+        for b in range(B):
+            outs[b].append(o[int(cu[b]):int(cu[b + 1])].cpu())
+    tol = 1e-4                      # inputs are exact in both; the recurrence itself is fp32
+    of = torch.tensor([a // (H // G) for a in range(H)])
+    for b, d in enumerate(data):
+        r = {k: t.to(dtype).double() for k, t in d.items()}
+        decay = torch.exp(-rate.double() * oracle.softplus(r["z"] + zb.double()))
+        want, last = oracle.delta_recurrence(
+            (oracle.unit(r["q"]) * D ** -0.5)[:, of], oracle.unit(r["k"])[:, of], r["v"],
+            oracle.sigmoid(r["b"]), decay)
+        got_S = S[int(slots[b])].double().cpu()
+        assert (got_S - last).abs().max() < tol * last.abs().max().clamp(min=0.1), b
+        err = (torch.cat(outs[b]).double() - want).abs().max() / want.abs().max()
+        assert err < tol, (b, float(err))
+
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("decay", [1e-4, 0.3, 40.0], ids=["slow", "middle", "fast"])
+def test_delta_rule_one_write_far_back(target, decay):
+    """A single write read hundreds of tokens later survives (or fades) by
+    exactly the decays between; a second write to the same key replaces the
+    value it still holds."""
+    device, dtype = dev_dtype(target)
+    T, H, D, DV, at, again = 400, 2, 16, 24, 37, 250
+    k = torch.zeros(T, 1, D, dtype=dtype)
+    q = torch.zeros(T, 1, D, dtype=dtype)
+    v = torch.zeros(T, H, DV, dtype=dtype)
+    k[:, :, 5] = 1.0                      # idle tokens write along another key ...
+    k[at, 0, 5], k[at, 0, 3] = 0.0, 1.0
+    k[again, 0, 5], k[again, 0, 3] = 0.0, 1.0
+    q[:, :, 3] = 1.0
+    v[at], v[again] = 1.0, -2.0
+    z, step = torch.zeros(T, H, dtype=dtype), math.log(2.0)
+    beta = torch.full((T, H), -100.0, dtype=dtype)      # ... with strength 0
+    beta[at] = beta[again] = 100.0
+    S = torch.zeros(1, H, D, DV, device=device)
+    o = ops.gated_delta_rule(q.to(device), k.to(device), v.to(device), z.to(device),
+                             torch.zeros(H, device=device),
+                             torch.full((H,), decay / step, device=device), beta.to(device), S,
+                             torch.tensor([0, T], dtype=torch.int32, device=device),
+                             torch.tensor([0], dtype=torch.int32, device=device),
+                             torch.tensor([1], dtype=torch.int32, device=device), 1.0)
+    o = o.double().cpu()
+    for t in (0, at - 1):
+        assert float(o[t].abs().max()) == 0.0
+    for t in (at, at + 1, 52, 63, 64, 128, again - 1, again, again + 1, 399):
+        since, val = (t - at, 1.0) if t < again else (t - again, -2.0)
+        want = val * math.exp(-decay * since)
+        assert float((o[t] - want).abs().max()) < 2e-4 * abs(want) + 1e-30, (t, o[t], want)
+
+
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("W", [48, 27, 512, 1000, 2048, 3072, 6000, 9000])
+@pytest.mark.parametrize("final", [False, True])
+def test_output_norm_residual_op(target, W, final):
+    """Residual += normed sublayer output; the next sublayer reads the stream
+    itself (rounded), the head its norm."""
+    device, dtype = dev_dtype(target)
+    g = torch.Generator().manual_seed(W)
+    T, eps = 19, 1e-5
+    y = (torch.randn(T, W, generator=g) * 3).to(dtype)
+    res = torch.randn(T, W, generator=g)
+    w1 = (torch.randn(W, generator=g) * 0.1 + 0.6).to(dtype)
+    w2 = (torch.randn(W, generator=g) * 0.1 + 1).to(dtype)
+    r = res.clone().to(device)
+    h = ops.sandwich_norm_res32(y.clone().to(device), r, w1.to(device),
+                                w2.to(device) if final else None, eps, 0.0)
+    want_r = res.double() + oracle.rms(y.double(), eps) * w1.double()
+    want_h = oracle.rms(want_r, eps) * w2.double() if final else want_r
+    assert (r.double().cpu() - want_r).abs().max() < 2e-5
+    tol = 1e-2 if dtype == torch.bfloat16 else 1e-5
+    assert h.dtype == dtype and h.data_ptr() != r.data_ptr()
+    assert (h.double().cpu() - want_h).abs().max() < tol * want_h.abs().max()
+
+
+# -------------------------------------------- generation and entry points --
+
+@pytest.mark.parametrize("target", DEVICES[:2])
+def test_greedy_generation_through_the_scheduler(mixed_model, target):
+    """add_request / step: the scheduler's own admission, chunked prefill
+    (a budget smaller than the prompts), decode batching and sampler."""
+    cfg, tensors, path = mixed_model
+    prompts = {"p": tokens_for(21, cfg["vocab"], 40), "q": tokens_for(5, cfg["vocab"], 41),
+               "r": tokens_for(34, cfg["vocab"], 42)}
+    eng = make_engine(path, target, prefill_budget=16)
+    params = SamplingParams(temperature=0.0, max_tokens=6, ignore_eos=True)
+    for rid, toks in prompts.items():
+        eng.add_request(rid, prompt_token_ids=toks, params=params)
+    got = {rid: [] for rid in prompts}
+    while eng.has_unfinished():
+        for out in eng.step():
+            got[out.request_id].extend(out.new_token_ids)
+    for rid, toks in prompts.items():
+        assert got[rid] == oracle.greedy(cfg, tensors, toks, 6), rid
+    assert eng.allocator.num_free == eng.allocator.num_blocks
+
+
+def test_preset_runs_through_generate():
+    eng = LLMEngine(EngineConfig(model="tiny-zarisun", device="cpu", max_num_seqs=2,
+                                 max_model_len=64, num_kv_blocks=8))
+    spare = sum(lw.t["in"].shape[0] - sum(n for _, n in lw.seg.values()) for lw in eng.model.layers)
+    assert spare > 0        # alignment rows are zero: the model does not depend on them
+    total = sum(t.numel() for n, t in eng.model.named_tensors().items())
+    conv_spare = sum((lw.conv_cols - sum(n for at, n in lw.seg.values() if at < lw.conv_cols)) *
+                     lw.t["conv_w"].shape[1] for lw in eng.model.layers if "conv_w" in lw.t)
+    assert eng.spec.param_count() == total - spare * 64 - conv_spare
+    out = eng.generate_batch(["ab", "c"], SamplingParams(temperature=0.0, max_tokens=4,
+                                                         ignore_eos=True))
+    assert len(out) == 2
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_decode_graph_replays_equal_eager(mixed_model, dtype):
+    """Captured decode steps replayed several times, with eager work between
+    the replays, against the same steps run eagerly."""
+    target = ("cuda", dtype)
+    cfg, tensors, path = mixed_model
+    toks = {r: tokens_for(n, cfg["vocab"], 50 + i) for i, (r, n) in enumerate(
+        {"a": 30, "b": 12, "c": 19, "d": 9, "e": 25, "f": 14, "g": 11, "h": 21}.items())}
+    results = []
+    for eager in (True, False):
+        eng = LLMEngine(EngineConfig(model=path, device="cuda", dtype=dtype, max_num_seqs=8,
+                                     max_model_len=256, num_kv_blocks=32, enforce_eager=eager))
+        assert eng.runner.use_graphs == (not eager)
+        rows = []
+        eng.replay_step([{"id": r, "tokens": t[:-8], "want": []} for r, t in toks.items()])
+        for k in range(8, 0, -1):
+            rows.append(eng.replay_step(
+                [{"id": r, "tokens": [t[len(t) - k]], "want": [0]} for r, t in toks.items()]))
+            torch.cuda.synchronize()
+        results.append(torch.cat(rows))
+    diff = (results[0] - results[1]).abs().max() / results[0].abs().max()
+    assert diff < (3e-2 if dtype == "bfloat16" else 1e-4)
+    want = torch.cat([torch.stack([oracle_logits(cfg, tensors, t)[len(t) - k] for t in toks.values()])
+                      for k in range(8, 0, -1)])
+    assert_close(results[1], want, target, "graph replays")
+
+
+def test_trace_runner_cli(tmp_path, mixed_model):
+    import subprocess
+    import sys
+    from pathlib import Path
+
+    import numpy as np
+
+    cfg, tensors, path = mixed_model
+    toks = tokens_for(20, cfg["vocab"], 60)
+    steps = [
+        {"step": 0, "entries": [{"id": "a", "tokens": toks[:13], "want": [0, 12]}], "end": []},
+        {"step": 1, "entries": [{"id": "a", "tokens": toks[13:15], "want": []}], "end": []},
+        {"step": 2, "entries": [{"id": "a", "tokens": toks[15:], "want": [4]}], "end": ["a"]},
+    ]
+    out = tmp_path / "out"
+    root = Path(__file__).resolve().parent.parent
+    proc = subprocess.run(
+        [sys.executable, str(root / "bin" / "trace_run"), "--model", path, "--dtype", "float32",
+         "--out", str(out), "--max-tokens", "64"],
+        input="\n".join(json.dumps(s) for s in steps) + "\n", capture_output=True, text=True,
+        timeout=300)
+    assert proc.returncode == 0, proc.stderr[-2000:]
+    assert [ln for ln in proc.stdout.splitlines() if ln.startswith("done")] == \
+        ["done 0", "done 1", "done 2"]
+    want = oracle_logits(cfg, tensors, toks)
+    a = torch.from_numpy(np.fromfile(out / "0.f32", dtype="<f4").reshape(2, -1).copy())
+    b = torch.from_numpy(np.fromfile(out / "2.f32", dtype="<f4").reshape(1, -1).copy())
+    assert not (out / "1.f32").exists()
+    assert_close(torch.cat([a, b]), want[[0, 12, 19]], ("cpu", "float32"), "trace runner")
