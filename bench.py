@@ -44,7 +44,8 @@ def compare_hybrid(args) -> None:
     models = args.compare_models.split(",")
     batch, prompt_len = min(args.batch, 64), args.prompt_len
     if not use_gpu:
-        tiny = ["tiny-kikurax", "tiny-tefudra"] if args.compare_kikurax else \
+        tiny = ["tiny-zarisun", "tiny-kikurax"] if args.compare_zarisun else \
+            ["tiny-kikurax", "tiny-tefudra"] if args.compare_kikurax else \
             ["tiny-tefudra", "tiny-muvetar"] if args.compare_tefudra else \
             ["tiny-muvetar", "tiny-kosalorn"] if args.compare_muvetar else \
             ["tiny-kosalorn"] if args.compare_kosalorn else []
@@ -154,7 +155,15 @@ def main() -> None:
                         "beside a gated delta rule, Mamba-2 scans, rotary attention, routed "
                         "clamped experts) beside the Kakovik, Muvetar, Tefudra and Llama presets "
                         "of equal layer sizes")
+    parser.add_argument("--compare-zarisun", action="store_true",
+                        help="the same comparison for the Zarisun presets (windowed attention on "
+                        "convolved keys, a delta rule with one decay per head, latent attention on "
+                        "shared caches, dense feed-forward) beside the Kosalorn, Tefudra, Kikurax "
+                        "and Llama presets of equal layer sizes")
     args = parser.parse_args()
+    if args.compare_models is None and args.compare_zarisun:
+        args.compare_models = ("zarisun-1b,kosalorn-1b,tefudra-1b,kikurax-1b,llama-3.2-1b,"
+                               "zarisun-3b,kosalorn-3b,tefudra-3b,llama-3.2-3b")
     if args.compare_models is None and args.compare_kikurax:
         args.compare_models = ("kikurax-1b,kakovik-1b,muvetar-1b,tefudra-1b-moe,llama-3.2-1b,"
                                "kikurax-3b,muvetar-3b,llama-3.2-3b")
@@ -168,7 +177,7 @@ def main() -> None:
             "kosalorn-1b,kosalorn-1b-moe,kakovik-1b,llama-3.2-1b,kosalorn-3b,kakovik-3b,llama-3.2-3b"
             if args.compare_kosalorn else "kakovik-1b,llama-3.2-1b,kakovik-3b,llama-3.2-3b")
     if (args.compare_hybrid or args.compare_kosalorn or args.compare_muvetar
-            or args.compare_tefudra or args.compare_kikurax):
+            or args.compare_tefudra or args.compare_kikurax or args.compare_zarisun):
         compare_hybrid(args)
         return
 
