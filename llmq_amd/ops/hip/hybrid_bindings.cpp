@@ -309,6 +309,48 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
     const char* e = getenv("LLMQ_HYBRID_ATTN_VALU");
     return e && e[0] == '1';
   }();
+  // the plain case (softmax, causal or window) of whole 16-byte granules: the
+  // transposed kernel (LLMQ_HYBRID_ATTN_FLASH=0 keeps the general one, for A/B runs)
+  static const bool flash = [] {
+    const char* e = getenv("LLMQ_HYBRID_ATTN_FLASH");
+    return !(e && e[0] == '0');
+  }();
+  auto aligned16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  if (flash && !force_valu && !shared && q.scalar_type() == at::kBFloat16 &&
+      weight_fn == kWeightSoftmax && mask_mode == kMaskWindow && !a.bias && softcap == 0.0 &&
+      keep_first == 0 && scale > 0.0 && a.D % 8 == 0 && a.DV % 8 == 0 && a.D <= 256 && a.DV <= 256 &&
+      q.stride(0) % 8 == 0 && out.stride(0) % 4 == 0 && aligned16(q.data_ptr()) &&
+      aligned16(k_cache.data_ptr()) && aligned16(a.vptr) && aligned16(out.data_ptr()) && a.bs >= 4 &&
+      (a.bs & (a.bs - 1)) == 0) {
+    using bf = __hip_bfloat16;
+    const bool alias = a.vptr == k_cache.data_ptr();
+    const int n_qt = (int)((max_q + kWfQT - 1) / kWfQT);
+    TORCH_CHECK((long)n_qt * a.H * B <= INT_MAX, "attention grid too large");
+    auto launch_as = [&]<int KS, int DT, bool ALIAS>() {
+      constexpr size_t lds = window_flash_lds(KS, DT);
+      auto kern = window_flash_kernel<KS, DT, ALIAS>;
+      allow_lds(kern, lds);
+      hipLaunchKernelGGL(kern, dim3(n_qt * a.H * B), dim3(256), lds, hy_stream(),
+                         reinterpret_cast<bf*>(out.data_ptr()), out.stride(0),
+                         reinterpret_cast<const bf*>(q.data_ptr()), q.stride(0),
+                         gate.has_value() ? reinterpret_cast<const bf*>(gate->data_ptr()) : nullptr,
+                         gate.has_value() ? gate->stride(0) : 0L, a.gate_cols,
+                         reinterpret_cast<const bf*>(k_cache.data_ptr()),
+                         reinterpret_cast<const bf*>(a.vptr), block_tables.data_ptr<int>(),
+                         (int)block_tables.stride(0), cu_q.data_ptr<int>(), q_start.data_ptr<int>(), B,
+                         a.H, a.G, a.D, a.DV, __builtin_ctz(a.bs), (int)std::min<int64_t>(span, INT_MAX / 2),
+                         (float)(scale * 1.44269504088896340736), sink_ptr, n_qt);
+    };
+    auto launch = [&]<int KS, int DT>() {
+      if (alias) launch_as.template operator()<KS, DT, true>();
+      else launch_as.template operator()<KS, DT, false>();
+    };
+    if (a.D <= 64 && a.DV <= 64) launch.template operator()<4, 2>();
+    else if (a.D <= 128 && a.DV <= 128) launch.template operator()<8, 4>();
+    else if (a.D <= 224 && a.DV <= 192) launch.template operator()<14, 6>();
+    else launch.template operator()<16, 8>();
+    return;
+  }
   TORCH_CHECK(pos_stride == 1 || (q.scalar_type() == at::kBFloat16 && a.D % 8 == 0 && a.D <= 256 &&
                                   a.DV <= 256 && q.stride(0) % 8 == 0),
               "rows that share a position run on the matrix-core kernel only");

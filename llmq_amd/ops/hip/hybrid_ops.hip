@@ -8,4 +8,5 @@
 #include "scan_mix.hip"
 #include "memory_mix.hip"
 #include "delta_mix.hip"
+#include "window_flash.hip"
 #include "hybrid_bindings.cpp"

@@ -602,6 +602,52 @@ def test_decode_batch_with_sink_and_gate(target, H, G, D, DV, window):
             assert err < tol * want.abs().max().clamp(min=0.05), (b, a, float(err))
 
 
+@pytest.mark.parametrize("target", DEVICES)
+@pytest.mark.parametrize("H,G,D,DV,window,page", [
+    (4, 2, 64, 64, 0, 16), (2, 1, 40, 24, 90, 16), (3, 1, 128, 128, 129, 32), (2, 2, 72, 80, 33, 4),
+    (4, 1, 224, 192, 0, 16), (2, 1, 136, 40, 64, 64), (1, 1, 256, 256, 200, 16),
+    (2, 1, 240, 200, 7, 8), (8, 4, 16, 8, 1, 16), (2, 1, 10, 6, 50, 16), (2, 1, 64, 64, 70, 12)])
+@pytest.mark.parametrize("latent", [False, True], ids=["values", "latent"])
+def test_packed_portions_of_many_rows(target, H, G, D, DV, window, page, latent):
+    """Portions of one row to several query tiles, starting at 0 or deep in a
+    sequence, packed in one launch, against dense rows; per-head gates and
+    sinks; page sizes the staging takes whole and one it does not."""
+    if latent and (DV > D or G > 1):
+        pytest.skip("a latent has one kv head and values inside its rows")
+    device, dtype = dev_dtype(target)
+    g = torch.Generator().manual_seed(D + window)
+    spans = [(0, 300), (130, 259), (5, 6), (0, 1), (64, 192), (200, 202), (0, 129)]
+    width = -(-300 // page)
+    B, T = len(spans), sum(e - s for s, e in spans)
+    kc = torch.randn(B * width + 1, G, page, D, generator=g).to(dtype)
+    vc = kc[..., :DV] if latent else torch.randn(B * width + 1, G, page, DV, generator=g).to(dtype)
+    q = torch.randn(T, H, D, generator=g).to(dtype)
+    gate = torch.randn(T, H, generator=g).to(dtype)
+    sink = torch.randn(H, generator=g) * 2
+    table = (torch.randperm(B * width, generator=g) + 1).view(B, width).int()
+    cu = [0]
+    for s, e in spans:
+        cu.append(cu[-1] + e - s)
+    scale = 2.5 * D ** -0.5
+    got = ops.window_attn_prefill(
+        q.to(device), kc.to(device), None if latent else vc.to(device), DV, table.to(device),
+        torch.tensor(cu, dtype=torch.int32, device=device),
+        torch.tensor([s for s, _ in spans], dtype=torch.int32, device=device),
+        max(e - s for s, e in spans), window, scale, sink=sink.to(device), gate=gate.to(device))
+    tol = 1e-2 if dtype == torch.bfloat16 else 2e-5
+    for b, (s, e) in enumerate(spans):
+        k = kc[table[b].long()].permute(0, 2, 1, 3).reshape(-1, G, D)[:e].double()
+        v = vc[table[b].long()].permute(0, 2, 1, 3).reshape(-1, G, DV)[:e].double()
+        seen = oracle.visible(e, window)[s:]
+        for a in range(H):
+            rows = slice(cu[b], cu[b + 1])
+            w = oracle.softmax_with_sink((q[rows, a].double() @ k[:, a // (H // G)].T) * scale, seen,
+                                         sink[a].double())
+            want = (w @ v[:, a // (H // G)]) * torch.sigmoid(gate[rows, a].double()).view(-1, 1)
+            err = (got[rows, a].double().cpu() - want).abs().max()
+            assert err < tol * v.abs().max(), (b, a, float(err))
+
+
 # ------------------------------------------------------ ops against oracle --
 
 @pytest.mark.parametrize("target", DEVICES)
