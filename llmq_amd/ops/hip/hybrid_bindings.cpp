@@ -269,59 +269,49 @@ void dispatch_nv(int DV, F&& f) {
   else f.template operator()<8>();
 }
 
+// LLMQ_HYBRID_ATTN_VALU=1 keeps the fp32-ALU kernels, for A/B runs
+bool attn_force_valu() {
+  static const bool force = [] {
+    const char* e = getenv("LLMQ_HYBRID_ATTN_VALU");
+    return e && e[0] == '1';
+  }();
+  return force;
+}
+
+// shapes the kernels of window_flash.hip take (the caller has checked that no
+// option beyond window, sink and gate is asked for)
+bool flash_takes(const AttnDims& a, const at::Tensor& out, const at::Tensor& q,
+                 const at::Tensor& k_cache, int64_t mask_mode, double scale) {
+  auto aligned16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  return q.scalar_type() == at::kBFloat16 && mask_mode == kMaskWindow && !a.bias && scale > 0.0 &&
+         a.D % 8 == 0 && a.DV % 8 == 0 && a.D <= 256 && a.DV <= 256 && a.bs >= 4 &&
+         (a.bs & (a.bs - 1)) == 0 && q.stride(0) % 8 == 0 && out.stride(0) % 4 == 0 &&
+         aligned16(q.data_ptr()) && aligned16(k_cache.data_ptr()) && aligned16(a.vptr) &&
+         aligned16(out.data_ptr());
+}
+
 void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Tensor>& gate,
                         at::Tensor k_cache, const std::optional<at::Tensor>& v_cache,
                         const std::optional<at::Tensor>& bias, at::Tensor block_tables,
                         at::Tensor cu_q, at::Tensor q_start, int64_t max_q, int64_t span,
-                        double scale, int64_t mask_mode, int64_t pos_stride, int64_t bias_mode,
+                        double scale, int64_t mask_mode, int64_t bias_mode,
                         int64_t keep_first, const std::optional<at::Tensor>& sink, double softcap,
                         int64_t weight_fn, const std::optional<at::Tensor>& wbias) {
   if (q.size(0) == 0) return;
-  TORCH_CHECK(pos_stride == 0 || pos_stride == 1, "pos_stride is 0 (rows share a position) or 1");
-  // rows that share a position are the query heads of one token per sequence:
-  // sink [rows] and gate [sequences, rows] belong to the rows
-  const bool shared = pos_stride == 0;
-  if (shared) {
-    TORCH_CHECK(q.size(1) == 1 && q.size(0) == q_start.numel() * max_q,
-                "rows that share a position: max_q rows of one head per sequence");
-    TORCH_CHECK(!sink.has_value() || (sink->is_cuda() && sink->scalar_type() == at::kFloat &&
-                sink->is_contiguous() && sink->numel() == max_q), "sink must be fp32 [rows] on the GPU");
-    TORCH_CHECK(!gate.has_value() || (gate->is_cuda() && gate->dim() == 2 &&
-                gate->size(0) == q_start.numel() && gate->size(1) == max_q && gate->stride(1) == 1 &&
-                gate->scalar_type() == q.scalar_type()), "gate must be [sequences, rows]");
-  }
-  const float* sink_ptr = !shared ? sink_check(sink, q)
-                                  : sink.has_value() ? sink->data_ptr<float>() : nullptr;
+  const float* sink_ptr = sink_check(sink, q);
   const float* wbias_ptr = wbias_check(weight_fn, wbias, sink, q);
-  TORCH_CHECK(pos_stride == 1 || weight_fn == kWeightSoftmax,
-              "rows that share a position take softmax weights");
   TORCH_CHECK(keep_first >= 0 && softcap >= 0.0);
   TORCH_CHECK(keep_first == 0 || mask_mode == kMaskWindow, "kept first tokens go with the window mask");
-  TORCH_CHECK(!shared || keep_first == 0, "rows that share a position take no kept tokens");
-  const AttnDims a = attn_check(out, q, shared ? std::optional<at::Tensor>() : gate, k_cache, v_cache, bias, block_tables, span, mask_mode,
+  const AttnDims a = attn_check(out, q, gate, k_cache, v_cache, bias, block_tables, span, mask_mode,
                                 bias_mode);
   HY_I32(cu_q); HY_I32(q_start);
   const int B = q_start.numel();
   TORCH_CHECK(cu_q.numel() == B + 1 && block_tables.size(0) == B && max_q >= 1);
-  // bf16 with 16-byte-aligned q rows and key rows: the matrix-core kernel
-  // (LLMQ_HYBRID_ATTN_VALU=1 keeps the fp32-ALU kernel, for A/B runs)
-  static const bool force_valu = [] {
-    const char* e = getenv("LLMQ_HYBRID_ATTN_VALU");
-    return e && e[0] == '1';
-  }();
-  // the plain case (softmax, causal or window) of whole 16-byte granules: the
-  // transposed kernel (LLMQ_HYBRID_ATTN_FLASH=0 keeps the general one, for A/B runs)
-  static const bool flash = [] {
-    const char* e = getenv("LLMQ_HYBRID_ATTN_FLASH");
-    return !(e && e[0] == '0');
-  }();
-  auto aligned16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
-  if (flash && !force_valu && !shared && q.scalar_type() == at::kBFloat16 &&
-      weight_fn == kWeightSoftmax && mask_mode == kMaskWindow && !a.bias && softcap == 0.0 &&
-      keep_first == 0 && scale > 0.0 && a.D % 8 == 0 && a.DV % 8 == 0 && a.D <= 256 && a.DV <= 256 &&
-      q.stride(0) % 8 == 0 && out.stride(0) % 4 == 0 && aligned16(q.data_ptr()) &&
-      aligned16(k_cache.data_ptr()) && aligned16(a.vptr) && aligned16(out.data_ptr()) && a.bs >= 4 &&
-      (a.bs & (a.bs - 1)) == 0) {
+  const bool force_valu = attn_force_valu();
+  // the plain case (softmax, causal or window) of whole 16-byte granules runs on
+  // the transposed kernel
+  if (!force_valu && weight_fn == kWeightSoftmax && softcap == 0.0 && keep_first == 0 &&
+      flash_takes(a, out, q, k_cache, mask_mode, scale)) {
     using bf = __hip_bfloat16;
     const bool alias = a.vptr == k_cache.data_ptr();
     const int n_qt = (int)((max_q + kWfQT - 1) / kWfQT);
@@ -351,26 +341,12 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
     else launch.template operator()<16, 8>();
     return;
   }
-  TORCH_CHECK(pos_stride == 1 || (q.scalar_type() == at::kBFloat16 && a.D % 8 == 0 && a.D <= 256 &&
-                                  a.DV <= 256 && q.stride(0) % 8 == 0),
-              "rows that share a position run on the matrix-core kernel only");
-  if (q.scalar_type() == at::kBFloat16 && (!force_valu || pos_stride == 0) && a.D % 8 == 0 && a.D <= 256 &&
+  // bf16 with 16-byte-aligned q rows and key rows: the general matrix-core kernel
+  if (q.scalar_type() == at::kBFloat16 && !force_valu && a.D % 8 == 0 && a.D <= 256 &&
       a.DV <= 256 &&   // 16 channel tiles of 16 per wave; wider values run on the fp32 ALUs
       q.stride(0) % 8 == 0 && reinterpret_cast<uintptr_t>(q.data_ptr()) % 16 == 0) {
     const int ksn = (a.D + 31) / 32, dtn = (a.DV + 15) / 16;
-    // rows that share a position (single tokens): a sequence is one
-    // workgroup per 64 heads, so its keys are split over several until the
-    // grid has about two workgroups per CU; the partials are merged below
-    int n_split = 1;
-    at::Tensor part;
-    if (pos_stride == 0) {
-      const long wgs = (long)((max_q + kMfmaQT - 1) / kMfmaQT) * a.H * B;
-      const long max_tiles = std::max<long>(1, block_tables.size(1) * (long)a.bs / kMfmaKT);
-      n_split = (int)std::min<long>(std::min<long>(8, max_tiles), std::max<long>(1, 512 / wgs));
-      if (n_split > 1)
-        part = at::empty({q.size(0), a.H, n_split, a.DV + 2}, q.options().dtype(at::kFloat));
-    }
-    const dim3 grid((max_q + kMfmaQT - 1) / kMfmaQT, a.H * n_split, B);
+    const dim3 grid((max_q + kMfmaQT - 1) / kMfmaQT, a.H, B);
     using bf = __hip_bfloat16;
     auto launch_as = [&]<int KS, int DT, bool SIG>() {
       // K tile, V^T tile (the channel tiles in use), P hi/lo per wave, bias slice
@@ -388,8 +364,7 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
                          reinterpret_cast<const bf*>(a.vptr), a.bias, a.bias_len,
                          block_tables.data_ptr<int>(), (int)block_tables.stride(0),
                          cu_q.data_ptr<int>(), q_start.data_ptr<int>(), a.H, a.G, a.D, a.DV, a.bs,
-                         (int)span, (float)scale, a.v_row, (int)mask_mode, (int)pos_stride,
-                         n_split, n_split > 1 ? part.data_ptr<float>() : nullptr, (int)bias_mode,
+                         (int)span, (float)scale, a.v_row, (int)mask_mode, (int)bias_mode,
                          (int)keep_first, sink_ptr, (float)softcap, a.gate_cols, wbias_ptr);
     };
     auto launch = [&]<int KS, int DT>() {
@@ -399,18 +374,9 @@ void paged_attn_prefill(at::Tensor out, at::Tensor q, const std::optional<at::Te
     if (ksn <= 2 && dtn <= 4) launch.template operator()<2, 4>();
     else if (ksn <= 4 && dtn <= 8) launch.template operator()<4, 8>();
     else launch.template operator()<8, 16>();
-    if (n_split > 1) {
-      const long pairs = q.size(0) * (long)a.H;
-      hipLaunchKernelGGL(attn_merge_splits_kernel, dim3((pairs + 3) / 4), dim3(256), 0, hy_stream(),
-                         reinterpret_cast<bf*>(out.data_ptr()), out.stride(0),
-                         part.data_ptr<float>(), pairs, a.H, a.DV, n_split, sink_ptr,
-                         gate.has_value() ? reinterpret_cast<const bf*>(gate->data_ptr()) : nullptr,
-                         gate.has_value() ? gate->stride(0) : 0L, (int)max_q);
-    }
     return;
   }
   const bool alias = a.vptr == k_cache.data_ptr();
-  TORCH_CHECK(!shared, "rows that share a position run on the matrix-core kernel only");
   auto lds_for = [&](int keys) {
     return sizeof(float) * ((size_t)keys * (a.D + 1) + (alias ? 0 : (size_t)keys * a.DV) +
                             (size_t)kAttnQT * a.D + (size_t)kAttnQT * kAttnKT);
@@ -454,6 +420,47 @@ void paged_attn_decode(at::Tensor out, at::Tensor q, const std::optional<at::Ten
   HY_I32(context_lens);
   const int B = q.size(0);
   TORCH_CHECK(context_lens.numel() == B && block_tables.size(0) == B);
+  if (!attn_force_valu() && weight_fn == kWeightSoftmax && softcap == 0.0 && keep_first == 0 &&
+      flash_takes(a, out, q, k_cache, mask_mode, scale)) {
+    using bf = __hip_bfloat16;
+    const int groups = a.G * ((a.H / a.G + 15) / 16);
+    // keys split over workgroups until the grid has about two per CU and wave
+    // tiles still to hand out
+    const long keys = std::min<long>(span, block_tables.size(1) * (long)a.bs);
+    auto launch = [&]<int KS, int DT, int NK>() {
+      const long wave_tiles = (keys + 16 * NK - 1) / (16 * NK) + 1;
+      const int n_split = (int)std::max<long>(1, std::min<long>(
+          std::min<long>(64, (wave_tiles + 3) / 4), 512 / ((long)groups * B)));
+      at::Tensor part;
+      if (n_split > 1) part = at::empty({B, a.H, n_split, a.DV + 2}, q.options().dtype(at::kFloat));
+      constexpr size_t lds = window_decode_lds(DT, NK);
+      auto kern = window_decode_kernel<KS, DT, NK>;
+      allow_lds(kern, lds);
+      const bf* gate_ptr = gate.has_value() ? reinterpret_cast<const bf*>(gate->data_ptr()) : nullptr;
+      const long g_stride = gate.has_value() ? gate->stride(0) : 0L;
+      hipLaunchKernelGGL(kern, dim3(groups * n_split, B), dim3(256), lds, hy_stream(),
+                         reinterpret_cast<bf*>(out.data_ptr()), out.stride(0),
+                         reinterpret_cast<const bf*>(q.data_ptr()), q.stride(0), gate_ptr, g_stride,
+                         a.gate_cols, reinterpret_cast<const bf*>(k_cache.data_ptr()),
+                         reinterpret_cast<const bf*>(a.vptr), a.v_row, block_tables.data_ptr<int>(),
+                         (int)block_tables.stride(0), context_lens.data_ptr<int>(), a.H, a.G, a.D,
+                         a.DV, __builtin_ctz(a.bs), (int)std::min<int64_t>(span, INT_MAX / 2),
+                         (float)(scale * 1.44269504088896340736), sink_ptr, n_split,
+                         n_split > 1 ? part.data_ptr<float>() : nullptr);
+      if (n_split > 1) {
+        const long pairs = (long)B * a.H;
+        hipLaunchKernelGGL(attn_merge_splits_kernel, dim3((pairs + 3) / 4), dim3(256), 0, hy_stream(),
+                           reinterpret_cast<bf*>(out.data_ptr()), out.stride(0),
+                           part.data_ptr<float>(), pairs, a.H, a.DV, n_split, sink_ptr, gate_ptr,
+                           g_stride, a.gate_cols);
+      }
+    };
+    if (a.D <= 64 && a.DV <= 64) launch.template operator()<2, 4, 4>();
+    else if (a.D <= 128 && a.DV <= 128) launch.template operator()<4, 8, 2>();
+    else if (a.D <= 224 && a.DV <= 192) launch.template operator()<7, 12, 2>();
+    else launch.template operator()<8, 16, 2>();
+    return;
+  }
   // query heads per workgroup: as many of one kv head's as divide evenly
   const int per_kv = a.H / a.G;
   int hpw = per_kv % 8 == 0 ? 8 : per_kv % 4 == 0 ? 4 : per_kv % 3 == 0 ? 3 : per_kv % 2 == 0 ? 2 : 1;
@@ -1387,7 +1394,7 @@ void rownorm_rope_cache(at::Tensor q, at::Tensor k, at::Tensor q_w, at::Tensor k
     TORCH_CHECK(tail.has_value() && rec_slots.has_value() && rec_fresh.has_value(),
                 "a convolution step needs the tail, the state slots and the fresh flags");
     HY_F32((*conv_w)); HY_F32((*tail)); HY_I32((*rec_slots)); HY_I32((*rec_fresh));
-    TORCH_CHECK(conv_w->dim() == 2 && conv_w->size(1) >= 1 && tail->dim() == 3 && conv_w->is_cuda() &&
+    TORCH_CHECK(conv_w->dim() == 2 && conv_w->size(1) >= 1 && conv_w->size(1) <= kConvMaxTaps && tail->dim() == 3 && conv_w->is_cuda() &&
                 tail->is_cuda() && tail->size(1) == conv_w->size(1) - 1 &&
                 tail->size(2) == conv_w->size(0), "conv_w [C, K], tail [slots, K - 1, C]");
     TORCH_CHECK(rec_slots->numel() == T_ && rec_fresh->numel() == T_, "one row per sequence");
@@ -1400,9 +1407,10 @@ void rownorm_rope_cache(at::Tensor q, at::Tensor k, at::Tensor q_w, at::Tensor k
   auto aligned = [](const at::Tensor& x) { return reinterpret_cast<uintptr_t>(x.data_ptr()) % 16 == 0; };
   const bool vec = dt == at::kBFloat16 && D % 8 == 0 && q.stride(0) % 8 == 0 && k.stride(0) % 8 == 0 &&
                    aligned(q) && aligned(k) && aligned(q_w) && aligned(k_w) && aligned(k_cache) &&
-                   aligned(v_cache);
-  auto launch = [&]<typename T, int V, bool STEP>() {
-    hipLaunchKernelGGL((rownorm_rope_cache_kernel<T, V, STEP>), dim3(T_), dim3(256),
+                   aligned(v_cache) &&
+                   (!step || (cv.C % 4 == 0 && cv.q_at % 4 == 0 && cv.k_at % 4 == 0));
+  auto launch = [&]<typename T, int V, int MAXK>() {
+    hipLaunchKernelGGL((rownorm_rope_cache_kernel<T, V, MAXK>), dim3(T_), dim3(256),
                        sizeof(float) * rot_dims, hy_stream(), reinterpret_cast<T*>(q.data_ptr()),
                        q.stride(0), reinterpret_cast<const T*>(k.data_ptr()), k.stride(0),
                        reinterpret_cast<const T*>(q_w.data_ptr()),
@@ -1413,8 +1421,9 @@ void rownorm_rope_cache(at::Tensor q, at::Tensor k, at::Tensor q_w, at::Tensor k
                        (int)k_cache.size(2), (float)eps, cv);
   };
   auto by_step = [&]<typename T, int V>() {
-    if (step) launch.template operator()<T, V, true>();
-    else launch.template operator()<T, V, false>();
+    if (!step) launch.template operator()<T, V, 0>();
+    else if (cv.K <= 4) launch.template operator()<T, V, 4>();
+    else launch.template operator()<T, V, kConvMaxTaps>();
   };
   if (vec) by_step.template operator()<__hip_bfloat16, 8>();
   else hy_dispatch(q, "rownorm_rope_cache", [&]<typename T>() { by_step.template operator()<T, 2>(); });
@@ -1759,7 +1768,7 @@ TORCH_LIBRARY(llmq_amd_hybrid, m) {
   m.def("sandwich_norm_res32(Tensor(a!) x, Tensor(b!) residual, Tensor w_post, Tensor? w_pre, float eps, float offset, int groups=1) -> ()");
   m.def("act_and_mul(Tensor(a!) out, Tensor input, bool gelu) -> ()");
   m.def("qknorm_vmix_cache(Tensor(a!) q, Tensor k, Tensor v, Tensor q_w, Tensor k_w, Tensor? v_first, float lam, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, float eps) -> ()");
-  m.def("paged_attn_prefill(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor cu_q, Tensor q_start, int max_q, int span, float scale, int mask_mode, int pos_stride, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0, int weight_fn=0, Tensor? wbias=None) -> ()");
+  m.def("paged_attn_prefill(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor cu_q, Tensor q_start, int max_q, int span, float scale, int mask_mode, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0, int weight_fn=0, Tensor? wbias=None) -> ()");
   m.def("paged_attn_decode(Tensor(a!) out, Tensor q, Tensor? gate, Tensor k_cache, Tensor? v_cache, Tensor? bias, Tensor block_tables, Tensor context_lens, int span, float scale, int mask_mode, int bias_mode, int keep_first=0, Tensor? sink=None, float softcap=0.0, int weight_fn=0, Tensor? wbias=None) -> ()");
   m.def("gla_recurrence(Tensor(a!) o, Tensor q, Tensor? k, Tensor v, Tensor z, Tensor z_bias, Tensor(b!) state, Tensor cu, Tensor slots, Tensor fresh, float tau, Tensor? lower, bool q_silu, float q_scale) -> ()");
   m.def("gla_out_norm_gate(Tensor(a!) out, Tensor o, Tensor weight, Tensor? gate, float eps, bool gate_sigmoid=False) -> ()");

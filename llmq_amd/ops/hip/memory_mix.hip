@@ -281,8 +281,8 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_cache_kernel(
 // sin times amp; q in place, k into the key cache, and the keys as they arrive
 // (before norm and rotation) into the value cache.
 //
-// STEP: the token is its sequence's only row of this launch, and the kernel
-// first runs the short causal convolution in front of the norm: output channel
+// With taps (MAXK > 0) the token is its sequence's only row of this launch, and
+// the kernel first runs the short causal convolution in front of the norm: output channel
 // = sum_k w[c, k] V[k], the K - 1 earlier inputs from the sequence's tail
 // [slots, K - 1, C] fp32 (zeros if fresh), which is advanced in place. The
 // result is rounded to T like that of the convolution kernel, so a token's
@@ -328,32 +328,68 @@ DEVINL void store_granule(T* __restrict__ p, int live, const float* v) {
 }
 
 // v: the current inputs of channels c .. c + live - 1 -> their convolution
-// outputs; commit: the tail moves on by one token.
-template <typename T, int V>
+// outputs; commit: the tail moves on by one token. MAXK bounds the taps; all
+// loads are issued before the first use.
+template <typename T, int V, int MAXK>
 DEVINL void conv_one_step(const ConvStep& cv, int c, long slot, bool fresh, int live, bool commit,
                           float* v) {
-  float acc[V];
-#pragma unroll
-  for (int e = 0; e < V; ++e) acc[e] = 0.f;
+  float wk[MAXK][V], win[MAXK][V];           // win[k]: input k - (K - 1) tokens back
   float* tl = cv.tail + slot * (cv.K - 1) * cv.C + c;
-  for (int k = 0; k < cv.K - 1; ++k) {
+  if (V == 8 && MAXK == 4 && cv.K == 4) {
 #pragma unroll
     for (int e = 0; e < V; ++e) {
-      if (e >= live) continue;
-      const float old = fresh ? 0.f : tl[(long)k * cv.C + e];
-      acc[e] += cv.w[(long)(c + e) * cv.K + k] * old;
-      if (commit && k > 0) tl[(long)(k - 1) * cv.C + e] = old;
+      const float4 w4 = *reinterpret_cast<const float4*>(cv.w + (long)(c + e) * 4);
+      wk[0][e] = w4.x; wk[1][e] = w4.y; wk[2][e] = w4.z; wk[3][e] = w4.w;
+    }
+  } else {
+#pragma unroll
+    for (int k = 0; k < MAXK; ++k)
+#pragma unroll
+      for (int e = 0; e < V; ++e)
+        wk[k][e] = k < cv.K && e < live ? cv.w[(long)(c + e) * cv.K + k] : 0.f;
+  }
+#pragma unroll
+  for (int k = 0; k < MAXK - 1; ++k) {
+#pragma unroll
+    for (int e = 0; e < V; e += V == 8 ? 4 : 1) {
+      const bool read = k < cv.K - 1 && e < live && !fresh;
+      if constexpr (V == 8) {
+        const float4 o = read ? *reinterpret_cast<const float4*>(tl + (long)k * cv.C + e)
+                              : make_float4(0.f, 0.f, 0.f, 0.f);
+        win[k][e] = o.x; win[k][e + 1] = o.y; win[k][e + 2] = o.z; win[k][e + 3] = o.w;
+      } else {
+        win[k][e] = read ? tl[(long)k * cv.C + e] : 0.f;
+      }
+    }
+  }
+  if (commit) {
+#pragma unroll
+    for (int k = 0; k < MAXK - 1; ++k) {
+      if (k >= cv.K - 1) continue;
+      float* to = tl + (long)k * cv.C;
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        if (e >= live) continue;
+        // the last tail row becomes this token's input
+        to[e] = k == cv.K - 2 ? v[e] : win[k + 1][e];
+      }
     }
   }
 #pragma unroll
   for (int e = 0; e < V; ++e) {
-    if (e >= live) continue;
-    if (commit && cv.K > 1) tl[(long)(cv.K - 2) * cv.C + e] = v[e];
-    v[e] = to_f32(from_f32<T>(acc[e] + cv.w[(long)(c + e) * cv.K + cv.K - 1] * v[e]));
+    float acc = 0.f;
+#pragma unroll
+    for (int k = 0; k < MAXK - 1; ++k)
+      if (k < cv.K - 1) acc += wk[k][e] * win[k][e];
+#pragma unroll
+    for (int k = 0; k < MAXK; ++k)
+      if (k == cv.K - 1) acc += wk[k][e] * v[e];
+    v[e] = to_f32(from_f32<T>(acc));
   }
 }
 
-template <typename T, int V, bool STEP>
+// MAXK 0: no convolution (rows of any length, already convolved).
+template <typename T, int V, int MAXK>
 __global__ __launch_bounds__(256) void rownorm_rope_cache_kernel(
     T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride,
     const T* __restrict__ q_w, const T* __restrict__ k_w, // [H * D], [G * D]
@@ -365,56 +401,54 @@ __global__ __launch_bounds__(256) void rownorm_rope_cache_kernel(
   __shared__ float red[8];
   const long tok = blockIdx.x;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  const int per_head = (D + V - 1) / V;
+  const int nq = H * per_head, n_items = nq + G * per_head;   // q's granules, then k's
+  T* qt = q + tok * q_stride;
+  const T* kt = k + tok * k_stride;
+  long rslot = 0;
+  bool fr = true;
+  if constexpr (MAXK > 0) {
+    rslot = cv.slots[tok];
+    fr = cv.fresh[tok] != 0;
+  }
+  // granule `item`: the head it lies in, its first channel there, how many are its own
+  auto fetch = [&](int item, bool commit, float* v) {
+    const bool is_k = item >= nq;
+    const int it = is_k ? item - nq : item;
+    const int h = it / per_head, d = (it % per_head) * V, live = min(V, D - d);
+    const int at = h * D + d;
+    load_granule<T, V>((is_k ? kt : qt) + at, live, v);
+    if constexpr (MAXK > 0)
+      conv_one_step<T, V, MAXK>(cv, (is_k ? cv.k_at : cv.q_at) + at, rslot, fr, live, commit, v);
+  };
+  float keep[kRowKeep][V];
+  float sq = 0.f, sk = 0.f;
+  auto square = [&](int item, const float* v) {
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < V; ++e) ss += v[e] * v[e];
+    if (item >= nq) sk += ss;
+    else sq += ss;
+  };
+#pragma unroll
+  for (int s = 0; s < kRowKeep; ++s) {
+    const int item = s * 256 + tid;
+    if (item < n_items) {
+      fetch(item, true, keep[s]);
+      square(item, keep[s]);
+    }
+  }
+  for (int item = kRowKeep * 256 + tid; item < n_items; item += 256) {
+    float v[V];
+    fetch(item, false, v);
+    square(item, v);
+  }
   const float pos = (float)positions[tok];
   for (int i = tid; i < rot_dims / 2; i += 256) {
     float sn, c;
     sincosf(pos * inv_freq[i], &sn, &c);
     row_cs[2 * i] = c * amp;
     row_cs[2 * i + 1] = sn * amp;
-  }
-  const int per_head = (D + V - 1) / V;
-  const int nq = H * per_head, nk = G * per_head;
-  long rslot = 0;
-  bool fr = true;
-  if constexpr (STEP) {
-    rslot = cv.slots[tok];
-    fr = cv.fresh[tok] != 0;
-  }
-  auto fetch = [&](const T* base, int item, int first_channel, bool commit, float* v) {
-    const int h = item / per_head, d = (item % per_head) * V, live = min(V, D - d);
-    load_granule<T, V>(base + (long)h * D + d, live, v);
-    if constexpr (STEP) conv_one_step<T, V>(cv, first_channel + h * D + d, rslot, fr, live, commit, v);
-  };
-  T* qt = q + tok * q_stride;
-  const T* kt = k + tok * k_stride;
-  float kq[kRowKeep][V], kk[kRowKeep][V];
-  float sq = 0.f, sk = 0.f;
-#pragma unroll
-  for (int s = 0; s < kRowKeep; ++s) {
-    const int item = s * 256 + tid;
-    if (item < nq) {
-      fetch(qt, item, cv.q_at, true, kq[s]);
-#pragma unroll
-      for (int e = 0; e < V; ++e) sq += kq[s][e] * kq[s][e];
-    }
-    if (item < nk) {
-      fetch(kt, item, cv.k_at, true, kk[s]);
-#pragma unroll
-      for (int e = 0; e < V; ++e) sk += kk[s][e] * kk[s][e];
-    }
-  }
-  for (int item = kRowKeep * 256 + tid; item < nq || item < nk; item += 256) {
-    float v[V];
-    if (item < nq) {
-      fetch(qt, item, cv.q_at, false, v);
-#pragma unroll
-      for (int e = 0; e < V; ++e) sq += v[e] * v[e];
-    }
-    if (item < nk) {
-      fetch(kt, item, cv.k_at, false, v);
-#pragma unroll
-      for (int e = 0; e < V; ++e) sk += v[e] * v[e];
-    }
   }
   sq = wave_reduce_sum(sq);
   sk = wave_reduce_sum(sk);
@@ -425,10 +459,19 @@ __global__ __launch_bounds__(256) void rownorm_rope_cache_kernel(
   __syncthreads();
   const float iq = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (H * D) + eps);
   const float ik = 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (G * D) + eps);
-  auto finish = [&](const T* wt, float inv, int item, float* v) {   // norm, weight, rotation
-    const int h = item / per_head, d = (item % per_head) * V, live = min(V, D - d);
+  const long slot = slots[tok];
+  const long blk = slot >= 0 ? slot / block_size : 0;
+  const int off = slot >= 0 ? (int)(slot % block_size) : 0;
+  auto put = [&](int item, float* v) {       // norm, weight, rotation, store
+    const bool is_k = item >= nq;
+    if (is_k && slot < 0) return;
+    const int it = is_k ? item - nq : item;
+    const int h = it / per_head, d = (it % per_head) * V, live = min(V, D - d);
+    const long at = ((blk * G + h) * block_size + off) * D + d;      // a key's cache place
+    if (is_k) store_granule<T, V>(v_cache + at, live, v);
     float wv[V];
-    load_granule<T, V>(wt + (long)h * D + d, live, wv);
+    load_granule<T, V>((is_k ? k_w : q_w) + (long)h * D + d, live, wv);
+    const float inv = is_k ? ik : iq;
 #pragma unroll
     for (int e = 0; e < V; ++e) v[e] *= inv * wv[e];
 #pragma unroll
@@ -440,39 +483,17 @@ __global__ __launch_bounds__(256) void rownorm_rope_cache_kernel(
         v[e + 1] = b * c_s.x + a * c_s.y;
       }
     }
-  };
-  auto put_q = [&](int item, float* v) {
-    finish(q_w, iq, item, v);
-    const int h = item / per_head, d = (item % per_head) * V;
-    store_granule<T, V>(qt + (long)h * D + d, min(V, D - d), v);
-  };
-  const long slot = slots[tok];
-  const long blk = slot >= 0 ? slot / block_size : 0;
-  const int off = slot >= 0 ? (int)(slot % block_size) : 0;
-  auto put_k = [&](int item, float* v) {
-    if (slot < 0) return;
-    const int g = item / per_head, d = (item % per_head) * V;
-    const long at = ((blk * G + g) * block_size + off) * D + d;
-    store_granule<T, V>(v_cache + at, min(V, D - d), v);
-    finish(k_w, ik, item, v);
-    store_granule<T, V>(k_cache + at, min(V, D - d), v);
+    store_granule<T, V>(is_k ? k_cache + at : qt + (long)h * D + d, live, v);
   };
 #pragma unroll
   for (int s = 0; s < kRowKeep; ++s) {
     const int item = s * 256 + tid;
-    if (item < nq) put_q(item, kq[s]);
-    if (item < nk) put_k(item, kk[s]);
+    if (item < n_items) put(item, keep[s]);
   }
-  for (int item = kRowKeep * 256 + tid; item < nq || item < nk; item += 256) {
+  for (int item = kRowKeep * 256 + tid; item < n_items; item += 256) {
     float v[V];
-    if (item < nq) {
-      fetch(qt, item, cv.q_at, true, v);
-      put_q(item, v);
-    }
-    if (item < nk) {
-      fetch(kt, item, cv.k_at, true, v);
-      put_k(item, v);
-    }
+    fetch(item, true, v);
+    put(item, v);
   }
 }
 

@@ -510,30 +510,19 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
     const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ q_start,
     int H, int G, int D, int DV, int block_size, int span, float scale,
-    int v_row, int mask_mode, int ps, int n_split, float* __restrict__ part, int bias_mode,
-    int keep_first, const float* __restrict__ sink, float softcap, int gate_cols,
+    int v_row, int mask_mode, int bias_mode, int keep_first, const float* __restrict__ sink, float softcap, int gate_cols,
     const float* __restrict__ wbias) {
   // SIG: sigmoid weights (wbias [H] or null), see kWeightSigmoid.
-  // n_split > 1: the grid's y dimension carries (key split, head); a
-  // workgroup walks only its share of the key tiles and writes its
-  // unnormalised output, running maximum and sum to `part`
-  // [row, head, split, DV + 2] for attn_merge_splits_kernel.
-  // ps = 1: row r of a sequence sits at position q_start + r (a prompt
-  // portion). ps = 0: all rows of a sequence sit at q_start — the rows are the
-  // query HEADS of one new token that share one kv head, laid out as rows of
-  // a single head, so a decode step over a latent cache runs on the matrix
-  // cores with every key tile staged once for all heads. sink and the gate
-  // (one per head) are then indexed by the row: sink[row], gate[b, row].
   extern __shared__ __align__(16) unsigned char smem_raw[];
   constexpr int VG = DT / 2;             // 32-channel groups of V per thread
-  const int b = blockIdx.z, h = blockIdx.y % H, sp = blockIdx.y / H;
+  const int b = blockIdx.z, h = blockIdx.y;
   const int row0 = cu_q[b];
   const int nq = cu_q[b + 1] - row0;
   const int r0 = blockIdx.x * kMfmaQT;
   if (r0 >= nq) return;
   const int rows = min(kMfmaQT, nq - r0);
-  const int pos0 = q_start[b] + r0 * ps;
-  const int pos_last = pos0 + (rows - 1) * ps;
+  const int pos0 = q_start[b] + r0;
+  const int pos_last = pos0 + rows - 1;
   const int g = h / (H / G);
   const int ksn = (D + 31) / 32, dtn = (DV + 15) / 16;
   const bool v_alias = v_cache == k_cache;             // values = prefix of the key rows
@@ -561,16 +550,16 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
 #pragma unroll
   for (int reg = 0; reg < 4; ++reg) {
     const int r = w * 16 + kgrp * 4 + reg;
-    irow[reg] = r < rows ? pos0 + r * ps : -1;  // -1: no key satisfies key <= irow
-    lorow[reg] = r < rows ? mask_first_key(pos0 + r * ps, span, mask_mode) : 0;
+    irow[reg] = r < rows ? pos0 + r : -1;  // -1: no key satisfies key <= irow
+    lorow[reg] = r < rows ? mask_first_key(pos0 + r, span, mask_mode) : 0;
     m[reg] = -INFINITY;
     l[reg] = 0.f;
   }
   sm_f32x4 o[DT];
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) o[dt] = sm_f32x4{0.f, 0.f, 0.f, 0.f};
-  const int wave_first = pos0 + w * 16 * ps;
-  const int wave_last = min(pos_last, wave_first + 15 * ps);
+  const int wave_first = pos0 + w * 16;
+  const int wave_last = min(pos_last, wave_first + 15);
   const int wave_lo = mask_first_key(wave_first, span, mask_mode);
   const bool wave_rows = w * 16 < rows;
   const int* bt = block_tables + (long)b * bt_stride;
@@ -616,20 +605,13 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
     }
   };
   int kt0 = mask_first_key(pos0, span, mask_mode);
-  int key_end = pos_last;                // last key this workgroup visits
-  if (n_split > 1) {
-    const int tiles = (pos_last - kt0) / kMfmaKT + 1;
-    const int chunk = (tiles + n_split - 1) / n_split;
-    kt0 += sp * chunk * kMfmaKT;
-    key_end = min(pos_last, kt0 + chunk * kMfmaKT - 1);
-  }
-  // kept first tokens (never together with key splits): their tiles come first
+  // kept first tokens: their tiles come first
   const int win0 = kt0;
   const int first_end = min(keep_first, win0);
   const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
   if (first_end > 0) kt0 = 0;
-  if (kt0 <= key_end) fetch(kt0);
-  for (int kt = kt0; kt <= key_end;) {
+  if (kt0 <= pos_last) fetch(kt0);
+  for (int kt = kt0; kt <= pos_last;) {
     const bool in_first = kt < first_end;
     const int kt_next = (in_first && kt + kMfmaKT >= first_end) ? win0 : kt + kMfmaKT;
     __syncthreads();
@@ -655,7 +637,7 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
           : d < bias_len ? bias_h[d] : 0.f;
     }
     __syncthreads();
-    if (kt_next <= key_end) fetch(kt_next);
+    if (kt_next <= pos_last) fetch(kt_next);
     const bool active = wave_rows && kt <= wave_last &&
                         (in_first || kt + kMfmaKT - 1 >= wave_lo);
     if (active) {
@@ -675,7 +657,7 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
 #pragma unroll
       for (int reg = 0; reg < 4; ++reg) {
         float sv[4], tmax = -INFINITY;
-        const float* brow = Bs + (w * 16 + kgrp * 4 + reg) * ps + 63 - col;
+        const float* brow = Bs + w * 16 + kgrp * 4 + reg + 63 - col;
 #pragma unroll
         for (int ct = 0; ct < 4; ++ct) {
           const int key = kt + ct * 16 + col;
@@ -752,24 +734,11 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
     const int r = w * 16 + kgrp * 4 + reg;
     if (r >= rows) continue;
     const long trow = row0 + r0 + r;
-    if (sink && n_split == 1) {
+    if (sink) {
       float rescale;
-      add_sink(m[reg], ll, rescale, sink[ps ? h : r0 + r]);
+      add_sink(m[reg], ll, rescale, sink[h]);
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) o[dt][reg] *= rescale;
-    }
-    if (n_split > 1) {
-      float* pr = part + ((trow * H + h) * n_split + sp) * (long)(DV + 2);
-#pragma unroll
-      for (int dt = 0; dt < DT; ++dt) {
-        const int c = dt * 16 + col;
-        if (dt < dtn && c < DV) pr[c] = o[dt][reg];
-      }
-      if (col == 0) {
-        pr[DV] = m[reg];
-        pr[DV + 1] = ll;
-      }
-      continue;
     }
     const float inv = SIG ? 1.f : 1.f / ll;
 #pragma unroll
@@ -777,47 +746,8 @@ __global__ __launch_bounds__(256, 2) void chunk_bias_attn_prefill_mfma_kernel(
       const int c = dt * 16 + col;
       if (dt < dtn && c < DV)
         out[trow * out_stride + (long)h * DV + c] = __float2bfloat16(
-            o[dt][reg] * inv * (ps ? head_gate(gate, trow * g_stride, gate_cols, h, c)
-                                   : head_gate(gate, (long)b * g_stride, 1, r0 + r, c)));
+            o[dt][reg] * inv * head_gate(gate, trow * g_stride, gate_cols, h, c));
     }
-  }
-}
-
-// Merge of key splits: out[row, head] = sum_s o_s e^(m_s - M) / sum_s l_s e^(m_s - M),
-// M = max_s m_s; a split that saw no key has m = -inf and counts nothing. A
-// sink joins as one more l; rows are the hps query heads of one sequence each
-// (sink [hps], gate [sequence, hps]). One wave per (row, head), lanes over
-// value channels.
-__global__ __launch_bounds__(256) void attn_merge_splits_kernel(
-    __hip_bfloat16* __restrict__ out, long out_stride, const float* __restrict__ part,
-    long pairs, int H, int DV, int n_split, const float* __restrict__ sink,
-    const __hip_bfloat16* __restrict__ gate, long g_stride, int hps) {
-  const long pair = blockIdx.x * 4L + (threadIdx.x >> 6);
-  if (pair >= pairs) return;
-  const int lane = threadIdx.x & 63;
-  const float* pp = part + pair * n_split * (long)(DV + 2);
-  float M = -INFINITY;
-  for (int sidx = 0; sidx < n_split; ++sidx) M = fmaxf(M, pp[sidx * (DV + 2) + DV]);
-  const long row = pair / H;
-  const int h = (int)(pair % H);
-  float L = 0.f;
-  if (sink) {
-    const float sk = sink[row % hps];
-    M = fmaxf(M, sk);
-    L = expf(sk - M);
-  }
-  for (int sidx = 0; sidx < n_split; ++sidx) {
-    const float ms = pp[sidx * (DV + 2) + DV];
-    if (ms > -INFINITY) L += pp[sidx * (DV + 2) + DV + 1] * expf(ms - M);
-  }
-  const float gs = head_gate(gate, (row / hps) * g_stride, 1, (int)(row % hps), 0) / L;
-  for (int c = lane; c < DV; c += 64) {
-    float a = 0.f;
-    for (int sidx = 0; sidx < n_split; ++sidx) {
-      const float ms = pp[sidx * (DV + 2) + DV];
-      if (ms > -INFINITY) a += pp[sidx * (DV + 2) + c] * expf(ms - M);
-    }
-    out[row * out_stride + (long)h * DV + c] = __float2bfloat16(a * gs);
   }
 }
 

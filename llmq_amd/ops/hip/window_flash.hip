@@ -254,3 +254,251 @@ __global__ __launch_bounds__(256, (KS <= 8 ? 2 : 1)) void window_flash_kernel(
       *reinterpret_cast<int2*>(orow + c) = *reinterpret_cast<const int2*>(v.data);
     }
 }
+
+// ------------------------------------------------------------ single tokens --
+// The same attention for one new token per sequence: the query heads that share
+// a kv head (16 at a time) are the columns of S^T = K Q^T and O^T = V^T P^T on
+// v_mfma_f32_16x16x32_bf16 (A: row = lane%16, k = 8*(lane/16)..+7; B: column =
+// lane%16; C: column = lane%16, rows 4*(lane/16)+r), so every key row is read
+// once for all of them. Slot order of a 32-key step: slot 8 h + 4 b + i = key
+// 16 b + 4 h + i.
+//
+// Waves are independent: each takes every (4 * n_split)-th tile of 16 NK keys, K
+// operands straight from memory, V through a wave-private transposed LDS tile,
+// the next tile's rows in flight during the current tile's products. The four
+// waves' partials merge through LDS; with n_split > 1 a workgroup writes its
+// unnormalised output, maximum (natural log domain) and sum to `part`
+// [sequence, head, split, DV + 2] for attn_merge_splits_kernel.
+constexpr size_t window_decode_lds(int dt, int nk) {
+  const size_t tiles = 4 * sizeof(short) * (size_t)dt * 16 * (nk * 16 + 8);
+  const size_t merge = 4 * sizeof(float) * (size_t)16 * (dt * 16 + 2);
+  return tiles > merge ? tiles : merge;
+}
+
+// KS: key channels padded to 32 KS; DT: value channels padded to 16 DT.
+template <int KS, int DT, int NK>
+__global__ __launch_bounds__(256, (KS <= 4 ? 2 : 1)) void window_decode_kernel(
+    __hip_bfloat16* __restrict__ out, long out_stride,
+    const __hip_bfloat16* __restrict__ q, long q_stride,
+    const __hip_bfloat16* __restrict__ gate, long g_stride, int gate_cols,
+    const __hip_bfloat16* __restrict__ k_cache, const __hip_bfloat16* __restrict__ v_cache,
+    int v_row, const int* __restrict__ block_tables, int bt_stride,
+    const int* __restrict__ context_lens, int H, int G, int D, int DV, int bs_shift, int window,
+    float scale_log2, const float* __restrict__ sink, int n_split, float* __restrict__ part) {
+  extern __shared__ __align__(16) unsigned char wd_smem[];
+  constexpr int KT = 16 * NK, KP = KT + 8;
+  constexpr int KG = KT / 4, GW = 64 / KG;               // key groups and granules of a V task
+  constexpr int NV = (DT * 2 + GW - 1) / GW;             // V tasks per lane
+  const int hp = H / G, ng = (hp + 15) / 16;
+  const int sp = blockIdx.x % n_split, grp = blockIdx.x / n_split;
+  const int g = grp / ng, c0 = (grp % ng) * 16;          // kv head, its first query head here
+  const int heads = min(16, hp - c0), h0 = g * hp + c0;
+  const int b = blockIdx.y;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int col = lane & 15, grp4 = lane >> 4;
+  short* Vt = reinterpret_cast<short*>(wd_smem) + w * (DT * 16 * KP);    // [16 DT][KP]
+  const int pos = context_lens[b] - 1;
+  const int lo = max(0, pos - window + 1);
+  const int* bt = block_tables + (long)b * bt_stride;
+  const int bs_mask = (1 << bs_shift) - 1;
+  const wf_bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
+  wf_bf16x8 qf[KS];
+  {
+    const __hip_bfloat16* qr = q + (long)b * q_stride + (long)(h0 + col) * D;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int d8 = ks * 32 + grp4 * 8;
+      qf[ks] = col < heads && d8 < D ? *reinterpret_cast<const wf_bf16x8*>(qr + d8) : zero8;
+    }
+  }
+  const int sg = lane % GW, kg = lane / GW;
+  const int kpos = (kg >> 3) * 32 + (kg & 3) * 8 + ((kg >> 2) & 1) * 4;
+  auto row_of = [&](int key) -> long {
+    return (((long)bt[key >> bs_shift] * G + g) << bs_shift) + (key & bs_mask);
+  };
+  wf_bf16x8 kf[NK][KS], vf[NV][4];
+  auto fetch = [&](int kt) {
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int key = kt + i * 16 + col;
+      const bool live = key <= pos;
+      const __hip_bfloat16* kr = k_cache + (live ? row_of(key) : 0L) * D;
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const int d8 = ks * 32 + grp4 * 8;
+        kf[i][ks] = live && d8 < D ? *reinterpret_cast<const wf_bf16x8*>(kr + d8) : zero8;
+      }
+    }
+    const int key = kt + kg * 4;
+    const __hip_bfloat16* vr = v_cache + (key <= pos ? row_of(key) : 0L) * v_row;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int d8 = (i * GW + sg) * 8;
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        vf[i][e] = d8 < DV && key + e <= pos
+            ? *reinterpret_cast<const wf_bf16x8*>(vr + (long)e * v_row + d8) : zero8;
+    }
+  };
+  float m = -INFINITY, l = 0.f;              // log2 domain
+  sm_f32x4 o[DT];
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt) o[dt] = sm_f32x4{0.f, 0.f, 0.f, 0.f};
+  const int step = KT * 4 * n_split;
+  int kt = (lo / KT) * KT + (sp * 4 + w) * KT;
+  if (kt <= pos) fetch(kt);
+  for (; kt <= pos; kt += step) {
+    sm_f32x4 s[NK];
+#pragma unroll
+    for (int i = 0; i < NK; ++i) s[i] = sm_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks)
+#pragma unroll
+      for (int i = 0; i < NK; ++i)
+        s[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i][ks], qf[ks], s[i], 0, 0, 0);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int d8 = (i * GW + sg) * 8;
+      if (d8 < DV) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          wf_u32x2 v4;
+          v4[0] = (unsigned)(unsigned short)vf[i][0][j] | ((unsigned)(unsigned short)vf[i][1][j] << 16);
+          v4[1] = (unsigned)(unsigned short)vf[i][2][j] | ((unsigned)(unsigned short)vf[i][3][j] << 16);
+          *reinterpret_cast<wf_u32x2*>(Vt + (d8 + j) * KP + kpos) = v4;
+        }
+      }
+    }
+    if (kt + step <= pos) fetch(kt + step);
+    if (kt < lo || kt + KT - 1 > pos) {
+#pragma unroll
+      for (int i = 0; i < NK; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int key = kt + i * 16 + grp4 * 4 + r;
+          s[i][r] = key >= lo && key <= pos ? s[i][r] : -INFINITY;
+        }
+    }
+    float tmax = s[0][0];
+#pragma unroll
+    for (int i = 0; i < NK; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) tmax = fmaxf(tmax, s[i][r]);
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, WAVE));
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, WAVE));
+    const float m_new = fmaxf(m, tmax * scale_log2);         // scale > 0
+    const float mb = m_new > -INFINITY ? m_new : 0.f;
+    const float alpha = __builtin_amdgcn_exp2f(m - mb);      // m = -inf -> 0
+    l *= alpha;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) o[dt] *= alpha;
+    m = m_new;
+    // the tile's writes come before its reads: one wave, LDS in order
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int j = 0; j < NK / 2; ++j) {       // 32 keys per step
+      wf_u32x4 hi, lw;
+#pragma unroll
+      for (int e = 0; e < 8; e += 2) {
+        const float p0 = __builtin_amdgcn_exp2f(fmaf(s[2 * j + e / 4][e % 4], scale_log2, -mb));
+        const float p1 = __builtin_amdgcn_exp2f(fmaf(s[2 * j + e / 4][e % 4 + 1], scale_log2, -mb));
+        l += p0 + p1;
+        const unsigned b0 = __float_as_uint(p0), b1 = __float_as_uint(p1);
+        hi[e / 2] = __builtin_amdgcn_perm(b1, b0, 0x07060302u);
+        const wf_f32x2 rest = {p0 - __uint_as_float(b0 & 0xffff0000u),
+                               p1 - __uint_as_float(b1 & 0xffff0000u)};
+        lw[e / 2] = __builtin_bit_cast(unsigned, __builtin_convertvector(rest, wf_bfx2));
+      }
+      const wf_bf16x8 ph = __builtin_bit_cast(wf_bf16x8, hi), pl = __builtin_bit_cast(wf_bf16x8, lw);
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) {
+        const wf_bf16x8 va = *reinterpret_cast<const wf_bf16x8*>(
+            Vt + (dt * 16 + col) * KP + j * 32 + grp4 * 8);
+        o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, ph, o[dt], 0, 0, 0);
+        o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, pl, o[dt], 0, 0, 0);
+      }
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+  }
+  l += __shfl_xor(l, 16, WAVE);
+  l += __shfl_xor(l, 32, WAVE);
+  // merge of the four waves: [wave][column][DV, m, l] fp32 over the V tiles
+  __syncthreads();
+  float* Mg = reinterpret_cast<float*>(wd_smem);
+  constexpr int MW = DT * 16 + 2;
+  float* mine = Mg + (w * 16 + col) * MW;
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) mine[dt * 16 + grp4 * 4 + r] = o[dt][r];
+  if (grp4 == 0) {
+    mine[DT * 16] = m;
+    mine[DT * 16 + 1] = l;
+  }
+  __syncthreads();
+  for (int idx = tid; idx < heads * DV; idx += 256) {
+    const int hh = idx / DV, c = idx % DV, h = h0 + hh;
+    const float* pw = Mg + hh * MW;
+    float top = -INFINITY;
+#pragma unroll
+    for (int ww = 0; ww < 4; ++ww) top = fmaxf(top, pw[ww * 16 * MW + DT * 16]);
+    const float sk = sink && n_split == 1 ? sink[h] * 1.44269504088896340736f : -INFINITY;
+    top = fmaxf(top, sk);
+    const float tb = top > -INFINITY ? top : 0.f;
+    float a = 0.f, ll = __builtin_amdgcn_exp2f(sk - tb);
+#pragma unroll
+    for (int ww = 0; ww < 4; ++ww) {
+      const float f = __builtin_amdgcn_exp2f(pw[ww * 16 * MW + DT * 16] - tb);
+      a += pw[ww * 16 * MW + c] * f;
+      ll += pw[ww * 16 * MW + DT * 16 + 1] * f;
+    }
+    if (n_split > 1) {
+      float* pr = part + (((long)b * H + h) * n_split + sp) * (DV + 2);
+      pr[c] = a;
+      if (c == 0) {
+        pr[DV] = top * 0.69314718055994530942f;
+        pr[DV + 1] = ll;
+      }
+    } else {
+      out[(long)b * out_stride + (long)h * DV + c] = __float2bfloat16(
+          a / ll * head_gate(gate, (long)b * g_stride, gate_cols, h, c));
+    }
+  }
+}
+
+// Merge of key splits: out[b, h] = sum_s o_s e^(m_s - M) / sum_s l_s e^(m_s - M),
+// M = max_s m_s, a sink joining as one more l; a split that saw no key has
+// m = -inf and counts nothing. One wave per (sequence, head), lanes over value
+// channels.
+__global__ __launch_bounds__(256) void attn_merge_splits_kernel(
+    __hip_bfloat16* __restrict__ out, long out_stride, const float* __restrict__ part,
+    long pairs, int H, int DV, int n_split, const float* __restrict__ sink,
+    const __hip_bfloat16* __restrict__ gate, long g_stride, int gate_cols) {
+  const long pair = blockIdx.x * 4L + (threadIdx.x >> 6);
+  if (pair >= pairs) return;
+  const int lane = threadIdx.x & 63;
+  const long b = pair / H;
+  const int h = (int)(pair % H);
+  const float* pp = part + pair * n_split * (long)(DV + 2);
+  // a lane reads one split's maximum and sum (at most 64 splits)
+  const float ms = lane < n_split ? pp[lane * (DV + 2) + DV] : -INFINITY;
+  const float ls = lane < n_split ? pp[lane * (DV + 2) + DV + 1] : 0.f;
+  float M = wave_reduce_max(ms);
+  if (sink) M = fmaxf(M, sink[h]);
+  const float f = ms > -INFINITY ? expf(ms - M) : 0.f;
+  const float L = wave_reduce_sum(ls * f) + (sink ? expf(sink[h] - M) : 0.f);
+  const float inv = 1.0f / L;
+  for (int c = lane; c - lane < DV; c += 64) {      // all lanes stay for the shuffles
+    float a = 0.f;
+    for (int s = 0; s < n_split; ++s) {
+      const float fs = __shfl(f, s, WAVE);
+      if (c < DV) a += pp[s * (DV + 2) + c] * fs;
+    }
+    if (c < DV)
+      out[b * out_stride + (long)h * DV + c] =
+          __float2bfloat16(a * inv * head_gate(gate, b * g_stride, gate_cols, h, c));
+  }
+}
