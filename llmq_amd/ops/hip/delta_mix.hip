@@ -208,7 +208,7 @@ __global__ __launch_bounds__(256) void gated_delta_kernel(
           const int i = g * GW + e;
 #pragma unroll
           for (int c = 0; c < NC; ++c) {
-            S[c][i] *= ga[e];
+            if constexpr (!HEAD_DECAY) S[c][i] *= ga[e];
             pk[c] += S[c][i] * kk[i];
             pq[c] += S[c][i] * qa[e];
           }
@@ -218,13 +218,16 @@ __global__ __launch_bounds__(256) void gated_delta_kernel(
       float u[NC];
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
-        u[c] = bt * (vs[tt * COLS + lc + c] - row16_sum(pk[c]));
-        pq[c] = row16_sum(pq[c]) + kqt * u[c];
+        // one decay per head: it comes out of both products, and the state takes
+        // it together with the write
+        u[c] = bt * (vs[tt * COLS + lc + c] - gh * row16_sum(pk[c]));
+        pq[c] = gh * row16_sum(pq[c]) + kqt * u[c];
       }
 #pragma unroll
       for (int i = 0; i < DPL; ++i)
 #pragma unroll
-        for (int c = 0; c < NC; ++c) S[c][i] += kk[i] * u[c];
+        for (int c = 0; c < NC; ++c)
+          S[c][i] = (HEAD_DECAY ? gh * S[c][i] : S[c][i]) + kk[i] * u[c];
       if (l == 0) {
         float* op = o + ((long)(row0 + t0 + tt) * H + h) * DV + c0;
         if (vec_cols) {

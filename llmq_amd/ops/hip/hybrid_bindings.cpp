@@ -424,13 +424,13 @@ void paged_attn_decode(at::Tensor out, at::Tensor q, const std::optional<at::Ten
       flash_takes(a, out, q, k_cache, mask_mode, scale)) {
     using bf = __hip_bfloat16;
     const int groups = a.G * ((a.H / a.G + 15) / 16);
-    // keys split over workgroups until the grid has about two per CU and wave
-    // tiles still to hand out
+    // keys split over workgroups until the chip is full (two workgroups per CU,
+    // of the wide-row kernels' registers one) and wave tiles still to hand out
     const long keys = std::min<long>(span, block_tables.size(1) * (long)a.bs);
     auto launch = [&]<int KS, int DT, int NK>() {
       const long wave_tiles = (keys + 16 * NK - 1) / (16 * NK) + 1;
       const int n_split = (int)std::max<long>(1, std::min<long>(
-          std::min<long>(64, (wave_tiles + 3) / 4), 512 / ((long)groups * B)));
+          std::min<long>(64, (wave_tiles + 3) / 4), (KS <= 4 ? 512 : 256) / ((long)groups * B)));
       at::Tensor part;
       if (n_split > 1) part = at::empty({B, a.H, n_split, a.DV + 2}, q.options().dtype(at::kFloat));
       constexpr size_t lds = window_decode_lds(DT, NK);
